@@ -327,6 +327,48 @@ int rb_attention_decode_bf16_opts(const void* q, const void* k_pages, const void
                                   const int32_t* tok_pos, const int32_t* block_table, int bt_stride, int n_seqs,
                                   int n_heads, int n_kv_heads, int head_dim, float scale, int window, int keep_first,
                                   float softcap, int n_splits, float* workspace, const float* sinks, void* stream);
+// The three of them with chunks and sigmoid weights.  chunk > 0: a query at position i sees the keys j <= i with
+// i / chunk == j / chunk only (0: no chunks).  sig_bias (float32 [Hq], null: softmax): a visible key's weight is
+// sigmoid(score + sig_bias[h]), not normalised over the keys; goes without sinks.
+int rb_attention_generic_chunked(const void* q, const void* k_pages, const void* v_pages, void* out, int dtype,
+                                 const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* block_table, int bt_stride,
+                                 int n_tokens, int n_heads, int n_kv_heads, int head_dim, float scale, int window, int keep_first,
+                                 float softcap, const float* sinks, int chunk, const float* sig_bias, void* stream);
+int rb_attention_prefill_bf16_chunked(const void* q, const void* k_pages, const void* v_pages, void* out,
+                                      const int32_t* cu_seqlens, const int32_t* past_len, const int32_t* block_table, int bt_stride,
+                                      int n_seqs, int max_q_len, int n_heads, int n_kv_heads, int head_dim, float scale, int window,
+                                      int keep_first, float softcap, const float* sinks, int chunk, const float* sig_bias,
+                                      void* stream);
+int rb_attention_decode_bf16_chunked(const void* q, const void* k_pages, const void* v_pages, void* out, const int32_t* tok_pos,
+                                     const int32_t* block_table, int bt_stride, int n_seqs, int n_heads, int n_kv_heads, int head_dim,
+                                     float scale, int window, int keep_first, float softcap, int n_splits, float* workspace,
+                                     const float* sinks, int chunk, const float* sig_bias, void* stream);
+// rb_rope_store with norms over the whole projections in front of the rotation: q (all Hq * dim numbers together) divided by its
+// root mean square and multiplied by q_norm [Hq * dim], k likewise by k_norm [Hk * dim] (both null: neither); either pairing
+// (style 0: 2i with 2i + 1, 1: i with i + rot / 2); value_norm != 0: every value head divided by its own root mean square.
+int rb_heads_prepare(const float* qkv, long long row_width, const float* cos, const float* sin, int rot, int style, const float* q_norm,
+                     const float* k_norm, int value_norm, float eps, void* q_out, void* k_pages, void* v_pages, int cache_dtype,
+                     const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* block_table, int bt_stride, int n_tokens,
+                     int n_heads, int n_kv_heads, int dim, int vdim, int pad, void* stream);
+// tanh(alpha v) w + b as a norm, on a sublayer's output and in front of the next sublayer, in one pass over the stream's rows:
+//   v = x[src] + (a1 ? tanh(a1 y) w1 + b1 : y);  without rows x[src] = v;  out[r] = tanh(a2 v) w2 + b2,  src = rows ? rows[r] : r
+// with y[src] = sum_k (weights ? weights[src * n_terms + k] : 1) y[src * row_stride + k * term_stride].  y null: nothing is
+// added; out null: no rows.  The alphas are numbers in device memory.
+int rb_tanh_norm(float* x, const float* y, int n_terms, long long term_stride, long long row_stride, const float* weights,
+                 const float* a1, const float* w1, const float* b1, const float* a2, const float* w2, const float* b2,
+                 const int32_t* rows, int n_rows, int width, void* out, int out_dtype, void* stream);
+// The plain rule of rb_linear_recurrence with one constant decay per head (decay float32 [H]) and silu on q, k, v as they are read.
+int rb_lightning_recurrence(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride, const float* decay,
+                            float* state, const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs, int n_tokens,
+                            int n_heads, int dim, int vdim, void* stream);
+// rb_gated_rmsnorm_act with ONE norm over the whole row (all heads together); weight [width].
+int rb_gated_rmsnorm_rows(const float* o, const float* weight, const float* gate, long long gate_stride, int act, float eps, void* out,
+                          int out_dtype, int n_tokens, int width, void* stream);
+// rb_route_choose with a bias on the router's logits (float32 [n_outputs], null: none) and a third score, 2: the choice by the
+// logits, the weights the softmax over the chosen logits alone (top <= 64).
+int rb_route_choose_bias(const float* z, long long z_stride, const float* bias, int n_outputs, int n_experts, int top, int score,
+                         const float* correction, int32_t* sel, float* weight, int32_t* row_pair, int32_t* tile_expert, int max_rows,
+                         int n_tokens, void* stream);
 // rb_rope_store with every query and key head RMS-normed first over its dim numbers, x / sqrt(mean(x^2) + eps) * w, with a
 // weight of dim numbers that the heads share (q_norm, k_norm float32 [dim]).
 int rb_norm_rope_store(const float* qkv, long long row_width, const float* cos, const float* sin, int rot, const float* q_norm,

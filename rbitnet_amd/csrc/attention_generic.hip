@@ -25,7 +25,7 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_kern
     const T* __restrict__ q, const T* __restrict__ k_pages, const T* __restrict__ v_pages, T* __restrict__ out,
     const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
     const int32_t* __restrict__ block_table, int bt_stride, int n_heads, int n_kv, int head_dim, float scale,
-    int window, const float* __restrict__ sinks, int keep_first, float softcap) {
+    int window, const float* __restrict__ sinks, int keep_first, float softcap, int chunk, const float* __restrict__ sig_bias) {
   __shared__ float qs[AG_MAX_D];
   __shared__ float ps_all[AG_MAX_WAVES][RB_PAGE];
   __shared__ float red_m[AG_MAX_WAVES], red_l[AG_MAX_WAVES];
@@ -37,14 +37,17 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_kern
   float* ps = ps_all[wave];
   const int pos = tok_pos[t];
   const int kvh = h / (n_heads / n_kv);
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_visible(pos, window, chunk);
   const int32_t* pages = block_table + (size_t)tok_seq[t] * bt_stride;
 
   const T* qrow = q + ((size_t)t * n_heads + h) * head_dim;
   for (int d = threadIdx.x; d < head_dim; d += blockDim.x) qs[d] = Num<T>::load(qrow + d);
   __syncthreads();
 
-  float m_run = -INFINITY, l_run = 0.f;
+  // sigmoid weights (sig_bias): a key's weight is sigmoid(score + sig_bias[h]) by itself, so the maximum stays 0, nothing is
+  // rescaled and nothing divided
+  const float sb = sig_bias ? sig_bias[h] : 0.f;
+  float m_run = sig_bias ? 0.f : -INFINITY, l_run = 0.f;
   float acc[AG_MAX_D / RB_WAVE];
 #pragma unroll
   for (int i = 0; i < AG_MAX_D / RB_WAVE; ++i) acc[i] = 0.f;
@@ -67,8 +70,8 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_kern
       s = dot * scale;
       if (softcap > 0.f) s = softcap * tanhf(s / softcap);
     }
-    const float m_new = fmaxf(m_run, wave_max(s));      // finite: the page holds at least one valid key
-    const float pexp = (s == -INFINITY) ? 0.f : expf(s - m_new);
+    const float m_new = sig_bias ? 0.f : fmaxf(m_run, wave_max(s));      // finite: the page holds at least one valid key
+    const float pexp = (s == -INFINITY) ? 0.f : (sig_bias ? 1.0f / (1.0f + expf(-(s + sb))) : expf(s - m_new));
     const float corr = (m_run == -INFINITY) ? 0.f : expf(m_run - m_new);
     l_run = l_run * corr + wave_sum(pexp);
     m_run = m_new;
@@ -118,7 +121,7 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_kern
     }
   }
   if (sinks) l_run += expf(sinks[h] - m_run);          // a term of the denominator with no key and no value
-  const float inv = l_run > 0.f ? 1.0f / l_run : 0.f;
+  const float inv = sig_bias ? 1.0f : (l_run > 0.f ? 1.0f / l_run : 0.f);
   T* orow = out + ((size_t)t * n_heads + h) * head_dim;
 #pragma unroll
   for (int i = 0; i < AG_MAX_D / RB_WAVE; ++i) {
@@ -154,7 +157,8 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_vec_
     const T* __restrict__ q, const T* __restrict__ k_pages, const T* __restrict__ v_pages, T* __restrict__ out,
     const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
     const int32_t* __restrict__ block_table, int bt_stride, int n_heads, int n_kv, int head_dim, float scale,
-    int window, int group_lanes, const float* __restrict__ sinks, int keep_first, float softcap) {
+    int window, int group_lanes, const float* __restrict__ sinks, int keep_first, float softcap, int chunk,
+    const float* __restrict__ sig_bias) {
   __shared__ __attribute__((aligned(16))) float qs[AG_MAX_D];
   __shared__ float ps_all[AG_MAX_WAVES][RB_PAGE];
   __shared__ float red_m[AG_MAX_WAVES], red_l[AG_MAX_WAVES];
@@ -166,7 +170,7 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_vec_
   float* ps = ps_all[wave];
   const int pos = tok_pos[t];
   const int kvh = h / (n_heads / n_kv);
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_visible(pos, window, chunk);
   const int32_t* pages = block_table + (size_t)tok_seq[t] * bt_stride;
   const int chunks = head_dim / 4;
   const int c = lane % group_lanes, g = lane / group_lanes, n_groups = RB_WAVE / group_lanes;
@@ -176,7 +180,10 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_vec_
   for (int d = threadIdx.x; d < head_dim; d += blockDim.x) qs[d] = Num<T>::load(qrow + d);
   __syncthreads();
 
-  float m_run = -INFINITY, l_run = 0.f;
+  // sigmoid weights (sig_bias): a key's weight is sigmoid(score + sig_bias[h]) by itself, so the maximum stays 0, nothing is
+  // rescaled and nothing divided
+  const float sb = sig_bias ? sig_bias[h] : 0.f;
+  float m_run = sig_bias ? 0.f : -INFINITY, l_run = 0.f;
   float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
   // the pages that hold visible keys: those of the kept first tokens that lie before the window's first page, then the
   // window's (every one of them holds at least one visible key)
@@ -203,8 +210,8 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_vec_
       s = ((d0 + d1) + (d2 + d3)) * scale;
       if (softcap > 0.f) s = softcap * tanhf(s / softcap);
     }
-    const float m_new = fmaxf(m_run, wave_max(s));      // finite: the page holds at least one valid key
-    const float pexp = (s == -INFINITY) ? 0.f : expf(s - m_new);
+    const float m_new = sig_bias ? 0.f : fmaxf(m_run, wave_max(s));      // finite: the page holds at least one valid key
+    const float pexp = (s == -INFINITY) ? 0.f : (sig_bias ? 1.0f / (1.0f + expf(-(s + sb))) : expf(s - m_new));
     const float corr = (m_run == -INFINITY) ? 0.f : expf(m_run - m_new);
     l_run = l_run * corr + wave_sum(pexp);
     m_run = m_new;
@@ -264,7 +271,7 @@ __global__ __launch_bounds__(RB_WAVE * AG_MAX_WAVES) void attention_generic_vec_
   }
   if (owner) {
     if (sinks) l_run += expf(sinks[h] - m_run);        // a term of the denominator with no key and no value
-    const float inv = l_run > 0.f ? 1.0f / l_run : 0.f;
+    const float inv = sig_bias ? 1.0f : (l_run > 0.f ? 1.0f / l_run : 0.f);
     T* orow = out + ((size_t)t * n_heads + h) * head_dim + 4 * c;
     Num<T>::store(orow + 0, acc.x * inv);
     Num<T>::store(orow + 1, acc.y * inv);
@@ -306,7 +313,23 @@ extern "C" int rb_attention_generic_opts(const void* q, const void* k_pages, con
                                          void* stream) {
   RB_RECORDED(rb_attention_generic_opts(q, k_pages, v_pages, out, dtype, tok_pos, tok_seq, block_table, bt_stride, n_tokens,
                                         n_heads, n_kv_heads, head_dim, scale, window, keep_first, softcap, sinks, stream));
-  RB_REQUIRE(keep_first >= 0 && softcap >= 0.f, "rb_attention_generic: negative keep_first or softcap");
+  return rb_attention_generic_chunked(q, k_pages, v_pages, out, dtype, tok_pos, tok_seq, block_table, bt_stride, n_tokens, n_heads,
+                                      n_kv_heads, head_dim, scale, window, keep_first, softcap, sinks, 0, nullptr, stream);
+}
+
+// The same with two more.  chunk > 0: a query at position i sees the keys j <= i with i / chunk == j / chunk only (beside
+// what the window says).  sig_bias (float32 [Hq], null: softmax): a visible key's weight is sigmoid(score + sig_bias[h]), and
+// the weights are not normalised over the keys (a sink then has no meaning and must be null).
+extern "C" int rb_attention_generic_chunked(const void* q, const void* k_pages, const void* v_pages, void* out, int dtype,
+                                            const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* block_table,
+                                            int bt_stride, int n_tokens, int n_heads, int n_kv_heads, int head_dim,
+                                            float scale, int window, int keep_first, float softcap, const float* sinks, int chunk,
+                                            const float* sig_bias, void* stream) {
+  RB_RECORDED(rb_attention_generic_chunked(q, k_pages, v_pages, out, dtype, tok_pos, tok_seq, block_table, bt_stride, n_tokens,
+                                           n_heads, n_kv_heads, head_dim, scale, window, keep_first, softcap, sinks, chunk, sig_bias,
+                                           stream));
+  RB_REQUIRE(keep_first >= 0 && softcap >= 0.f && chunk >= 0, "rb_attention_generic: negative keep_first, softcap or chunk");
+  RB_REQUIRE(sig_bias == nullptr || sinks == nullptr, "rb_attention_generic: a sink belongs to the softmax");
   RB_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0,
              "rb_attention_generic: bad head counts Hq=%d Hk=%d", n_heads, n_kv_heads);
   RB_REQUIRE(head_dim > 0 && head_dim <= AG_MAX_D, "rb_attention_generic: head_dim %d not supported (at most %d)", head_dim,
@@ -328,12 +351,14 @@ extern "C" int rb_attention_generic_opts(const void* q, const void* k_pages, con
       attention_generic_vec_kernel<float><<<grid, threads, 0, s>>>((const float*)q, (const float*)k_pages,
                                                                   (const float*)v_pages, (float*)out, tok_pos, tok_seq,
                                                                   block_table, bt_stride, n_heads, n_kv_heads, head_dim,
-                                                                  scale, window, group_lanes, sinks, keep_first, softcap);
+                                                                  scale, window, group_lanes, sinks, keep_first, softcap,
+                                                                  chunk, sig_bias);
     else
       attention_generic_vec_kernel<bf16_t><<<grid, threads, 0, s>>>((const bf16_t*)q, (const bf16_t*)k_pages,
                                                                    (const bf16_t*)v_pages, (bf16_t*)out, tok_pos,
                                                                    tok_seq, block_table, bt_stride, n_heads, n_kv_heads,
-                                                                   head_dim, scale, window, group_lanes, sinks, keep_first, softcap);
+                                                                   head_dim, scale, window, group_lanes, sinks, keep_first, softcap, chunk,
+                                                                   sig_bias);
     RB_LAUNCH_CHECK();
     return 0;
   }
@@ -341,12 +366,12 @@ extern "C" int rb_attention_generic_opts(const void* q, const void* k_pages, con
     attention_generic_kernel<float><<<grid, threads, 0, s>>>((const float*)q, (const float*)k_pages,
                                                             (const float*)v_pages, (float*)out, tok_pos, tok_seq,
                                                             block_table, bt_stride, n_heads, n_kv_heads, head_dim,
-                                                            scale, window, sinks, keep_first, softcap);
+                                                            scale, window, sinks, keep_first, softcap, chunk, sig_bias);
   else if (dtype == RB_BF16)
     attention_generic_kernel<bf16_t><<<grid, threads, 0, s>>>((const bf16_t*)q, (const bf16_t*)k_pages,
                                                              (const bf16_t*)v_pages, (bf16_t*)out, tok_pos,
                                                              tok_seq, block_table, bt_stride, n_heads, n_kv_heads,
-                                                             head_dim, scale, window, sinks, keep_first, softcap);
+                                                             head_dim, scale, window, sinks, keep_first, softcap, chunk, sig_bias);
   else
     RB_REQUIRE(false, "rb_attention_generic: unknown dtype %d", dtype);
   RB_LAUNCH_CHECK();

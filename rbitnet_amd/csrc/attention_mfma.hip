@@ -24,12 +24,15 @@
 #define LOG2E 1.4426950408889634f
 
 // =============================================================================== prefill
-template <int D, int NW>
+template <int D, int NW, bool SIG>
 __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void attn_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     bf16_t* __restrict__ out, const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ past_len,
     const int32_t* __restrict__ block_table, int bt_stride, int n_heads, int n_kv, float scale_log2, int window,
-    int gw, int paired, const float* __restrict__ sinks, int keep_first, float cap, float cap_pre) {
+    int gw, int paired, const float* __restrict__ sinks, int keep_first, float cap, float cap_pre, int chunk,
+    const float* __restrict__ sig_bias) {
+  // chunk > 0: a query sees the keys of its own chunk of positions only.  SIG: a visible key's weight is
+  // sigmoid(score + sig_bias[head]), without maximum, sum or division.
   // keep_first (with a window): the sequence's first keep_first keys stay visible behind the window; the tiles that hold
   // them are walked first.  cap > 0: a raw score s becomes cap * tanh(s * cap_pre) (cap_pre = scale / cap) before the mask,
   // and scale_log2 is then log2(e) alone.
@@ -78,7 +81,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void attn_prefill_kernel(
   const bool q_ok = ql < q_len;
   if (ql >= q_len) ql = q_len - 1;
   const int qpos = past + ql;
-  const int q_lo = (window > 0 && qpos - window + 1 > 0) ? qpos - window + 1 : 0;
+  const int q_lo = first_visible(qpos, window, chunk);
   Frag8 qf[D / 16];
   {
     const bf16_t* qrow = q + ((size_t)(seq_start + ql) * n_heads + head) * D;
@@ -89,7 +92,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void attn_prefill_kernel(
   // ---- key tiles of the workgroup and of this wave
   const int wg_q_end = (wg_q0 + q_per_wg < q_len ? wg_q0 + q_per_wg : q_len) - 1;
   const int wg_min_pos = past + wg_q0;
-  const int wg_lo = (window > 0 && wg_min_pos - window + 1 > 0) ? wg_min_pos - window + 1 : 0;
+  const int wg_lo = first_visible(wg_min_pos, window, chunk);
   const int first_tile = wg_lo / RB_PAGE;
   const int last_tile = (past + wg_q_end) / RB_PAGE;
   const int kept_tiles = keep_first > 0 ? (keep_first + RB_PAGE - 1) / RB_PAGE : 0;
@@ -101,11 +104,12 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void attn_prefill_kernel(
     const int w_end = (q0 + 32 < q_len ? q0 + 32 : q_len) - 1;
     wave_last = (past + w_end) / RB_PAGE;
     const int w_min = past + q0;
-    wave_first = ((window > 0 && w_min - window + 1 > 0) ? w_min - window + 1 : 0) / RB_PAGE;
+    wave_first = first_visible(w_min, window, chunk) / RB_PAGE;
     wave_min_pos = w_min;
-    wave_max_lo = (window > 0 && past + w_end - window + 1 > 0) ? past + w_end - window + 1 : 0;
+    wave_max_lo = first_visible(past + w_end, window, chunk);
   }
 
+  const float nb = SIG ? -LOG2E * sig_bias[head] : 0.f;
   float m_run = -INFINITY, l_run = 0.f;
   f32x16_t oacc[D / 32];
 #pragma unroll
@@ -228,7 +232,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void attn_prefill_kernel(
     // ---- mask (only tiles that touch the diagonal or the window's edge), running maximum.
     // Scores stay unscaled: the scale is positive, so the maximum can be taken first and the
     // scale folded into the exponent's argument.
-    const bool edge = kept || (kt * RB_PAGE + RB_PAGE - 1 > wave_min_pos) || (window > 0 && kt * RB_PAGE < wave_max_lo);
+    const bool edge = kept || (kt * RB_PAGE + RB_PAGE - 1 > wave_min_pos) || (kt * RB_PAGE < wave_max_lo);
     float mx = -INFINITY;
     if (cap > 0.f) {
       // cap * tanh(x) as cap - 2 cap / (2^(2 x log2 e) + 1), on the hardware's exponential and reciprocal
@@ -239,15 +243,24 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void attn_prefill_kernel(
         for (int e = 0; e < 16; ++e)
           sacc[rt][e] = fmaf(-cap2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sacc[rt][e] * pre2) + 1.0f), cap);
     }
+    if (SIG) {
+      // 1 / (1 + 2^(-(score + bias) log2 e)) on the hardware's exponential and reciprocal
+#pragma unroll
+      for (int rt = 0; rt < 2; ++rt)
+#pragma unroll
+        for (int e = 0; e < 16; ++e)
+          sacc[rt][e] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(sacc[rt][e], -scale_log2, nb)));
+    }
     if (edge) {
 #pragma unroll
       for (int rt = 0; rt < 2; ++rt)
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
           const int key = kt * RB_PAGE + rt * 32 + 8 * (e / 4) + 4 * g + (e % 4);
-          if (key > qpos || (key < q_lo && key >= keep_first)) sacc[rt][e] = -INFINITY;
+          if (key > qpos || (key < q_lo && key >= keep_first)) sacc[rt][e] = SIG ? 0.f : -INFINITY;
         }
     }
+    if (!SIG) {
 #pragma unroll
     for (int rt = 0; rt < 2; ++rt)
 #pragma unroll
@@ -277,6 +290,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void attn_prefill_kernel(
     }
     l_run += lsum;
     m_run = m_new;
+    }
 
     // ---- O^T += V^T P^T.  Step (rt, mm) takes the 16 keys whose probabilities sit in
     // registers 8 mm .. 8 mm + 7 of row tile rt: for lane group g these are keys
@@ -304,8 +318,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void attn_prefill_kernel(
 
   if (!wave_on || !q_ok) return;
   // a sink: a term of the denominator with no key and no value, not scaled (m_run is in the exponent's base-2 units)
-  if (sinks) l_run += __builtin_amdgcn_exp2f(fmaf(sinks[head], LOG2E, -m_run));
-  const float inv = l_run > 0.f ? 1.0f / l_run : 0.f;
+  if (!SIG && sinks) l_run += __builtin_amdgcn_exp2f(fmaf(sinks[head], LOG2E, -m_run));
+  const float inv = SIG ? 1.0f : (l_run > 0.f ? 1.0f / l_run : 0.f);
   bf16_t* orow = out + ((size_t)(seq_start + ql) * n_heads + head) * D;
 #pragma unroll
   for (int i = 0; i < D / 32; ++i)
@@ -352,7 +366,24 @@ extern "C" int rb_attention_prefill_bf16_opts(const void* q, const void* k_pages
   RB_RECORDED(rb_attention_prefill_bf16_opts(q, k_pages, v_pages, out, cu_seqlens, past_len, block_table, bt_stride, n_seqs,
                                              max_q_len, n_heads, n_kv_heads, head_dim, scale, window, keep_first, softcap, sinks,
                                              stream));
-  RB_REQUIRE(keep_first >= 0 && softcap >= 0.f, "rb_attention_prefill_bf16: negative keep_first or softcap");
+  return rb_attention_prefill_bf16_chunked(q, k_pages, v_pages, out, cu_seqlens, past_len, block_table, bt_stride, n_seqs, max_q_len,
+                                           n_heads, n_kv_heads, head_dim, scale, window, keep_first, softcap, sinks, 0, nullptr,
+                                           stream);
+}
+
+// With chunks (a query sees the keys of its own chunk of positions only) and with sigmoid weights (sig_bias float32 [Hq]):
+// see rb_attention_generic_chunked.
+extern "C" int rb_attention_prefill_bf16_chunked(const void* q, const void* k_pages, const void* v_pages, void* out,
+                                                 const int32_t* cu_seqlens, const int32_t* past_len,
+                                                 const int32_t* block_table, int bt_stride, int n_seqs, int max_q_len,
+                                                 int n_heads, int n_kv_heads, int head_dim, float scale, int window,
+                                                 int keep_first, float softcap, const float* sinks, int chunk,
+                                                 const float* sig_bias, void* stream) {
+  RB_RECORDED(rb_attention_prefill_bf16_chunked(q, k_pages, v_pages, out, cu_seqlens, past_len, block_table, bt_stride, n_seqs,
+                                                max_q_len, n_heads, n_kv_heads, head_dim, scale, window, keep_first, softcap, sinks,
+                                                chunk, sig_bias, stream));
+  RB_REQUIRE(keep_first >= 0 && softcap >= 0.f && chunk >= 0, "rb_attention_prefill_bf16: negative keep_first, softcap or chunk");
+  RB_REQUIRE(sig_bias == nullptr || sinks == nullptr, "rb_attention_prefill_bf16: a sink belongs to the softmax");
   if (window == 0) keep_first = 0;
   RB_REQUIRE(n_seqs > 0 && max_q_len > 0, "rb_attention_prefill_bf16: empty batch");
   RB_REQUIRE(n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0,
@@ -378,17 +409,26 @@ extern "C" int rb_attention_prefill_bf16_opts(const void* q, const void* k_pages
   hipStream_t s = (hipStream_t)stream;
   const float sl2 = softcap > 0.f ? LOG2E : scale * LOG2E;
   const float cap_pre = softcap > 0.f ? scale / softcap : 0.f;
-#define RB_PF(DV, NWV)                                                                                          \
-  attn_prefill_kernel<DV, NWV><<<grid, 64 * NWV, 0, s>>>((const bf16_t*)q, (const bf16_t*)k_pages,              \
-                                                         (const bf16_t*)v_pages, (bf16_t*)out, cu_seqlens,      \
-                                                         past_len, block_table, bt_stride, n_heads, n_kv_heads, \
-                                                         sl2, window, gw, paired, sinks, keep_first, softcap, cap_pre)
-  if (head_dim == 128) {
-    if (nw == 8) RB_PF(128, 8);
-    else RB_PF(128, 4);
+#define RB_PF(DV, NWV, SIGV)                                                                                          \
+  attn_prefill_kernel<DV, NWV, SIGV><<<grid, 64 * NWV, 0, s>>>((const bf16_t*)q, (const bf16_t*)k_pages,              \
+                                                               (const bf16_t*)v_pages, (bf16_t*)out, cu_seqlens,      \
+                                                               past_len, block_table, bt_stride, n_heads, n_kv_heads, \
+                                                               sl2, window, gw, paired, sinks, keep_first, softcap,   \
+                                                               cap_pre, chunk, sig_bias)
+  if (sig_bias) {
+    if (head_dim == 128) {
+      if (nw == 8) RB_PF(128, 8, true);
+      else RB_PF(128, 4, true);
+    } else {
+      if (nw == 8) RB_PF(64, 8, true);
+      else RB_PF(64, 4, true);
+    }
+  } else if (head_dim == 128) {
+    if (nw == 8) RB_PF(128, 8, false);
+    else RB_PF(128, 4, false);
   } else {
-    if (nw == 8) RB_PF(64, 8);
-    else RB_PF(64, 4);
+    if (nw == 8) RB_PF(64, 8, false);
+    else RB_PF(64, 4, false);
   }
 #undef RB_PF
   RB_LAUNCH_CHECK();
@@ -713,13 +753,16 @@ __device__ __forceinline__ int v_swizzle(int key) {
   return D == 128 ? ((key & 7) << 1) : (((key >> 1) & 3) << 1);
 }
 
-template <int D, int NW, bool FUSED, int ONCE>
+template <int D, int NW, bool FUSED, int ONCE, bool SIG>
 __global__ __launch_bounds__(64 * NW) void attn_decode_mfma_kernel(
     const float* __restrict__ qkv, const bf16_t* __restrict__ q_in, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, int style, bf16_t* k_pages, bf16_t* v_pages, bf16_t* __restrict__ out,
     const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ block_table, int bt_stride, int n_heads,
     int n_kv, float scale_log2, int window, int n_splits, float* __restrict__ ws, int qkv_terms, size_t qkv_stride,
-    const float* __restrict__ sinks, int keep_first, float cap, float cap_pre, int kv_rep) {
+    const float* __restrict__ sinks, int keep_first, float cap, float cap_pre, int kv_rep, int chunk,
+    const float* __restrict__ sig_bias) {
+  // chunk > 0: the query sees the keys of its own chunk of positions only.  SIG: a visible key's weight is
+  // sigmoid(score + sig_bias[head]); the waves' and the splits' outputs are then simply added.
   // kv_rep > 1: n_kv counts every key/value head kv_rep times (head kvh reads the pages of head kvh / kv_rep), so that more
   // than 16 query heads on one key/value head run as several groups of at most 16.
   // keep_first (with a window): the first keep_first keys stay visible behind the window; their pages are walked before the
@@ -747,7 +790,7 @@ __global__ __launch_bounds__(64 * NW) void attn_decode_mfma_kernel(
   const int split = blockIdx.x, kvh = blockIdx.y, b = blockIdx.z;
   const int G = n_heads / n_kv;
   const int pos = tok_pos[b];
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_visible(pos, window, chunk);
   const int first_page = lo / RB_PAGE, last_page = pos / RB_PAGE;
   const int32_t* pages = block_table + (size_t)b * bt_stride;
   // the pages are walked by a running number: those of kept keys that lie before the window's first page, then the window's
@@ -846,7 +889,8 @@ __global__ __launch_bounds__(64 * NW) void attn_decode_mfma_kernel(
 #pragma unroll
   for (int st = 0; st < KS; ++st) qf[st].u = *reinterpret_cast<const uint4*>(q_h + c16 * D + 32 * st + 8 * grp);
 
-  float m_run = -INFINITY, l_part = 0.f;
+  const float nb = (SIG && c16 < G) ? -LOG2E * sig_bias[kvh * G + c16] : 0.f;
+  float m_run = SIG ? 0.f : -INFINITY, l_part = 0.f;
   f32x4_t acc_o[DT];
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) acc_o[dt] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
@@ -904,10 +948,16 @@ __global__ __launch_bounds__(64 * NW) void attn_decode_mfma_kernel(
         float raw = sc[t][i];
         if (cap > 0.f)      // cap * tanh(x) as cap - 2 cap / (2^(2 x log2 e) + 1)
           raw = fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(raw * (2.0f * LOG2E * cap_pre)) + 1.0f), cap);
-        const float v = (key <= pos && (key >= lo || key < keep_first)) ? raw * scale_log2 : -INFINITY;
+        const bool seen = key <= pos && (key >= lo || key < keep_first);
+        if constexpr (SIG) {
+          sc[t][i] = seen ? __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(raw, -scale_log2, nb))) : 0.f;
+          continue;
+        }
+        const float v = seen ? raw * scale_log2 : -INFINITY;
         sc[t][i] = v;
         mx = fmaxf(mx, v);
       }
+    if constexpr (!SIG) {
     mx = fmaxf(mx, __shfl_xor(mx, 16));
     mx = fmaxf(mx, __shfl_xor(mx, 32));
     const float m_new = fmaxf(m_run, mx);
@@ -928,6 +978,7 @@ __global__ __launch_bounds__(64 * NW) void attn_decode_mfma_kernel(
     for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
       for (int i = 0; i < 4; ++i) acc_o[dt][i] *= corr;
+    }
     Frag8 pf[2];
 #pragma unroll
     for (int s2 = 0; s2 < 2; ++s2) {
@@ -1004,13 +1055,13 @@ __global__ __launch_bounds__(64 * NW) void attn_decode_mfma_kernel(
 #pragma unroll
     for (int w = 0; w < NW; ++w) {
       const float f = exp2f(red_m[w * 16 + gg] - m_safe);
-      a += red_acc[((size_t)w * 16 + gg) * D + d] * f;
+      a += SIG ? red_acc[((size_t)w * 16 + gg) * D + d] : red_acc[((size_t)w * 16 + gg) * D + d] * f;
       const float* lw = red_l + w * 64 + gg;
       l += ((lw[0] + lw[16]) + (lw[32] + lw[48])) * f;
     }
     if (n_splits == 1) {
       if (sinks) l += exp2f(fmaf(sinks[kvh * G + gg], LOG2E, -m_safe));      // the sink: in the denominator only
-      out[((size_t)b * n_heads + kvh * G + gg) * D + d] = f32_to_bf16(l > 0.f ? a / l : 0.f);
+      out[((size_t)b * n_heads + kvh * G + gg) * D + d] = f32_to_bf16(SIG ? a : (l > 0.f ? a / l : 0.f));
     } else {
       float* dst = ws + (((size_t)b * n_heads + kvh * G + gg) * n_splits + split) * (D + 2);
       dst[d] = a;
@@ -1022,12 +1073,19 @@ __global__ __launch_bounds__(64 * NW) void attn_decode_mfma_kernel(
   }
 }
 
+// sum_only: the splits' outputs are added as they are (sigmoid weights), without maxima and denominators
 template <int D>
 __global__ void attn_decode_combine_kernel(const float* __restrict__ ws, bf16_t* __restrict__ out, int n_splits,
-                                           const float* __restrict__ sinks, int n_heads) {
+                                           const float* __restrict__ sinks, int n_heads, int sum_only) {
   const size_t row = blockIdx.x;            // sequence * heads + head
   const int d = threadIdx.x;
   const float* src = ws + row * n_splits * (D + 2);
+  if (sum_only) {
+    float v = 0.f;
+    for (int s = 0; s < n_splits; ++s) v += src[(size_t)s * (D + 2) + d];
+    out[row * D + d] = f32_to_bf16(v);
+    return;
+  }
   float mx = -INFINITY;
   for (int s = 0; s < n_splits; ++s) mx = fmaxf(mx, src[(size_t)s * (D + 2) + D]);
   const float m_safe = (mx == -INFINITY) ? 0.f : mx;
@@ -1062,6 +1120,8 @@ struct DecodeArgs {
   int keep_first = 0;     // with a window: the first keys that stay visible behind it
   float cap = 0.f;        // > 0: scores capped at cap * tanh(score / cap); sl2 is then log2(e) and cap_pre scale / cap
   float cap_pre = 0.f;
+  int chunk = 0;          // > 0: only the keys of the query's own chunk of positions
+  const float* sig_bias = nullptr;      // per query head: sigmoid weights
   int kv_rep = 1;         // n_kv counts every key/value head this many times (groups of at most 16 query heads on one of them)
 };
 
@@ -1071,13 +1131,15 @@ static void launch_decode(const DecodeArgs& a, hipStream_t s) {
   attn_decode_kernel<D, G, FUSED><<<grid, 256, 0, s>>>(a.qkv, a.q, a.cos_t, a.sin_t, a.style, a.k, a.v, a.out,
                                                        a.tok_pos, a.bt, a.bt_stride, a.n_heads, a.n_kv, a.sl2,
                                                        a.window, a.n_splits, a.ws, a.qkv_terms, a.qkv_stride, a.sinks);
-  if (a.n_splits > 1) attn_decode_combine_kernel<D><<<a.n_seqs * a.n_heads, D, 0, s>>>(a.ws, a.out, a.n_splits, a.sinks, a.n_heads);
+  if (a.n_splits > 1) attn_decode_combine_kernel<D><<<a.n_seqs * a.n_heads, D, 0, s>>>(a.ws, a.out, a.n_splits, a.sinks, a.n_heads, a.sig_bias != nullptr);
 }
 
-template <int D, int NW, bool FUSED, int ONCE>
+template <int D, int NW, bool FUSED, int ONCE, bool SIG = false>
 static int launch_decode_mfma_nw(const DecodeArgs& a, hipStream_t s) {
   const size_t lds = (size_t)NW * RB_PAGE * D * 2 + 16 * D * 2 + 2 * D * 2 + (size_t)NW * (16 + 64) * sizeof(float);
-  auto kern = attn_decode_mfma_kernel<D, NW, FUSED, ONCE>;
+  if constexpr (!FUSED && !SIG)
+    if (a.sig_bias) return launch_decode_mfma_nw<D, NW, FUSED, ONCE, true>(a, s);
+  auto kern = attn_decode_mfma_kernel<D, NW, FUSED, ONCE, SIG>;
   static bool configured = false;
   if (!configured) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
@@ -1088,8 +1150,8 @@ static int launch_decode_mfma_nw(const DecodeArgs& a, hipStream_t s) {
   dim3 grid(a.n_splits, a.n_kv, a.n_seqs);
   kern<<<grid, 64 * NW, lds, s>>>(a.qkv, a.q, a.cos_t, a.sin_t, a.style, a.k, a.v, a.out, a.tok_pos, a.bt,
                                   a.bt_stride, a.n_heads, a.n_kv, a.sl2, a.window, a.n_splits, a.ws, a.qkv_terms,
-                                  a.qkv_stride, a.sinks, a.keep_first, a.cap, a.cap_pre, a.kv_rep);
-  if (a.n_splits > 1) attn_decode_combine_kernel<D><<<a.n_seqs * a.n_heads, D, 0, s>>>(a.ws, a.out, a.n_splits, a.sinks, a.n_heads);
+                                  a.qkv_stride, a.sinks, a.keep_first, a.cap, a.cap_pre, a.kv_rep, a.chunk, a.sig_bias);
+  if (a.n_splits > 1) attn_decode_combine_kernel<D><<<a.n_seqs * a.n_heads, D, 0, s>>>(a.ws, a.out, a.n_splits, a.sinks, a.n_heads, a.sig_bias != nullptr);
   return 0;
 }
 
@@ -1143,7 +1205,8 @@ static int dispatch_decode(const DecodeArgs& a, int head_dim, hipStream_t s, con
   RB_REQUIRE(group <= 16, "%s: %d query heads per kv head not supported (at most 16; use rb_attention_generic)", who,
              group);
   RB_REQUIRE(g_decode_mfma != 2 || vector_ok, "%s: the vector kernel is built for 1, 2, 4 or 8 heads per kv head", who);
-  const bool opts = a.keep_first > 0 || a.cap > 0.f || a.kv_rep > 1;      // kept first keys, capped scores, repeated kv heads: the matrix-core kernel has them
+  // kept first keys, capped scores, repeated kv heads, chunks, sigmoid weights: the matrix-core kernel has them
+  const bool opts = a.keep_first > 0 || a.cap > 0.f || a.kv_rep > 1 || a.chunk > 0 || a.sig_bias != nullptr;
   RB_REQUIRE(!opts || g_decode_mfma != 2, "%s: kept first keys and capped scores need the matrix-core kernel", who);
   if (opts || g_decode_mfma == 1 || !vector_ok || (g_decode_mfma == 0 && group > 1)) {
     const int rc = head_dim == 128 ? launch_decode_mfma<128, FUSED>(a, s) : launch_decode_mfma<64, FUSED>(a, s);
@@ -1181,13 +1244,29 @@ extern "C" int rb_attention_decode_bf16_opts(const void* q, const void* k_pages,
   RB_RECORDED(rb_attention_decode_bf16_opts(q, k_pages, v_pages, out, tok_pos, block_table, bt_stride, n_seqs, n_heads,
                                             n_kv_heads, head_dim, scale, window, keep_first, softcap, n_splits, workspace, sinks,
                                             stream));
-  RB_REQUIRE(keep_first >= 0 && softcap >= 0.f, "rb_attention_decode_bf16: negative keep_first or softcap");
+  return rb_attention_decode_bf16_chunked(q, k_pages, v_pages, out, tok_pos, block_table, bt_stride, n_seqs, n_heads, n_kv_heads,
+                                          head_dim, scale, window, keep_first, softcap, n_splits, workspace, sinks, 0, nullptr, stream);
+}
+
+// With chunks and sigmoid weights: see rb_attention_generic_chunked.
+extern "C" int rb_attention_decode_bf16_chunked(const void* q, const void* k_pages, const void* v_pages, void* out,
+                                                const int32_t* tok_pos, const int32_t* block_table, int bt_stride, int n_seqs,
+                                                int n_heads, int n_kv_heads, int head_dim, float scale, int window, int keep_first,
+                                                float softcap, int n_splits, float* workspace, const float* sinks, int chunk,
+                                                const float* sig_bias, void* stream) {
+  RB_RECORDED(rb_attention_decode_bf16_chunked(q, k_pages, v_pages, out, tok_pos, block_table, bt_stride, n_seqs, n_heads,
+                                               n_kv_heads, head_dim, scale, window, keep_first, softcap, n_splits, workspace, sinks,
+                                               chunk, sig_bias, stream));
+  RB_REQUIRE(keep_first >= 0 && softcap >= 0.f && chunk >= 0, "rb_attention_decode_bf16: negative keep_first, softcap or chunk");
+  RB_REQUIRE(sig_bias == nullptr || sinks == nullptr, "rb_attention_decode_bf16: a sink belongs to the softmax");
   DecodeArgs a = {nullptr, (const bf16_t*)q, nullptr, nullptr, 0, (bf16_t*)k_pages, (bf16_t*)v_pages, (bf16_t*)out,
                   tok_pos, block_table, bt_stride, n_seqs, n_heads, n_kv_heads, softcap > 0.f ? LOG2E : scale * LOG2E, window,
                   n_splits, workspace, 1, 0, sinks};
   a.keep_first = window > 0 ? keep_first : 0;
   a.cap = softcap;
   a.cap_pre = softcap > 0.f ? scale / softcap : 0.f;
+  a.chunk = chunk;
+  a.sig_bias = sig_bias;
   // more than 16 query heads on a key/value head: the fewest groups of equal size that hold at most 16 each
   if (n_kv_heads > 0 && n_heads % n_kv_heads == 0) {
     const int group = n_heads / n_kv_heads;

@@ -101,6 +101,15 @@ struct Num<bf16_t> {
   static __device__ __forceinline__ void store(bf16_t* p, float v) { *p = f32_to_bf16(v); }
 };
 
+// ---------------------------------------------------------------- the first key that a query sees
+// window > 0: the last `window` keys, the query's own among them; chunk > 0: the keys of the query's own chunk of positions,
+// chunks being counted from the sequence's first position.  0: no such limit.
+__device__ __forceinline__ int first_visible(int pos, int window, int chunk) {
+  const int w = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int c = chunk > 0 ? pos - pos % chunk : 0;
+  return w > c ? w : c;
+}
+
 // ---------------------------------------------------------------- rotation of a pair
 // (x0, x1) turned by the angle whose cosine and sine are c and s (llama/model.rs:122-136). The
 // operations are spelled out so that every kernel that rotates rounds the same way, whatever

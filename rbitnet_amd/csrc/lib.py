@@ -105,7 +105,7 @@ class KernelTimes:
         return "\n".join(lines)
 
 
-TIMED_OPS = ("short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
+TIMED_OPS = ("tanh_norm", "heads_prepare", "lightning_recurrence", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
              "route_top", "routed_experts", "pairs_sum", "embed_streams", "streams_layernorm", "streams_update", "xielu", "tanh_cap", "short_conv",
              "delta_prep", "delta_rule", "gated_rmsnorm", "latent_norm_store", "heads_linear", "attention_sinks", "embed_gather", "add_rmsnorm", "rope_kv_write", "swiglu", "gemm_generic", "gemm_bf16", "gemm_bf16_terms",
              "gemm_bf16_few", "attention_generic", "attention_prefill_bf16", "attention_decode_bf16",
@@ -196,6 +196,14 @@ class Kernels:
             "rb_heads_linear_more": [_P, _I, _L, _P, _I, _P, _I, _L, _I, _I, _I, _I, _P, _L, _I, _I, _I, _P, _P, _I, _P, _P],
             "rb_heads_linear_strided": [_P, _I, _L, _P, _I, _P, _I, _L, _I, _I, _I, _I, _P],
             "rb_latent_norm_rope_store": [_P, _L, _I, _P, _P, _I, _I, _P, _P, _I, _I, _I, _P, _P, _I, _I, _P, _P, _P, _I, _F, _I, _P],
+            "rb_attention_generic_chunked": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _F, _P, _I, _P, _P],
+            "rb_attention_prefill_bf16_chunked": [_P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _F, _P, _I, _P, _P],
+            "rb_attention_decode_bf16_chunked": [_P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _F, _I, _P, _P, _I, _P, _P],
+            "rb_heads_prepare": [_P, _L, _P, _P, _I, _I, _P, _P, _I, _F, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
+            "rb_tanh_norm": [_P, _P, _I, _L, _L, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _I, _P],
+            "rb_lightning_recurrence": [_P, _P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P],
+            "rb_gated_rmsnorm_rows": [_P, _P, _P, _L, _I, _F, _P, _I, _I, _I, _P],
+            "rb_route_choose_bias": [_P, _L, _P, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
             "rb_attention_mixed": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P, _I, _I, _P],
             "rb_attention_mixed_bf16": [_P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P, _I, _I, _I, _P, _P],
         }
@@ -396,7 +404,8 @@ class Kernels:
 
     def attention_prefill_bf16(self, q, k_pages, v_pages, out, cu_seqlens, past_len, block_table, n_seqs,
                                max_q_len, n_heads, n_kv, head_dim, scale, window, sinks=None, keep_first: int = 0,
-                               softcap: float = 0.0) -> None:
+                               softcap: float = 0.0, chunk: int = 0, sig_bias=None) -> None:
+        """chunk > 0: a query sees the keys of its own chunk of positions only; sig_bias float32 [Hq]: sigmoid weights."""
         n = q.shape[0]
         _check(q, "q", torch.bfloat16, (n, n_heads, head_dim))
         _check(k_pages, "k_pages", torch.bfloat16)
@@ -409,6 +418,16 @@ class Kernels:
         _check(block_table, "block_table", torch.int32)
         if sinks is not None:
             _check(sinks, "sinks", torch.float32, (n_heads,))
+        if chunk or sig_bias is not None:
+            if sig_bias is not None:
+                _check(sig_bias, "sig_bias", torch.float32, (n_heads,))
+            self._ok(self._lib.rb_attention_prefill_bf16_chunked(_ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(out),
+                                                                 _ptr(cu_seqlens), _ptr(past_len), _ptr(block_table),
+                                                                 block_table.shape[1], n_seqs, int(max_q_len), n_heads, n_kv,
+                                                                 head_dim, float(scale), int(window or 0), int(keep_first or 0),
+                                                                 float(softcap or 0.0), _ptr(sinks), int(chunk or 0),
+                                                                 _ptr(sig_bias), self._stream()))
+            return
         self._ok(self._lib.rb_attention_prefill_bf16_opts(_ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(out),
                                                           _ptr(cu_seqlens), _ptr(past_len), _ptr(block_table),
                                                           block_table.shape[1], n_seqs, int(max_q_len), n_heads, n_kv,
@@ -416,7 +435,9 @@ class Kernels:
                                                           float(softcap or 0.0), _ptr(sinks), self._stream()))
 
     def attention_decode_bf16(self, q, k_pages, v_pages, out, tok_pos, block_table, n_heads, n_kv, head_dim,
-                              scale, window, n_splits, workspace, sinks=None, keep_first: int = 0, softcap: float = 0.0) -> None:
+                              scale, window, n_splits, workspace, sinks=None, keep_first: int = 0, softcap: float = 0.0,
+                              chunk: int = 0, sig_bias=None) -> None:
+        """chunk > 0: a query sees the keys of its own chunk of positions only; sig_bias float32 [Hq]: sigmoid weights."""
         n = q.shape[0]
         _check(q, "q", torch.bfloat16, (n, n_heads, head_dim))
         _check(k_pages, "k_pages", torch.bfloat16)
@@ -431,6 +452,15 @@ class Kernels:
             raise KernelError("decode attention workspace too small")
         if sinks is not None:
             _check(sinks, "sinks", torch.float32, (n_heads,))
+        if chunk or sig_bias is not None:
+            if sig_bias is not None:
+                _check(sig_bias, "sig_bias", torch.float32, (n_heads,))
+            self._ok(self._lib.rb_attention_decode_bf16_chunked(_ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(out), _ptr(tok_pos),
+                                                                _ptr(block_table), block_table.shape[1], n, n_heads, n_kv,
+                                                                head_dim, float(scale), int(window or 0), int(keep_first or 0),
+                                                                float(softcap or 0.0), int(n_splits), _ptr(workspace), _ptr(sinks),
+                                                                int(chunk or 0), _ptr(sig_bias), self._stream()))
+            return
         if keep_first or softcap or n_heads // n_kv > 16:        # this entry point also runs more than 16 heads on a kv head, in groups
             self._ok(self._lib.rb_attention_decode_bf16_opts(_ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(out), _ptr(tok_pos),
                                                              _ptr(block_table), block_table.shape[1], n, n_heads, n_kv,
@@ -822,10 +852,10 @@ class Kernels:
 
     def route_choose(self, z: torch.Tensor, n_outputs: int, n_experts: int, top: int, score: int,
                      correction: Optional[torch.Tensor], sel: torch.Tensor, weight: torch.Tensor, row_pair: torch.Tensor,
-                     tile_expert: torch.Tensor) -> None:
+                     tile_expert: torch.Tensor, bias: Optional[torch.Tensor] = None) -> None:
         """`route_top` with its choices spelled out: the router's first n_experts outputs are experts with matrices, the
         rest stand for the token's own input; score 0 sigmoid, 1 softmax over all outputs with `correction` [n_outputs]
-        added for the choice only."""
+        added for the choice only, 2 softmax over the chosen logits alone; `bias` [n_outputs] is added to the logits first."""
         n = z.shape[0]
         _check(z, "z", torch.float32)
         if z.shape[1] < n_outputs or n_experts > n_outputs:
@@ -835,12 +865,15 @@ class Kernels:
             raise KernelError("route_choose: too little room for the sorted pairs")
         if correction is not None:
             _check(correction, "correction", torch.float32, (n_outputs,))
+        if bias is not None:
+            _check(bias, "bias", torch.float32, (n_outputs,))
         _check(sel, "sel", torch.int32, (n * top,))
         _check(weight, "weight", torch.float32, (n * top,))
         _check(row_pair, "row_pair", torch.int32, (max_rows,))
         _check(tile_expert, "tile_expert", torch.int32, (2 * (max_rows // 16),))
-        self._ok(self._lib.rb_route_choose(_ptr(z), z.shape[1], n_outputs, n_experts, top, int(score), _ptr(correction), _ptr(sel),
-                                           _ptr(weight), _ptr(row_pair), _ptr(tile_expert), max_rows, n, self._stream()))
+        self._ok(self._lib.rb_route_choose_bias(_ptr(z), z.shape[1], _ptr(bias), n_outputs, n_experts, top, int(score),
+                                                _ptr(correction), _ptr(sel), _ptr(weight), _ptr(row_pair), _ptr(tile_expert), max_rows,
+                                                n, self._stream()))
 
     def experts_combine(self, pairs: torch.Tensor, sel: torch.Tensor, weight: torch.Tensor, top: int, n_experts: int,
                         h: torch.Tensor, shared: Optional[torch.Tensor], gate: Optional[torch.Tensor], gate_col: int,
@@ -1056,8 +1089,9 @@ class Kernels:
         self._ok(self._lib.rb_tanh_cast(_ptr(z), _ptr(out), dtype_code(out.dtype), z.numel(), self._stream()))
 
     def attention_opts(self, q, k_pages, v_pages, out, tok_pos, tok_seq, block_table, n_heads, n_kv, head_dim, scale, window,
-                       keep_first, softcap, sinks) -> None:
-        """`attention_sinks` with kept first keys behind the window and capped scores."""
+                       keep_first, softcap, sinks, chunk: int = 0, sig_bias=None) -> None:
+        """`attention_sinks` with kept first keys behind the window, capped scores, chunks (a query sees the keys of its own
+        chunk of positions only) and sigmoid weights (sig_bias float32 [Hq])."""
         n = q.shape[0]
         _check(q, "q", None, (n, n_heads, head_dim))
         _check(k_pages, "k_pages", q.dtype)
@@ -1070,6 +1104,15 @@ class Kernels:
         _check(block_table, "block_table", torch.int32)
         if sinks is not None:
             _check(sinks, "sinks", torch.float32, (n_heads,))
+        if chunk or sig_bias is not None:
+            if sig_bias is not None:
+                _check(sig_bias, "sig_bias", torch.float32, (n_heads,))
+            self._ok(self._lib.rb_attention_generic_chunked(_ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(out), dtype_code(q.dtype),
+                                                            _ptr(tok_pos), _ptr(tok_seq), _ptr(block_table), block_table.shape[1],
+                                                            n, n_heads, n_kv, head_dim, float(scale), int(window or 0),
+                                                            int(keep_first or 0), float(softcap or 0.0), _ptr(sinks),
+                                                            int(chunk or 0), _ptr(sig_bias), self._stream()))
+            return
         self._ok(self._lib.rb_attention_generic_opts(_ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(out), dtype_code(q.dtype),
                                                      _ptr(tok_pos), _ptr(tok_seq), _ptr(block_table), block_table.shape[1],
                                                      n, n_heads, n_kv, head_dim, float(scale), int(window or 0),
@@ -1256,6 +1299,116 @@ class Kernels:
                                                      dtype_code(dtype), _ptr(ctx.tok_pos), _ptr(ctx.tok_seq),
                                                      _ptr(block_table) if has_kv else None, block_table.shape[1] if has_kv else 0,
                                                      float(eps), n, self._stream()))
+
+    # ------------------------------------------------------------------ norms in front of and behind a sublayer
+    def tanh_norm(self, x: torch.Tensor, y: Optional[torch.Tensor], after, before, rows: Optional[torch.Tensor],
+                  out: Optional[torch.Tensor], weights: Optional[torch.Tensor] = None) -> None:
+        """x [T, E] float32 <- x + (after ? tanh(a y) w + b : y) with after = (a, w, b) or None, then (out given)
+        out[r] = tanh(a x[r]) w + b with before = (a, w, b), on all rows, or on `rows` (x is then left as it is).
+        y: [T, E]; [P, T, E], terms that are added up; or, with weights float32 [T * k], the outputs [T * k, E] of every
+        token's k experts, each times its weight; None: nothing is added."""
+        t, width = x.shape
+        _check(x, "x", torch.float32)
+        n_terms, term_stride, row_stride = 1, 0, width
+        if y is not None:
+            if weights is not None:
+                n_terms, term_stride = y.shape[0] // max(1, t), width
+                row_stride = n_terms * width
+                _check(y, "y", torch.float32, (t * n_terms, width))
+                _check(weights, "weights", torch.float32, (t * n_terms,))
+            elif y.dim() == 3:
+                n_terms, term_stride = y.shape[0], x.numel()
+                _check(y, "y", torch.float32, (n_terms, t, width))
+            else:
+                _check(y, "y", torch.float32, (t, width))
+        for norm in (after, before):
+            if norm is not None:
+                _check(norm[0], "alpha", torch.float32)
+                _check(norm[1], "weight", torch.float32, (width,))
+                _check(norm[2], "bias", torch.float32, (width,))
+                if norm[0].numel() != 1:
+                    raise KernelError("tanh_norm: alpha is one number")
+        n_rows = t
+        if rows is not None:
+            n_rows = rows.shape[0]
+            _check(rows, "rows", torch.int32, (n_rows,))
+        if out is not None:
+            _check(out, "out", None, (n_rows, width))
+        a1, w1, b1 = after if after is not None else (None, None, None)
+        a2, w2, b2 = before if before is not None else (None, None, None)
+        self._ok(self._lib.rb_tanh_norm(_ptr(x), _ptr(y), n_terms, term_stride, row_stride, _ptr(weights), _ptr(a1), _ptr(w1), _ptr(b1),
+                                        _ptr(a2), _ptr(w2), _ptr(b2), _ptr(rows), n_rows, width, _ptr(out),
+                                        dtype_code(out.dtype) if out is not None else _F32, self._stream()))
+
+    def heads_prepare(self, qkv: torch.Tensor, cos, sin, rot: int, style: int, q_norm: Optional[torch.Tensor],
+                      k_norm: Optional[torch.Tensor], value_norm: bool, eps: float, q_out: torch.Tensor, k_pages, v_pages, tok_pos,
+                      tok_seq, block_table, n_heads: int, n_kv: int, dim: int, vdim: int, pad: int) -> None:
+        """`rope_store` with q and k normed over all their numbers together (weights [Hq dim], [Hk dim]; None: neither), either
+        pairing, and every value head divided by its root mean square (value_norm)."""
+        n, width = qkv.shape
+        _check(qkv, "qkv", torch.float32)
+        _check(q_out, "q_out", None, (n, n_heads, pad))
+        _check(tok_pos, "tok_pos", torch.int32, (n,))
+        _check(tok_seq, "tok_seq", torch.int32, (n,))
+        if q_norm is not None:
+            _check(q_norm, "q_norm", torch.float32, (n_heads * dim,))
+        if rot:
+            _check(cos, "cos", torch.float32)
+            _check(sin, "sin", torch.float32, cos.shape)
+            if cos.shape[1] != rot // 2:
+                raise KernelError("angle table width mismatch")
+        need = n_heads * dim
+        owns = k_pages is not None
+        if owns:
+            need += n_kv * (dim + vdim)
+            if k_norm is not None:
+                _check(k_norm, "k_norm", torch.float32, (n_kv * dim,))
+            _check(block_table, "block_table", torch.int32)
+            _check(k_pages, "k_pages", q_out.dtype)
+            _check(v_pages, "v_pages", q_out.dtype, k_pages.shape)
+            if tuple(k_pages.shape[1:]) != (n_kv, self.page_size, pad):
+                raise KernelError(f"cache pages have shape {tuple(k_pages.shape)}, expected [*, {n_kv}, {self.page_size}, {pad}]")
+        if width < need:
+            raise KernelError("heads_prepare: rows too short for the heads")
+        self._ok(self._lib.rb_heads_prepare(_ptr(qkv), width, _ptr(cos) if rot else None, _ptr(sin) if rot else None, int(rot), int(style),
+                                            _ptr(q_norm), _ptr(k_norm) if owns else None, int(bool(value_norm)), float(eps), _ptr(q_out),
+                                            _ptr(k_pages), _ptr(v_pages), dtype_code(q_out.dtype), _ptr(tok_pos), _ptr(tok_seq),
+                                            _ptr(block_table) if owns else None, block_table.shape[1] if owns else 0, n, n_heads,
+                                            n_kv if owns else 0, dim, vdim, pad, self._stream()))
+
+    # ------------------------------------------------------------------ linear attention with constant decays
+    def lightning_recurrence(self, qkv: torch.Tensor, dim: int, n_heads: int, vdim: int, decay: torch.Tensor, state: torch.Tensor, ctx,
+                             out: torch.Tensor) -> None:
+        """qkv rows [q | k | v | ...] float32, silu on all three as they are read; decay float32 [H]; state [slots, H, vdim, dim]
+        float32: S <- decay S + k v^T, out = S^T q, token after token."""
+        n, width = qkv.shape
+        _check(qkv, "qkv", torch.float32)
+        if width < n_heads * (2 * dim + vdim):
+            raise KernelError("lightning_recurrence: rows too short for q, k and v")
+        _check(decay, "decay", torch.float32, (n_heads,))
+        _check(state, "state", torch.float32)
+        if tuple(state.shape[1:]) != (n_heads, vdim, dim):
+            raise KernelError(f"lightning_recurrence: state of shape {tuple(state.shape)}, expected [*, {n_heads}, {vdim}, {dim}]")
+        _check(out, "out", torch.float32, (n, n_heads * vdim))
+        if ctx.n_tokens != n:
+            raise KernelError("lightning_recurrence: the step's tokens and the rows differ")
+        base, nq = qkv.data_ptr(), n_heads * dim
+        self._ok(self._lib.rb_lightning_recurrence(base, base + 4 * nq, width, base + 8 * nq, width, _ptr(decay), _ptr(state),
+                                                   _ptr(ctx.cu_seqlens), _ptr(ctx.slots), _ptr(out), ctx.n_seqs, n, n_heads, dim, vdim,
+                                                   self._stream()))
+
+    def gated_rmsnorm_rows(self, o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, gate_col: int, act: int, eps: float,
+                           out: torch.Tensor) -> None:
+        """`gated_rmsnorm_act` with one norm over the whole row; gate at columns gate_col .. of its rows."""
+        n, width = o.shape
+        _check(o, "o", torch.float32)
+        _check(weight, "weight", torch.float32, (width,))
+        _check(gate, "gate", torch.float32)
+        if gate.shape[0] != n or gate_col < 0 or gate_col + width > gate.shape[1]:
+            raise KernelError("gated_rmsnorm_rows: the gate's columns lie outside the rows")
+        _check(out, "out", None, (n, width))
+        self._ok(self._lib.rb_gated_rmsnorm_rows(_ptr(o), _ptr(weight), gate.data_ptr() + 4 * gate_col, gate.shape[1], int(act), float(eps),
+                                                 _ptr(out), dtype_code(out.dtype), n, width, self._stream()))
 
     # ------------------------------------------------------------------ recorded steps
     def plan_begin(self) -> int:

@@ -404,6 +404,163 @@ extern "C" int rb_norm_rope_store(const float* qkv, long long row_width, const f
   return 0;
 }
 
+// ---------------------------------------------------------------- norms over the whole projection in front of the rotation
+// A row of qkv as above.  The Hq * dim numbers of q are divided by their common root mean square and multiplied by q_norm
+// [Hq * dim] (null: neither), those of k likewise with k_norm [Hk * dim]; then the first `rot` numbers of every head are
+// rotated (style 0: 2i with 2i + 1; 1: i with i + rot / 2); every value head is divided by its own root mean square where
+// value_norm is set.  Padding and cache write as in rb_rope_store.  A workgroup a token; float32 arithmetic.
+template <typename TC>
+__global__ __launch_bounds__(1024) void heads_prepare_kernel(
+    const float* __restrict__ qkv, size_t row_width, const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot, int style,
+    const float* __restrict__ q_norm, const float* __restrict__ k_norm, int value_norm, float eps, TC* __restrict__ q_out,
+    TC* __restrict__ k_pages, TC* __restrict__ v_pages, const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_seq,
+    const int32_t* __restrict__ block_table, int bt_stride, int n_heads, int n_kv, int dim, int vdim, int pad, int vec) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x;
+  const int pos = tok_pos[t];
+  const int half = rot / 2;
+  const float* src = qkv + (size_t)t * row_width;
+  const float* cr = cos_t + (size_t)pos * half;
+  const float* sr = sin_t + (size_t)pos * half;
+  size_t page_base = 0;
+  if (k_pages) {
+    const int page = block_table[(size_t)tok_seq[t] * bt_stride + pos / RB_PAGE];
+    page_base = ((size_t)page * n_kv) * RB_PAGE * pad + (size_t)(pos % RB_PAGE) * pad;
+  }
+  const int nq = n_heads * dim, nk = k_pages ? n_kv * dim : 0;
+  float fq = 1.f, fk = 1.f;
+  auto squares = [&](const float* p, int n) {
+    float ss = 0.f;
+    if (vec) {
+      for (int j = 4 * threadIdx.x; j < n; j += 4 * blockDim.x) {
+        const float4 v = *reinterpret_cast<const float4*>(p + j);
+        ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+      }
+    } else {
+      for (int j = threadIdx.x; j < n; j += blockDim.x) ss = fmaf(p[j], p[j], ss);
+    }
+    return ss;
+  };
+  if (q_norm) {
+    const float sq = squares(src, nq), sk = nk ? squares(src + nq, nk) : 0.f;
+    fq = 1.0f / sqrtf(block_sum(sq, scratch) / (float)nq + eps);
+    if (nk) fk = 1.0f / sqrtf(block_sum(sk, scratch) / (float)nk + eps);
+  }
+  const int n_rot_heads = n_heads + (k_pages ? n_kv : 0);
+  auto dest = [&](int h) {
+    return h < n_heads ? q_out + ((size_t)t * n_heads + h) * pad : k_pages + page_base + (size_t)(h - n_heads) * RB_PAGE * pad;
+  };
+  if (vec) {
+    // four numbers a thread: sizes that are multiples of 4, and a rotated part that is (style 1: of 8)
+    const int quads = pad / 4;
+    for (int idx = threadIdx.x; idx < n_rot_heads * quads; idx += blockDim.x) {
+      const int h = idx / quads, d = 4 * (idx - h * quads);
+      const float f = h < n_heads ? fq : fk;
+      const float* wrow = q_norm ? (h < n_heads ? q_norm + (size_t)h * dim : k_norm + (size_t)(h - n_heads) * dim) : nullptr;
+      const float* hp = src + (size_t)h * dim;
+      auto normed = [&](int i) {
+        float4 v = *reinterpret_cast<const float4*>(hp + i);
+        if (wrow) {
+          const float4 w = *reinterpret_cast<const float4*>(wrow + i);
+          v = make_float4(v.x * f * w.x, v.y * f * w.y, v.z * f * w.z, v.w * f * w.w);
+        }
+        return v;
+      };
+      float4 y = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (d < rot && style == 0) {
+        const float4 v = normed(d);
+        const float2 c = *reinterpret_cast<const float2*>(cr + d / 2), sn = *reinterpret_cast<const float2*>(sr + d / 2);
+        rotate_pair(v.x, v.y, c.x, sn.x, y.x, y.y);
+        rotate_pair(v.z, v.w, c.y, sn.y, y.z, y.w);
+      } else if (d < rot) {
+        const bool first = d < half;
+        const int i = first ? d : d - half;
+        const float4 a = normed(i), b = normed(i + half);
+        const float4 c = *reinterpret_cast<const float4*>(cr + i), sn = *reinterpret_cast<const float4*>(sr + i);
+        float4 y0, y1;
+        rotate_pair(a.x, b.x, c.x, sn.x, y0.x, y1.x);
+        rotate_pair(a.y, b.y, c.y, sn.y, y0.y, y1.y);
+        rotate_pair(a.z, b.z, c.z, sn.z, y0.z, y1.z);
+        rotate_pair(a.w, b.w, c.w, sn.w, y0.w, y1.w);
+        y = first ? y0 : y1;
+      } else if (d < dim) {
+        y = normed(d);
+      }
+      store4(dest(h) + d, y.x, y.y, y.z, y.w);
+    }
+  } else {
+    for (int idx = threadIdx.x; idx < n_rot_heads * pad; idx += blockDim.x) {
+      const int h = idx / pad, d = idx - h * pad;
+      const float f = h < n_heads ? fq : fk;
+      const float* wrow = q_norm ? (h < n_heads ? q_norm + (size_t)h * dim : k_norm + (size_t)(h - n_heads) * dim) : nullptr;
+      const float* hp = src + (size_t)h * dim;
+      auto normed = [&](int i) { return wrow ? hp[i] * f * wrow[i] : hp[i]; };
+      float y = 0.f;
+      if (d < rot) {
+        const bool first = style == 0 ? (d & 1) == 0 : d < half;
+        const int i = style == 0 ? d / 2 : (first ? d : d - half);
+        const int a = style == 0 ? 2 * i : i, b = style == 0 ? 2 * i + 1 : i + half;
+        float y0, y1;
+        rotate_pair(normed(a), normed(b), cr[i], sr[i], y0, y1);
+        y = first ? y0 : y1;
+      } else if (d < dim) {
+        y = normed(d);
+      }
+      Num<TC>::store(dest(h) + d, y);
+    }
+  }
+  if (v_pages) {
+    // a wave a value head
+    const int lane = threadIdx.x & (RB_WAVE - 1), wave = threadIdx.x / RB_WAVE, n_waves = blockDim.x / RB_WAVE;
+    for (int h = wave; h < n_kv; h += n_waves) {
+      const float* vp = src + (size_t)(n_heads + n_kv) * dim + (size_t)h * vdim;
+      float f = 1.f;
+      if (value_norm) {
+        float ss = 0.f;
+        for (int d = lane; d < vdim; d += RB_WAVE) ss = fmaf(vp[d], vp[d], ss);
+        f = 1.0f / sqrtf(wave_sum(ss) / (float)vdim + eps);
+      }
+      TC* dst = v_pages + page_base + (size_t)h * RB_PAGE * pad;
+      for (int d = lane; d < pad; d += RB_WAVE) Num<TC>::store(dst + d, d < vdim ? (value_norm ? vp[d] * f : vp[d]) : 0.f);
+    }
+  }
+}
+
+extern "C" int rb_heads_prepare(const float* qkv, long long row_width, const float* cos, const float* sin, int rot, int style,
+                                const float* q_norm, const float* k_norm, int value_norm, float eps, void* q_out, void* k_pages,
+                                void* v_pages, int cache_dtype, const int32_t* tok_pos, const int32_t* tok_seq,
+                                const int32_t* block_table, int bt_stride, int n_tokens, int n_heads, int n_kv_heads, int dim, int vdim,
+                                int pad, void* stream) {
+  RB_RECORDED(rb_heads_prepare(qkv, row_width, cos, sin, rot, style, q_norm, k_norm, value_norm, eps, q_out, k_pages, v_pages, cache_dtype,
+                               tok_pos, tok_seq, block_table, bt_stride, n_tokens, n_heads, n_kv_heads, dim, vdim, pad, stream));
+  RB_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads >= 0 && dim > 0 && vdim > 0 && pad >= dim && pad >= vdim,
+             "rb_heads_prepare: bad sizes T=%d Hq=%d Hk=%d dim=%d vdim=%d pad=%d", n_tokens, n_heads, n_kv_heads, dim, vdim, pad);
+  RB_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dim && (style == 0 || style == 1), "rb_heads_prepare: %d rotated numbers in a head of %d", rot, dim);
+  RB_REQUIRE(rot == 0 || (cos != nullptr && sin != nullptr), "rb_heads_prepare: a rotation needs its tables");
+  RB_REQUIRE((k_pages == nullptr) == (v_pages == nullptr), "rb_heads_prepare: k and v pages go together");
+  RB_REQUIRE(q_norm == nullptr || k_pages == nullptr || k_norm != nullptr, "rb_heads_prepare: both norms' weights or none");
+  const long long need = (long long)n_heads * dim + (k_pages ? (long long)n_kv_heads * (dim + vdim) : 0);
+  RB_REQUIRE(row_width >= need, "rb_heads_prepare: rows of %lld numbers, %lld needed", row_width, need);
+  RB_REQUIRE(cache_dtype == RB_F32 || cache_dtype == RB_BF16, "rb_heads_prepare: unknown dtype %d", cache_dtype);
+  if (n_tokens == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const int vec = dim % 4 == 0 && pad % 4 == 0 && rot % (style == 0 ? 4 : 8) == 0 && row_width % 4 == 0 && aligned(qkv) && aligned(cos) &&
+                  aligned(sin) && aligned(q_norm) && aligned(k_norm) && aligned(q_out) && aligned(k_pages);
+  // a step of few tokens has few workgroups: more waves each
+  const int threads = n_tokens < 2 * rb_compute_units() ? 1024 : 256;
+  if (cache_dtype == RB_F32)
+    heads_prepare_kernel<float><<<n_tokens, threads, 0, s>>>(qkv, (size_t)row_width, cos, sin, rot, style, q_norm, k_norm, value_norm, eps,
+                                                             (float*)q_out, (float*)k_pages, (float*)v_pages, tok_pos, tok_seq,
+                                                             block_table, bt_stride, n_heads, n_kv_heads, dim, vdim, pad, vec);
+  else
+    heads_prepare_kernel<bf16_t><<<n_tokens, threads, 0, s>>>(qkv, (size_t)row_width, cos, sin, rot, style, q_norm, k_norm, value_norm, eps,
+                                                              (bf16_t*)q_out, (bf16_t*)k_pages, (bf16_t*)v_pages, tok_pos, tok_seq,
+                                                              block_table, bt_stride, n_heads, n_kv_heads, dim, vdim, pad, vec);
+  RB_LAUNCH_CHECK();
+  return 0;
+}
+
 // ---------------------------------------------------------------- a gate on every number
 // x[e] *= sigmoid(gate[e]), in place; x of dtype and gate float32 laid out alike, n numbers.
 template <typename TC>

@@ -245,12 +245,14 @@ __device__ __forceinline__ float lanes_sum(float v) {
   return v;
 }
 
-template <int DKL, int RG, int CH, bool BONUS>
+// MODE 0: as above; 1: the read before the write, with a bonus (see below); 2: q, k and v go through silu as they are fetched.
+template <int DKL, int RG, int CH, int MODE>
 __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
     const float* __restrict__ q, const float* __restrict__ k, size_t qk_stride, const float* __restrict__ v,
     size_t v_stride, const float* __restrict__ g, size_t g_stride, const float* __restrict__ beta, float* __restrict__ state,
     const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ slots, float* __restrict__ out, int n_heads,
     int n_kv, int dim, int vdim, int g_per_head, const float* __restrict__ bonus) {
+  constexpr bool BONUS = MODE == 1;
   constexpr int COLS = RB_WAVE / RG;
   constexpr int DK = DKL * RG;               // rows held, >= dim; rows beyond dim stay zero
   constexpr int NQ = DK * CH / RB_WAVE;      // q (or k, or g) values of a chunk per lane
@@ -305,11 +307,16 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
       rq[j] = in ? q[t * qk_stride + (size_t)kvh * dim + i] : 0.f;
       rk[j] = in ? k[t * qk_stride + (size_t)kvh * dim + i] : 0.f;
       rgt[j] = in ? (g_per_head ? g[t * g_stride + h] : g[t * g_stride + (size_t)h * dim + i]) : 0.f;
+      if (MODE == 2) {
+        rq[j] *= rb_sigmoid(rq[j]);
+        rk[j] *= rb_sigmoid(rk[j]);
+      }
     }
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int e = lane + RB_WAVE * j, tt = e / COLS, c = e - tt * COLS;
       rv[j] = (tt < nt && col0 + c < vdim) ? v[(size_t)(row0 + t0 + tt) * v_stride + (size_t)h * vdim + col0 + c] : 0.f;
+      if (MODE == 2) rv[j] *= rb_sigmoid(rv[j]);
     }
     rb = (beta && lane < nt) ? beta[(size_t)(row0 + t0 + lane) * n_heads + h] : 0.f;
   };
@@ -398,7 +405,7 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
   }
 }
 
-template <int DKL, int RG, int CH, bool BONUS>
+template <int DKL, int RG, int CH, int MODE>
 static void launch_delta_rule(const float* q, const float* k, size_t qk_stride, const float* v, size_t v_stride,
                               const float* g, size_t g_stride, const float* beta, float* state, const int32_t* cu_seqlens,
                               const int32_t* slots, float* out, int n_seqs, int n_heads, int n_kv, int dim, int vdim,
@@ -406,7 +413,7 @@ static void launch_delta_rule(const float* q, const float* k, size_t qk_stride, 
   constexpr int COLS = RB_WAVE / RG;
   static_assert((DKL * RG * CH) % RB_WAVE == 0 && CH <= RB_WAVE && DKL % 4 == 0, "a chunk's values are dealt evenly to the lanes");
   dim3 grid(n_seqs, n_heads, (vdim + COLS - 1) / COLS);
-  delta_rule_kernel<DKL, RG, CH, BONUS><<<grid, RB_WAVE, 0, s>>>(q, k, qk_stride, v, v_stride, g, g_stride, beta, state, cu_seqlens,
+  delta_rule_kernel<DKL, RG, CH, MODE><<<grid, RB_WAVE, 0, s>>>(q, k, qk_stride, v, v_stride, g, g_stride, beta, state, cu_seqlens,
                                                                  slots, out, n_heads, n_kv, dim, vdim, g_per_head, bonus);
 }
 
@@ -431,6 +438,11 @@ extern "C" int rb_linear_recurrence(const float* q, const float* k, long long qk
                                     out, n_seqs, n_tokens, n_heads, n_kv_heads, dim, vdim, stream);
 }
 
+static int linear_recurrence_launch(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride,
+                                    const float* g, long long g_stride, int g_per_head, const float* beta, const float* bonus,
+                                    int silu_in, float* state, const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs,
+                                    int n_tokens, int n_heads, int n_kv_heads, int dim, int vdim, void* stream);
+
 // bonus (float32 [H, dim], null: rb_linear_recurrence): the plain rule read BEFORE the token's write, with the token's own
 // k v^T weighted per key channel:  out = (S + diag(bonus) k v^T)^T q;  S <- diag(g) S + k v^T.  Goes without beta.
 extern "C" int rb_linear_recurrence_bonus(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride,
@@ -440,10 +452,31 @@ extern "C" int rb_linear_recurrence_bonus(const float* q, const float* k, long l
                                           void* stream) {
   RB_RECORDED(rb_linear_recurrence_bonus(q, k, qk_stride, v, v_stride, g, g_stride, g_per_head, beta, bonus, state, cu_seqlens, slots,
                                          out, n_seqs, n_tokens, n_heads, n_kv_heads, dim, vdim, stream));
+  return linear_recurrence_launch(q, k, qk_stride, v, v_stride, g, g_stride, g_per_head, beta, bonus, 0, state, cu_seqlens, slots, out,
+                                  n_seqs, n_tokens, n_heads, n_kv_heads, dim, vdim, stream);
+}
+
+// The plain rule with one constant decay per head (decay float32 [H]) and silu on q, k and v as they are read:
+// S <- decay[h] S + k v^T, out = S^T q, token after token.  q and k have as many heads as v.
+extern "C" int rb_lightning_recurrence(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride,
+                                       const float* decay, float* state, const int32_t* cu_seqlens, const int32_t* slots, float* out,
+                                       int n_seqs, int n_tokens, int n_heads, int dim, int vdim, void* stream) {
+  RB_RECORDED(rb_lightning_recurrence(q, k, qk_stride, v, v_stride, decay, state, cu_seqlens, slots, out, n_seqs, n_tokens, n_heads, dim,
+                                      vdim, stream));
+  return linear_recurrence_launch(q, k, qk_stride, v, v_stride, decay, 0, 1, nullptr, nullptr, 1, state, cu_seqlens, slots, out, n_seqs,
+                                  n_tokens, n_heads, n_heads, dim, vdim, stream);
+}
+
+// silu_in: q, k and v go through silu as they are read; g_stride 0 (with g_per_head): the same decays for every token.
+static int linear_recurrence_launch(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride,
+                                    const float* g, long long g_stride, int g_per_head, const float* beta, const float* bonus,
+                                    int silu_in, float* state, const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs,
+                                    int n_tokens, int n_heads, int n_kv_heads, int dim, int vdim, void* stream) {
   RB_REQUIRE(bonus == nullptr || beta == nullptr, "rb_linear_recurrence: a bonus goes with the plain rule (no beta)");
   RB_REQUIRE(n_seqs >= 0 && n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0 && dim > 0 && vdim > 0,
              "rb_linear_recurrence: bad sizes H=%d Hk=%d dim=%d vdim=%d", n_heads, n_kv_heads, dim, vdim);
-  RB_REQUIRE(g_stride >= (long long)n_heads * (g_per_head ? 1 : dim), "rb_linear_recurrence: the decays' row stride is too short");
+  RB_REQUIRE((g_stride == 0 && g_per_head && silu_in) || g_stride >= (long long)n_heads * (g_per_head ? 1 : dim),
+             "rb_linear_recurrence: the decays' row stride is too short");
   RB_REQUIRE(dim <= 512, "rb_linear_recurrence: key size %d not supported (at most 512)", dim);
   RB_REQUIRE(n_heads <= 65535 && vdim <= 65535 * 4, "rb_linear_recurrence: too many heads or value channels");
   if (n_seqs == 0) return 0;
@@ -455,17 +488,23 @@ extern "C" int rb_linear_recurrence_bonus(const float* q, const float* k, long l
 #define DR_GO(DKL, RG, CH)                                                                                                  \
   do {                                                                                                                      \
     constexpr int CH1 = (DKL * RG >= RB_WAVE) ? 1 : RB_WAVE / (DKL * RG);                                                   \
-    if (single && bonus)                                                                                                    \
-      launch_delta_rule<DKL, RG, CH1, true>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,     \
+    if (single && silu_in)                                                                                                  \
+      launch_delta_rule<DKL, RG, CH1, 2>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,        \
+                                         n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                     \
+    else if (silu_in)                                                                                                       \
+      launch_delta_rule<DKL, RG, CH, 2>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,         \
+                                        n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                      \
+    else if (single && bonus)                                                                                               \
+      launch_delta_rule<DKL, RG, CH1, 1>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,     \
                                             n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                  \
     else if (single)                                                                                                        \
-      launch_delta_rule<DKL, RG, CH1, false>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,    \
+      launch_delta_rule<DKL, RG, CH1, 0>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,    \
                                              n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                 \
     else if (bonus)                                                                                                         \
-      launch_delta_rule<DKL, RG, CH, true>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,      \
+      launch_delta_rule<DKL, RG, CH, 1>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,      \
                                            n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                   \
     else                                                                                                                    \
-      launch_delta_rule<DKL, RG, CH, false>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,     \
+      launch_delta_rule<DKL, RG, CH, 0>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,     \
                                             n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                  \
   } while (0)
   // Rows of a column over RG lanes, chunks as long as the registers that hold the next one allow.  A token's time is
@@ -513,6 +552,73 @@ __global__ void gated_rmsnorm_kernel(const float* __restrict__ o, const float* _
   const float f = 1.0f / sqrtf(ss / (float)vdim + eps);
   for (int i = lane; i < vdim; i += RB_WAVE)
     Num<TO>::store(out + (size_t)pair * vdim + i, p[i] * f * wp[i] * (act == 1 ? gp[i] * rb_sigmoid(gp[i]) : rb_sigmoid(gp[i])));
+}
+
+// The same for rows of many numbers (one norm over all heads together): a workgroup a row, 16-byte accesses where they fit.
+template <typename TO, bool VEC>
+__global__ __launch_bounds__(1024) void gated_rmsnorm_row_kernel(const float* __restrict__ o, const float* __restrict__ weight,
+                                                                 const float* __restrict__ gate, size_t gate_stride, float eps,
+                                                                 TO* __restrict__ out, int width, int act) {
+  __shared__ float scratch[16];
+  const size_t t = blockIdx.x;
+  const float* p = o + t * width;
+  const float* gp = gate + t * gate_stride;
+  auto gated = [&](float g) { return act == 1 ? g * rb_sigmoid(g) : rb_sigmoid(g); };
+  float ss = 0.f;
+  if (VEC) {
+    const int j0 = 4 * threadIdx.x;
+    float4 keep = make_float4(0.f, 0.f, 0.f, 0.f), g0 = keep;
+    for (int j = j0; j < width; j += 4 * blockDim.x) {
+      const float4 v = *reinterpret_cast<const float4*>(p + j);
+      if (j == j0) {
+        keep = v;
+        g0 = *reinterpret_cast<const float4*>(gp + j);
+      }
+      ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+    }
+    const float f = 1.0f / sqrtf(block_sum(ss, scratch) / (float)width + eps);
+    for (int j = j0; j < width; j += 4 * blockDim.x) {
+      const float4 v = j == j0 ? keep : *reinterpret_cast<const float4*>(p + j);
+      const float4 g = j == j0 ? g0 : *reinterpret_cast<const float4*>(gp + j);
+      const float4 w = *reinterpret_cast<const float4*>(weight + j);
+      const float a = v.x * f * w.x * gated(g.x), b = v.y * f * w.y * gated(g.y), c = v.z * f * w.z * gated(g.z),
+                  d = v.w * f * w.w * gated(g.w);
+      if (sizeof(TO) == 4)
+        *reinterpret_cast<float4*>(out + t * width + j) = make_float4(a, b, c, d);
+      else
+        *reinterpret_cast<uint2*>(out + t * width + j) = make_uint2(pack_bf16x2(a, b), pack_bf16x2(c, d));
+    }
+  } else {
+    for (int j = threadIdx.x; j < width; j += blockDim.x) ss = fmaf(p[j], p[j], ss);
+    const float f = 1.0f / sqrtf(block_sum(ss, scratch) / (float)width + eps);
+    for (int j = threadIdx.x; j < width; j += blockDim.x) Num<TO>::store(out + t * width + j, p[j] * f * weight[j] * gated(gp[j]));
+  }
+}
+
+// out[t, :] = o[t, :] / sqrt(mean(o[t, :]^2) + eps) * weight * act(gate[t, :]) over the whole row (act 0: sigmoid, 1: silu).
+extern "C" int rb_gated_rmsnorm_rows(const float* o, const float* weight, const float* gate, long long gate_stride, int act, float eps,
+                                     void* out, int out_dtype, int n_tokens, int width, void* stream) {
+  RB_RECORDED(rb_gated_rmsnorm_rows(o, weight, gate, gate_stride, act, eps, out, out_dtype, n_tokens, width, stream));
+  RB_REQUIRE(n_tokens >= 0 && width > 0 && (act == 0 || act == 1) && gate_stride >= width, "rb_gated_rmsnorm_rows: bad sizes");
+  RB_REQUIRE(out_dtype == RB_F32 || out_dtype == RB_BF16, "rb_gated_rmsnorm_rows: unknown dtype %d", out_dtype);
+  if (n_tokens == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = width % 4 == 0 && gate_stride % 4 == 0 && aligned(o) && aligned(weight) && aligned(gate) && aligned(out);
+  int threads = ((width / (vec ? 4 : 1) + RB_WAVE - 1) / RB_WAVE) * RB_WAVE;
+  threads = threads > 1024 ? 1024 : (threads < RB_WAVE ? RB_WAVE : threads);
+#define RB_GR(TO, VEC) \
+  gated_rmsnorm_row_kernel<TO, VEC><<<n_tokens, threads, 0, s>>>(o, weight, gate, (size_t)gate_stride, eps, (TO*)out, width, act)
+  if (out_dtype == RB_F32) {
+    if (vec) RB_GR(float, true);
+    else RB_GR(float, false);
+  } else {
+    if (vec) RB_GR(bf16_t, true);
+    else RB_GR(bf16_t, false);
+  }
+#undef RB_GR
+  RB_LAUNCH_CHECK();
+  return 0;
 }
 
 extern "C" int rb_gated_rmsnorm(const float* o, const float* weight, const float* gate, long long gate_stride, float eps,

@@ -26,19 +26,18 @@
 
 // ---------------------------------------------------------------- route
 // score 0: sigmoid(z) of the chosen logit.  score 1: the softmax of z over all outputs; the choice then goes by the
-// softmax plus `correction` (null: nothing added), the weight is the softmax itself.
-__global__ void route_kernel(const float* __restrict__ z, size_t z_stride, int n_experts, int top, int score,
-                             const float* __restrict__ correction, int32_t* __restrict__ sel, float* __restrict__ weight,
-                             int n_tokens) {
-  const int t = blockIdx.x * (blockDim.x / RB_WAVE) + threadIdx.x / RB_WAVE;
-  if (t >= n_tokens) return;
+// softmax plus `correction` (null: nothing added), the weight is the softmax itself.  score 2: the choice goes by the logits,
+// the weights are the softmax over the chosen logits alone.  bias (null: none) is added to the logits before anything else.
+__device__ void route_token(const float* __restrict__ z, size_t z_stride, int n_experts, int top, int score,
+                            const float* __restrict__ bias, const float* __restrict__ correction, int32_t* __restrict__ sel,
+                            float* __restrict__ weight, int t) {
   const int lane = threadIdx.x & (RB_WAVE - 1);
   constexpr int PER = RT_MAX_EXPERTS / RB_WAVE;
   float v[PER];
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
     const int e = lane + RB_WAVE * j;
-    v[j] = e < n_experts ? z[(size_t)t * z_stride + e] : -INFINITY;
+    v[j] = e < n_experts ? z[(size_t)t * z_stride + e] + (bias ? bias[e] : 0.f) : -INFINITY;
     if (v[j] != v[j]) v[j] = -INFINITY;
   }
   float own[PER];                    // score 1: the softmax, kept beside what the choice goes by
@@ -62,6 +61,7 @@ __global__ void route_kernel(const float* __restrict__ z, size_t z_stride, int n
       if (v[j] != v[j]) v[j] = -INFINITY;
     }
   }
+  float first = 0.f, chosen_sum = 0.f, mine = 0.f;      // score 2: the largest logit, the sum of exp(logit - largest), lane k's own of these
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY;
     int at = 0x7fffffff;
@@ -83,7 +83,12 @@ __global__ void route_kernel(const float* __restrict__ z, size_t z_stride, int n
       }
     }
     if (at == 0x7fffffff) at = k < n_experts ? k : 0;        // every logit was NaN or -inf: any expert, never out of range
-    if (score == 1) {                   // the chosen output's softmax: from the lane that holds it
+    if (score == 2) {
+      if (k == 0) first = best;
+      best = (best == -INFINITY) ? 0.f : expf(best - first);
+      chosen_sum += best;
+      if ((k & (RB_WAVE - 1)) == lane && k < RB_WAVE) mine = best;
+    } else if (score == 1) {            // the chosen output's softmax: from the lane that holds it
       float w = 0.f;
 #pragma unroll
       for (int j = 0; j < PER; ++j)
@@ -94,18 +99,29 @@ __global__ void route_kernel(const float* __restrict__ z, size_t z_stride, int n
     }
     if (lane == 0) {
       sel[(size_t)t * top + k] = at;
-      weight[(size_t)t * top + k] = best;
+      if (score != 2) weight[(size_t)t * top + k] = best;
     }
 #pragma unroll
     for (int j = 0; j < PER; ++j)
       if (lane + RB_WAVE * j == at) v[j] = -INFINITY;
   }
+  if (score == 2) {
+    // every logit -infinity or NaN: equal weights
+    const float inv = chosen_sum > 0.f ? 1.0f / chosen_sum : 0.f;
+    if (lane < top) weight[(size_t)t * top + lane] = inv > 0.f ? mine * inv : 1.0f / (float)top;
+  }
+}
+
+__global__ void route_kernel(const float* __restrict__ z, size_t z_stride, int n_experts, int top, int score,
+                             const float* __restrict__ bias, const float* __restrict__ correction, int32_t* __restrict__ sel,
+                             float* __restrict__ weight, int n_tokens) {
+  const int t = blockIdx.x * (blockDim.x / RB_WAVE) + threadIdx.x / RB_WAVE;
+  if (t < n_tokens) route_token(z, z_stride, n_experts, top, score, bias, correction, sel, weight, t);
 }
 
 // ---------------------------------------------------------------- sort (one workgroup)
-__global__ __launch_bounds__(1024) void route_sort_kernel(const int32_t* __restrict__ sel, int n_pairs, int n_experts,
-                                                          int32_t* __restrict__ row_pair, int32_t* __restrict__ tile_expert,
-                                                          int32_t* __restrict__ tile_pos, int max_rows) {
+__device__ void route_sort(const int32_t* sel, int n_pairs, int n_experts, int32_t* __restrict__ row_pair,
+                           int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_pos, int max_rows) {
   __shared__ int counts[RT_MAX_EXPERTS], offs[RT_MAX_EXPERTS], cursor[RT_MAX_EXPERTS];
   for (int e = threadIdx.x; e < n_experts; e += blockDim.x) counts[e] = cursor[e] = 0;
   __syncthreads();
@@ -133,22 +149,56 @@ __global__ __launch_bounds__(1024) void route_sort_kernel(const int32_t* __restr
   }
 }
 
+__global__ __launch_bounds__(1024) void route_sort_kernel(const int32_t* __restrict__ sel, int n_pairs, int n_experts,
+                                                          int32_t* __restrict__ row_pair, int32_t* __restrict__ tile_expert,
+                                                          int32_t* __restrict__ tile_pos, int max_rows) {
+  route_sort(sel, n_pairs, n_experts, row_pair, tile_expert, tile_pos, max_rows);
+}
+
+// A step of few tokens: the choice (a wave a token) and the sort in one launch of one workgroup.
+__global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict__ z, size_t z_stride, int n_outputs, int n_experts,
+                                                         int top, int score, const float* __restrict__ bias,
+                                                         const float* __restrict__ correction, int32_t* sel,
+                                                         float* __restrict__ weight, int n_tokens, int32_t* __restrict__ row_pair,
+                                                         int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_pos, int max_rows) {
+  for (int t = threadIdx.x / RB_WAVE; t < n_tokens; t += blockDim.x / RB_WAVE)
+    route_token(z, z_stride, n_outputs, top, score, bias, correction, sel, weight, t);
+  __threadfence_block();
+  __syncthreads();
+  route_sort(sel, n_tokens * top, n_experts, row_pair, tile_expert, tile_pos, max_rows);
+}
+
 extern "C" int rb_route_choose(const float* z, long long z_stride, int n_outputs, int n_experts, int top, int score,
                                const float* correction, int32_t* sel, float* weight, int32_t* row_pair, int32_t* tile_expert,
                                int max_rows, int n_tokens, void* stream) {
-  RB_RECORDED(rb_route_choose(z, z_stride, n_outputs, n_experts, top, score, correction, sel, weight, row_pair, tile_expert, max_rows,
-                              n_tokens, stream));
+  return rb_route_choose_bias(z, z_stride, nullptr, n_outputs, n_experts, top, score, correction, sel, weight, row_pair, tile_expert,
+                              max_rows, n_tokens, stream);
+}
+
+#define RT_FEW_TOKENS 32       // up to so many tokens the choice and the sort are one launch
+extern "C" int rb_route_choose_bias(const float* z, long long z_stride, const float* bias, int n_outputs, int n_experts, int top,
+                                    int score, const float* correction, int32_t* sel, float* weight, int32_t* row_pair,
+                                    int32_t* tile_expert, int max_rows, int n_tokens, void* stream) {
+  RB_RECORDED(rb_route_choose_bias(z, z_stride, bias, n_outputs, n_experts, top, score, correction, sel, weight, row_pair, tile_expert,
+                                   max_rows, n_tokens, stream));
   RB_REQUIRE(n_tokens >= 0 && n_experts >= 0 && n_outputs >= n_experts && n_outputs > 0 && n_outputs <= RT_MAX_EXPERTS && top > 0 &&
                  top <= n_outputs && z_stride >= n_outputs,
              "rb_route_choose: bad sizes T=%d outputs=%d (at most %d) experts=%d top=%d", n_tokens, n_outputs, RT_MAX_EXPERTS, n_experts, top);
-  RB_REQUIRE(score == 0 || score == 1, "rb_route_choose: score %d is neither the sigmoid (0) nor the softmax (1)", score);
+  RB_REQUIRE(score >= 0 && score <= 2, "rb_route_choose: score %d is neither the sigmoid (0), the softmax (1) nor the softmax over the chosen (2)", score);
+  RB_REQUIRE(score != 2 || top <= RB_WAVE, "rb_route_choose: the softmax over the chosen takes at most %d of them, not %d", RB_WAVE, top);
   RB_REQUIRE(correction == nullptr || score == 1, "rb_route_choose: a correction goes with the softmax");
   const long long pairs = (long long)n_tokens * top;
   RB_REQUIRE(max_rows % RT_TILE == 0 && max_rows >= (pairs + RT_TILE - 1) / RT_TILE * RT_TILE + (long long)RT_TILE * n_experts,
              "rb_route_choose: room for %d rows, %lld pairs of %d experts may need more", max_rows, pairs, n_experts);
   if (n_tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-  route_kernel<<<(n_tokens + 3) / 4, 256, 0, s>>>(z, (size_t)z_stride, n_outputs, top, score, correction, sel, weight, n_tokens);
+  if (n_tokens <= RT_FEW_TOKENS) {
+    route_few_kernel<<<1, 1024, 0, s>>>(z, (size_t)z_stride, n_outputs, n_experts, top, score, bias, correction, sel, weight, n_tokens,
+                                        row_pair, tile_expert, tile_expert + max_rows / RT_TILE, max_rows);
+    RB_LAUNCH_CHECK();
+    return 0;
+  }
+  route_kernel<<<(n_tokens + 3) / 4, 256, 0, s>>>(z, (size_t)z_stride, n_outputs, top, score, bias, correction, sel, weight, n_tokens);
   route_sort_kernel<<<1, 1024, 0, s>>>(sel, (int)pairs, n_experts, row_pair, tile_expert, tile_expert + max_rows / RT_TILE, max_rows);
   RB_LAUNCH_CHECK();
   return 0;

@@ -379,3 +379,140 @@ extern "C" int rb_tanh_cap(float* x, float cap, long long n, void* stream) {
   RB_LAUNCH_CHECK();
   return 0;
 }
+
+// ---------------------------------------------------------------- a norm that is an element-wise tanh
+// norm(v) = tanh(alpha v) w + b, number by number (alpha one number, w and b a row).  In one pass over the rows:
+//   v = x[src] + after(y[src]);  without rows x[src] = v;  out[r] = before(v),    src = rows ? rows[r] : r
+// where after is the norm on a sublayer's output (a1, w1, b1; a1 null: y is added as it is) and before the one in front of the
+// next sublayer (a2, w2, b2; out null: none).  y is a sum of n_terms terms, term_stride floats apart, a row of them row_stride
+// apart (K slices of a product, or the outputs of a token's experts), term k times weights[src * n_terms + k] where given;
+// y null: nothing is added.  A thread keeps the parameters of its columns and walks rows.
+struct TanhNormArgs {
+  float* x;
+  const float* y;
+  int n_terms;
+  size_t term_stride, row_stride;
+  const float* weights;
+  const float *a1, *w1, *b1, *a2, *w2, *b2;
+  const int32_t* rows;
+  int n_rows, width;
+};
+
+// tanh on the hardware's exponential and reciprocal: (1 - e) / (1 + e) with e = exp(-2 |z|), within 2e-7 of the function
+__device__ __forceinline__ float tanh_fast(float z) {
+  const float e = __builtin_amdgcn_exp2f(-2.8853900817779268f * fabsf(z));
+  return copysignf((1.0f - e) * __builtin_amdgcn_rcpf(1.0f + e), z);
+}
+template <typename TO>
+__device__ __forceinline__ float tanh_norm_value(float z) { return tanh_fast(z); }
+template <>
+__device__ __forceinline__ float tanh_norm_value<float>(float z) { return tanhf(z); }
+
+template <typename TO, int V>
+__global__ __launch_bounds__(256) void tanh_norm_kernel(TanhNormArgs p, TO* __restrict__ out) {
+  const int j = V * (blockIdx.x * blockDim.x + threadIdx.x);
+  if (j >= p.width) return;
+  float w1[V], b1[V], w2[V], b2[V];
+  const float a1 = p.a1 ? *p.a1 : 0.f, a2 = p.a2 ? *p.a2 : 0.f;
+  auto load = [&](float* d, const float* s) {
+    if (V == 4) {
+      const float4 v = ld4(s);
+      d[0] = v.x;
+      d[V > 1 ? 1 : 0] = v.y;
+      d[V > 2 ? 2 : 0] = v.z;
+      d[V - 1] = v.w;
+    } else {
+      d[0] = *s;
+    }
+  };
+  if (p.a1) {
+    load(w1, p.w1 + j);
+    load(b1, p.b1 + j);
+  }
+  if (out) {
+    load(w2, p.w2 + j);
+    load(b2, p.b2 + j);
+  }
+  for (int r = blockIdx.y; r < p.n_rows; r += gridDim.y) {
+    const size_t src = p.rows ? (size_t)p.rows[r] : (size_t)r;
+    float v[V];
+    load(v, p.x + src * p.width + j);
+    if (p.y) {
+      const float* yp = p.y + src * p.row_stride + j;
+      const float* wp = p.weights ? p.weights + src * p.n_terms : nullptr;
+      float acc[V];
+#pragma unroll
+      for (int i = 0; i < V; ++i) acc[i] = 0.f;
+      int k = 0;
+      for (; k + 3 < p.n_terms; k += 4) {               // four terms in flight
+        float e[4][V];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) load(e[u], yp + (size_t)(k + u) * p.term_stride);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const float f = wp ? wp[k + u] : 1.0f;
+#pragma unroll
+          for (int i = 0; i < V; ++i) acc[i] = fmaf(f, e[u][i], acc[i]);
+        }
+      }
+      for (; k < p.n_terms; ++k) {
+        float e[V];
+        load(e, yp + (size_t)k * p.term_stride);
+        const float f = wp ? wp[k] : 1.0f;
+#pragma unroll
+        for (int i = 0; i < V; ++i) acc[i] = fmaf(f, e[i], acc[i]);
+      }
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] += p.a1 ? fmaf(tanh_norm_value<TO>(a1 * acc[i]), w1[i], b1[i]) : acc[i];
+      if (!p.rows) {
+        float* xd = p.x + src * p.width + j;
+        if (V == 4) st4(xd, v[0], v[V > 1 ? 1 : 0], v[V > 2 ? 2 : 0], v[V - 1]);
+        else *xd = v[0];
+      }
+    }
+    if (out) {
+      float o[V];
+#pragma unroll
+      for (int i = 0; i < V; ++i) o[i] = fmaf(tanh_norm_value<TO>(a2 * v[i]), w2[i], b2[i]);
+      TO* od = out + (size_t)r * p.width + j;
+      if (V == 4) st4(od, o[0], o[V > 1 ? 1 : 0], o[V > 2 ? 2 : 0], o[V - 1]);
+      else Num<TO>::store(od, o[0]);
+    }
+  }
+}
+
+extern "C" int rb_tanh_norm(float* x, const float* y, int n_terms, long long term_stride, long long row_stride, const float* weights,
+                            const float* a1, const float* w1, const float* b1, const float* a2, const float* w2, const float* b2,
+                            const int32_t* rows, int n_rows, int width, void* out, int out_dtype, void* stream) {
+  RB_RECORDED(rb_tanh_norm(x, y, n_terms, term_stride, row_stride, weights, a1, w1, b1, a2, w2, b2, rows, n_rows, width, out, out_dtype,
+                           stream));
+  RB_REQUIRE(n_rows >= 0 && width > 0 && x != nullptr, "rb_tanh_norm: bad sizes %d x %d", n_rows, width);
+  RB_REQUIRE(y == nullptr || (n_terms >= 1 && term_stride >= 0 && row_stride >= width), "rb_tanh_norm: bad terms");
+  RB_REQUIRE(a1 == nullptr || (w1 != nullptr && b1 != nullptr), "rb_tanh_norm: a norm needs its weight and bias");
+  RB_REQUIRE(out == nullptr || (a2 != nullptr && w2 != nullptr && b2 != nullptr), "rb_tanh_norm: a norm needs its weight and bias");
+  RB_REQUIRE(out != nullptr || (y != nullptr && rows == nullptr), "rb_tanh_norm: nothing to do");
+  RB_REQUIRE(out_dtype == RB_F32 || out_dtype == RB_BF16, "rb_tanh_norm: unknown dtype %d", out_dtype);
+  if (n_rows == 0) return 0;
+  TanhNormArgs p = {x, y, n_terms, (size_t)term_stride, (size_t)row_stride, weights, a1, w1, b1, a2, w2, b2, rows, n_rows, width};
+  auto aligned = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
+  const bool vec = width % 4 == 0 && term_stride % 4 == 0 && row_stride % 4 == 0 && aligned(x) && aligned(y) && aligned(w1) && aligned(b1) &&
+                   aligned(w2) && aligned(b2) && aligned(out);
+  const int cols = vec ? width / 4 : width;
+  // few rows: small workgroups spread over the compute units; many: as many workgroups as keep them busy, each walking rows
+  const int threads = (long long)n_rows * ((cols + 255) / 256) >= rb_compute_units() ? 256 : RB_WAVE;
+  const int gx = (cols + threads - 1) / threads;
+  int gy = (8 * rb_compute_units() + gx - 1) / gx;
+  if (gy > n_rows) gy = n_rows;
+  if (gy > 65535) gy = 65535;
+  dim3 grid(gx, gy);
+  hipStream_t s = (hipStream_t)stream;
+  if (out_dtype == RB_F32) {
+    if (vec) tanh_norm_kernel<float, 4><<<grid, threads, 0, s>>>(p, (float*)out);
+    else tanh_norm_kernel<float, 1><<<grid, threads, 0, s>>>(p, (float*)out);
+  } else {
+    if (vec) tanh_norm_kernel<bf16_t, 4><<<grid, threads, 0, s>>>(p, (bf16_t*)out);
+    else tanh_norm_kernel<bf16_t, 1><<<grid, threads, 0, s>>>(p, (bf16_t*)out);
+  }
+  RB_LAUNCH_CHECK();
+  return 0;
+}

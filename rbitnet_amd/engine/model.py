@@ -118,8 +118,8 @@ class Model:
             if not earlier:
                 raise ConfigError(f"layer {i} reads the cache of layer {j}, which does not run before it")
             out[place] = earlier[-1]
-            own = getattr(self.blocks[i].mixer, "window", None)
-            theirs = getattr(self.blocks[int(j)].mixer, "window", None)
+            reach = lambda mixer: getattr(mixer, "reach", getattr(mixer, "window", None))
+            own, theirs = reach(self.blocks[i].mixer), reach(self.blocks[int(j)].mixer)
             if theirs is not None and (own is None or int(own) > int(theirs)):
                 raise ConfigError(
                     f"layer {i} looks back {own or 'without limit'} but reads the cache of layer {j}, "

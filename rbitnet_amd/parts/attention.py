@@ -27,8 +27,8 @@ and four more, each of which sends the layer through the kernels that take all h
               "talk" [heads, heads] (float32);
   chunk       None, or c: a query at position i sees the keys j <= i with i // c == j // c only, chunks being counted
               from the sequence's first position, whatever a step brings.
-These go without a rotation (position "none") and without a sink.
-Five more send the layer through a third way, in which q, k and v are prepared by kernels of their own in front of attention
+These go without a rotation (position "none") and without a sink.  (A chunk also goes with everything below.)
+Eight more send the layer through a third way, in which q, k and v are prepared by kernels of their own in front of attention
 (biases and a norm with a weight belong to it too, and a rotation is welcome):
   conv        None, or the taps of a short causal convolution over time on every channel of q, k and v (tensors "q_conv",
               "k_conv", "v_conv" [channels, taps], no bias), directly behind the projection and its bias; the last taps - 1
@@ -37,6 +37,11 @@ Five more send the layer through a third way, in which q, k and v are prepared b
               share (tensors "q_norm", "k_norm"), x / sqrt(mean(x^2) + e) * w, before the rotation;
   softcap     None, or c: score <- c tanh(score / c) after the scale;
   keep_first  with a window: the first keep_first tokens of a sequence stay visible behind it (at their own positions);
+  qk_norm     {"eps": e, "weight": True, "over": "projection"}: one norm over all of q's numbers (every head together, tensor
+              "q_norm" [heads * head_dim]) and one over all of k's ("k_norm" [kv_heads * head_dim]) instead, before the rotation;
+  value_norm  None, or e: every value head is divided by sqrt(mean(head^2) + e) (no weight) and cached so;
+  weights     "sigmoid": a visible key's weight is sigmoid(score + b[head]) by itself, not normalised over the keys, b the
+              tensor "score_bias" [heads] (float32); "softmax" otherwise;
   gate        "elementwise": the concatenated heads are multiplied number by number with sigmoid(Wg h) (tensor "gate"
               [heads * value_dim, E]) before the output matrix.
 A position part that rotates only the first numbers of a head says so with its own head_dim
@@ -69,7 +74,8 @@ from .short_conv import ACT_NONE, ShortConv
 
 DEFAULT_NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight", "sink": "sink",
                  "gate": "gate", "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "talk": "talk",
-                 "q_conv": "q.conv", "k_conv": "k.conv", "v_conv": "v.conv", "q_norm": "q.norm", "k_norm": "k.norm"}
+                 "q_conv": "q.conv", "k_conv": "k.conv", "v_conv": "v.conv", "q_norm": "q.norm", "k_norm": "k.norm",
+                 "score_bias": "score_bias"}
 MIXED_MAX_HEADS, MIXED_MAX_NUMBERS = 64, 8192      # what the kernels that take all heads of a token together hold
 MIXED_MATRIX_CORE_HEADS = 32                       # and the one on the matrix cores
 _MATRIX_CORE_HEAD_DIMS = (64, 128)
@@ -81,6 +87,7 @@ class Attention(Part):
     plan_safe = True
     takes_gained_rows = True
     adds_to_stream = True
+    leaves_terms = True
 
     def __init__(self, params: Dict, env: BuildEnv):
         self.env = env
@@ -122,6 +129,19 @@ class Attention(Part):
         # q, k and v prepared in front of attention: whenever one of these is asked for
         self.taps = None if params.get("conv") is None else int(params["conv"])
         self.qk_weight = bool(qk_norm and qk_norm.get("weight"))
+        over = str((qk_norm or {}).get("over", "head"))
+        if over not in ("head", "projection") or (over == "projection" and not self.qk_weight):
+            raise ConfigError(f"attention: a norm of q and k is over the 'head' or, with a weight, over the 'projection', found {over!r}")
+        self.whole_norm = over == "projection"
+        self.value_eps = None if params.get("value_norm") is None else float(params["value_norm"])
+        kind = str(params.get("weights") or "softmax")
+        if kind not in ("softmax", "sigmoid"):
+            raise ConfigError(f"attention: unknown weights {kind!r} (softmax, sigmoid)")
+        self.sigmoid = kind == "sigmoid"
+        if self.sigmoid and self.has_sink:
+            raise ConfigError("attention: a sink belongs to the softmax")
+        if self.value_eps is not None and self.qk_eps is not None and not (self.whole_norm and self.value_eps == self.qk_eps):
+            raise ConfigError("attention: a norm of the values goes with norms over the projections that share its eps, or with none")
         self.softcap = None if params.get("softcap") is None else float(params["softcap"])
         self.keep_first = int(params.get("keep_first") or 0)
         self.gate_kind = str(params.get("gate") or ("head" if self.has_gate else "none"))
@@ -133,10 +153,10 @@ class Attention(Part):
         if self.keep_first < 0 or (self.keep_first and self.window is None):
             raise ConfigError("attention: kept first tokens go with a window")
         self.prepared = bool(self.taps is not None or self.qk_weight or self.softcap is not None or self.keep_first
-                             or self.gate_kind == "elementwise")
-        if self.prepared and (self.has_talk or self.chunk is not None):
-            raise ConfigError("attention: mixed heads and chunks go without a convolution, weighted norms, capped scores, "
-                              "kept first tokens and an elementwise gate")
+                             or self.gate_kind == "elementwise" or self.value_eps is not None or self.sigmoid)
+        if self.prepared and self.has_talk:
+            raise ConfigError("attention: mixed heads go without a convolution, weighted norms, capped scores, "
+                              "kept first tokens, an elementwise gate, norms of the values and sigmoid weights")
         self.conv = None
         if self.prepared and (self.taps is not None or self.has_bias):
             # a bias alone runs as a convolution of one tap (of ones): the same kernel adds it
@@ -144,6 +164,12 @@ class Attention(Part):
             if self.cache_from is None:
                 n_ch += self.n_kv * (self.head_dim + self.value_dim)
             self.conv = ShortConv(n_ch, self.taps or 1, env, residual=False, act=ACT_NONE)
+        if self.prepared and (self.sigmoid or self.whole_norm) and env.dtype == torch.bfloat16 and not getattr(env, "generic_only", False):
+            # a head size of the matrix cores' kernels where one is near (zeros cost cache, not correctness)
+            for size in _MATRIX_CORE_HEAD_DIMS:
+                if self.pad <= size and 2 * self.pad >= size:
+                    self.pad = size
+                    break
         # all heads of a token in one workgroup: whenever one of the four is asked for
         self.mixed = (not self.prepared) and (self.has_bias or self.has_talk or self.qk_eps is not None or self.chunk is not None)
         if self.mixed:
@@ -188,9 +214,12 @@ class Attention(Part):
                 specs[self.names["k_conv"]] = gain(kd)
                 specs[self.names["v_conv"]] = gain(self.n_kv * self.value_dim)
         if self.qk_weight:
-            specs[self.names["q_norm"]] = TensorSpec((self.head_dim,), role="gain", init="ones_normal")
+            nq, nk = (qd, kd) if self.whole_norm else (self.head_dim, self.head_dim)
+            specs[self.names["q_norm"]] = TensorSpec((nq,), role="gain", init="ones_normal")
             if self.cache_from is None:
-                specs[self.names["k_norm"]] = TensorSpec((self.head_dim,), role="gain", init="ones_normal")
+                specs[self.names["k_norm"]] = TensorSpec((nk,), role="gain", init="ones_normal")
+        if self.sigmoid:
+            specs[self.names["score_bias"]] = TensorSpec((self.n_heads,), role="gain", init="normal")
         return specs
 
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
@@ -241,17 +270,24 @@ class Attention(Part):
                 self.conv.load(torch.cat([tensors[self.names[n + "_conv"]] for n in names]))
             else:
                 self.conv.load(torch.ones((self.conv.channels, 1), dtype=torch.float32, device=o.device))
+        self.score_bias = tensors[self.names["score_bias"]].contiguous() if self.sigmoid else None
         if self.qk_weight:
             self.q_norm_w = tensors[self.names["q_norm"]]
             self.k_norm_w = tensors[self.names["k_norm"]] if self.cache_from is None else None
         elif self.prepared and self.qk_eps is not None:
             self.q_norm_w = self.k_norm_w = torch.ones(self.head_dim, dtype=torch.float32, device=o.device)
 
+    @property
+    def reach(self) -> Optional[int]:
+        """How far back a query looks (None: to the sequence's start), so that the cache may give pages behind it back: the
+        window, or the chunk (no query looks further back than its chunk is long)."""
+        both = [int(w) for w in (self.window, self.chunk if self.prepared and not self.keep_first else None) if w is not None]
+        return min(both) if both else None
+
     def cache_request(self) -> Optional[CacheRequest]:
         if self.cache_from is not None:
             return None
-        return CacheRequest("kv", heads=self.n_kv, head_dim=self.pad,
-                            window=None if self.window is None else int(self.window), keep_first=self.keep_first)
+        return CacheRequest("kv", heads=self.n_kv, head_dim=self.pad, window=self.reach, keep_first=self.keep_first)
 
     def cache_requests(self):
         out = [r for r in (self.cache_request(),) if r is not None]
@@ -279,10 +315,15 @@ class Attention(Part):
             qkv = self.conv.forward(qkv, ctx, view.states.get("qkv_conv"), torch.float32, bias=self.bias)
         q = torch.empty((t, hq, d), dtype=self.env.dtype, device=h.device)
         cos, sin, style = self.position.rotation_tables() if self.rot else (None, None, 1)
-        if self.rot and style != 1:
-            raise ConfigError("attention: a head prepared in front of attention pairs i with i + rot / 2 (style 'half')")
         k_pages, v_pages = (view.k_pages, view.v_pages) if owns else (None, None)
-        if self.qk_eps is not None:
+        if self.whole_norm or self.value_eps is not None or (self.qk_eps is None and style == 0 and self.rot):
+            norms = (self.q_norm_w, self.k_norm_w) if self.whole_norm else (None, None)
+            lib.heads_prepare(qkv, cos, sin, self.rot, style, norms[0], norms[1], self.value_eps is not None,
+                              self.qk_eps if self.whole_norm else (self.value_eps or 0.0), q, k_pages, v_pages, ctx.tok_pos, ctx.tok_seq,
+                              view.block_table, hq, hk, self.head_dim, self.value_dim, d)
+        elif self.rot and style != 1:
+            raise ConfigError("attention: heads with a norm of each in front of the rotation pair i with i + rot / 2 (style 'half')")
+        elif self.qk_eps is not None:
             lib.norm_rope_store(qkv, cos, sin, self.rot, self.q_norm_w, self.k_norm_w, self.qk_eps, q, k_pages, v_pages,
                                 ctx.tok_pos, ctx.tok_seq, view.block_table, hq, hk, self.head_dim, self.value_dim, d)
         else:
@@ -295,14 +336,16 @@ class Attention(Part):
             n_splits, workspace = ctx.decode_workspace(hq, d, hk)
             lib.attention_decode_bf16(q, view.k_pages, view.v_pages, attn, ctx.tok_pos, view.block_table, hq, hk, d, self.scale,
                                       window, n_splits, workspace, sinks=self.sink, keep_first=self.keep_first,
-                                      softcap=self.softcap or 0.0)
+                                      softcap=self.softcap or 0.0, chunk=self.chunk or 0, sig_bias=self.score_bias)
         elif fast:
             lib.attention_prefill_bf16(q, view.k_pages, view.v_pages, attn, ctx.cu_seqlens, ctx.past_len, view.block_table,
                                        ctx.n_seqs, ctx.max_q_len, hq, hk, d, self.scale, window, sinks=self.sink,
-                                       keep_first=self.keep_first, softcap=self.softcap or 0.0)
+                                       keep_first=self.keep_first, softcap=self.softcap or 0.0, chunk=self.chunk or 0,
+                                       sig_bias=self.score_bias)
         else:
             lib.attention_opts(q, view.k_pages, view.v_pages, attn, ctx.tok_pos, ctx.tok_seq, view.block_table, hq, hk, d,
-                               self.scale, window, self.keep_first, self.softcap or 0.0, self.sink)
+                               self.scale, window, self.keep_first, self.softcap or 0.0, self.sink, chunk=self.chunk or 0,
+                               sig_bias=self.score_bias)
         return self._gate_and_project(attn, h, stream, next_norm)
 
     def _forward_mixed(self, h, ctx, view, stream, next_norm):

@@ -32,7 +32,8 @@ import torch
 from .base import BuildEnv, Part, TensorSpec, build_part, register_block
 from ..errors import ConfigError
 from .short_conv import ACT_NONE, ShortConv
-from .stream import GainedRows, ScaledSum, StreamCopy, WeightedTerms, normed_for, sublayer  # noqa: F401  (normed_for: its old home)
+from .stream import (GainedRows, NormedTerm, ScaledSum, StreamCopy, WeightedTerms, norm_adds_terms, normed_for,  # noqa: F401
+                     sublayer)                                                  # (normed_for: its old home)
 
 DEFAULT_SEGMENTS = {"norm1": "input_layernorm", "mixer": "self_attn", "norm2": "post_attention_layernorm",
                     "feed_forward": "mlp"}
@@ -253,6 +254,81 @@ class OutNormBlock:
         return StreamCopy(h)
 
 
+class SandwichBlock:
+    """"sandwich": a norm in front of each sublayer and one on its output:
+        x += norm1b(mixer(norm1(x)));  x += norm2b(feed_forward(norm2(x)))
+    The feed-forward (with norm2 and norm2b) may be left out.  The norms on the outputs must offer `add_normed`; where the norm
+    that reads the stream next says `adds_normed_terms`, the norm on the output, the residual sum and that norm are one kernel
+    (`NormedTerm`), which also adds up a product's K slices and the outputs of a token's experts.
+    Block parameters (`LayerSpec.params`): norm1b, norm2b (PartSpecs; norm2b not without a feed-forward)."""
+    takes_next_norm = True
+
+    def __init__(self, layer_spec, env: BuildEnv):
+        params = dict(getattr(layer_spec, "params", None) or {})
+        self.norm1 = build_part("norm", layer_spec.norm1, env)
+        self.mixer = build_part("mixer", layer_spec.mixer, env)
+        self.norm1b = build_part("norm", params["norm1b"], env)
+        self.norm2 = self.feed_forward = self.norm2b = None
+        if layer_spec.feed_forward is not None:
+            self.norm2 = build_part("norm", layer_spec.norm2, env)
+            self.feed_forward = build_part("feed_forward", layer_spec.feed_forward, env)
+            self.norm2b = build_part("norm", params["norm2b"], env)
+        self.segments = dict({"norm1": "norm1", "mixer": "mix", "norm1b": "norm1b", "norm2": "norm2", "feed_forward": "mlp",
+                              "norm2b": "norm2b"}, **(getattr(layer_spec, "segments", None) or {}))
+        for norm in (self.norm1b, self.norm2b):
+            if norm is not None and not hasattr(norm, "add_normed"):
+                raise ConfigError("a norm on a sublayer's output must offer add_normed (rmsnorm, tanh)")
+
+    def _named(self):
+        return {k: p for k, p in (("norm1", self.norm1), ("mixer", self.mixer), ("norm1b", self.norm1b), ("norm2", self.norm2),
+                                  ("feed_forward", self.feed_forward), ("norm2b", self.norm2b)) if p is not None}
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(getattr(p, "graph_safe", False) for p in self._named().values())
+
+    @property
+    def plan_safe(self) -> bool:
+        return all(getattr(p, "plan_safe", False) for p in self._named().values())
+
+    def parts(self) -> Dict[str, object]:
+        return {self.segments[k]: p for k, p in self._named().items()}
+
+    def cache_requests(self):
+        many = getattr(self.mixer, "cache_requests", None)
+        one = getattr(self.mixer, "cache_request", None)
+        return list(many()) if many else ([one()] if one and one() is not None else [])
+
+    @property
+    def first_norm(self):
+        return self.norm1
+
+    @staticmethod
+    def _after(norm, y, x: torch.Tensor, reader):
+        """x += norm(y), left to `reader`, the norm that reads the stream next, where that does it in its own pass."""
+        term = NormedTerm(norm, y)
+        if type(reader) is type(norm) and getattr(reader, "adds_normed_terms", False):
+            return term
+        term.apply(x)
+        return None
+
+    def forward(self, x: torch.Tensor, pending, ctx, view, next_norm=None):
+        h = normed_for(self.mixer, self.norm1, x, pending)
+        # a product's K slices may stay terms where the norm on the output adds them up
+        terms = self.norm1b if (norm_adds_terms(self.norm1b) and getattr(self.mixer, "leaves_terms", False)) else None
+        y = self.mixer.forward(h, ctx, view, stream=None, next_norm=terms) if terms is not None else self.mixer.forward(h, ctx, view)
+        if self.feed_forward is None:
+            return self._after(self.norm1b, y, x, next_norm)
+        pending = self._after(self.norm1b, y, x, self.norm2)
+        h = normed_for(self.feed_forward, self.norm2, x, pending)
+        if getattr(self.feed_forward, "leaves_pairs", False) and getattr(self.norm2b, "adds_normed_terms", False):
+            y = self.feed_forward.forward(h, ctx, pairs=True)
+        else:
+            y = self.feed_forward.forward(h, ctx)
+        return self._after(self.norm2b, y, x, next_norm)
+
+
 register_block("prenorm", PreNormBlock)
+register_block("sandwich", SandwichBlock)
 register_block("outnorm", OutNormBlock)
 register_block("parallel", ParallelBlock)

@@ -26,7 +26,7 @@ import torch
 
 from ..errors import ConfigError
 from .base import BuildEnv, CacheRequest, Part, TensorSpec, register_mixer
-from .linear import linear, pack_rows
+from .linear import linear, linear_to_stream, pack_rows
 from .short_conv import ACT_SILU, ShortConv
 
 DEFAULT_NAMES = {"q": "q", "k": "k", "v": "v", "q_conv": "q.conv", "k_conv": "k.conv", "v_conv": "v.conv", "b": "b",
@@ -353,7 +353,71 @@ class TimeMix(Part):
         return linear(lib, on, self.w_o, torch.float32)
 
 
+class LightningAttention(Part):
+    """Linear attention with one constant decay per head:
+        q, k = silu(Wq h), silu(Wk h)  (heads x dim each);  v = silu(Wv h)  (heads x vdim)
+        S <- decay[head] S + k v^T;  o = S^T q          (no other scale)
+        out = Wo (o / sqrt(mean(o^2) + eps) * norm * sigmoid(Wg h)),   the mean over all heads together, norm [heads * vdim]
+    All four projections are one product; silu is applied as the recurrence reads q, k and v; the state
+    (`view.states["lightning"]`, [slots, heads, vdim, dim] float32) lives in the cache's per-slot storage.
+    Parameters: heads, dim, vdim, decay (a number per head), eps, names."""
+    graph_safe = True
+    plan_safe = True
+    leaves_terms = True
+
+    NAMES = {"q": "q", "k": "k", "v": "v", "g": "g", "norm": "norm", "o": "o"}
+
+    def __init__(self, params: Dict, env: BuildEnv):
+        self.env = env
+        self.heads, self.dim, self.vdim = int(params["heads"]), int(params["dim"]), int(params["vdim"])
+        self.decay = [float(x) for x in params["decay"]]
+        self.eps = float(params["eps"])
+        if min(self.heads, self.dim, self.vdim) <= 0 or self.dim > 512:
+            raise ConfigError("lightning attention: sizes must be positive, the key size at most 512")
+        if len(self.decay) != self.heads:
+            raise ConfigError(f"lightning attention: {len(self.decay)} decays for {self.heads} heads")
+        self.names = dict(self.NAMES, **(params.get("names") or {}))
+        self.hidden = env.hidden_size
+        self.n_qk, self.n_v = self.heads * self.dim, self.heads * self.vdim
+        self.cache_from = None
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        n, e = self.names, self.hidden
+        return {n["q"]: TensorSpec((self.n_qk, e)), n["k"]: TensorSpec((self.n_qk, e)), n["v"]: TensorSpec((self.n_v, e)),
+                n["g"]: TensorSpec((self.n_v, e)), n["norm"]: TensorSpec((self.n_v,), role="gain", init="ones_normal"),
+                n["o"]: TensorSpec((e, self.n_v))}
+
+    def load(self, tensors: Dict[str, torch.Tensor]) -> None:
+        lib, allowed, n = self.env.lib, not getattr(self.env, "generic_only", False), self.names
+        first = tensors[n["q"]]
+        pieces, row = [], 0
+        for key in ("q", "k", "v", "g"):                     # one product: [q | k | v | gate]
+            pieces.append((tensors[n[key]], row, None, None))
+            row += tensors[n[key]].shape[0]
+        self.w_in = pack_rows(lib, pieces, row, self.hidden, first.dtype, first.device, allowed)
+        self.norm = tensors[n["norm"]]
+        o = tensors[n["o"]]
+        self.w_o = pack_rows(lib, [(o, 0, None, None)], o.shape[0], o.shape[1], o.dtype, o.device, allowed)
+        self.decay_t = torch.tensor(self.decay, dtype=torch.float32, device=first.device)
+
+    def cache_requests(self) -> List[CacheRequest]:
+        return [CacheRequest("state", state_shape=(self.heads, self.vdim, self.dim), state_init=0.0, name="lightning")]
+
+    def cache_request(self) -> Optional[CacheRequest]:
+        return self.cache_requests()[0]
+
+    def forward(self, h: torch.Tensor, ctx, view, stream: Optional[torch.Tensor] = None, next_norm=None) -> torch.Tensor:
+        lib, t = self.env.lib, h.shape[0]
+        proj = linear(lib, h, self.w_in, torch.float32)                       # [T, q | k | v | gate]
+        o = torch.empty((t, self.n_v), dtype=torch.float32, device=h.device)
+        lib.lightning_recurrence(proj, self.dim, self.heads, self.vdim, self.decay_t, view.states["lightning"], ctx, o)
+        on = torch.empty((t, self.n_v), dtype=self.env.dtype, device=h.device)
+        lib.gated_rmsnorm_rows(o, self.norm, proj, 2 * self.n_qk + self.n_v, 0, self.eps, on)
+        return linear_to_stream(lib, on, self.w_o, None, next_norm)
+
+
 register_mixer("channel_delta", ChannelDelta)
+register_mixer("lightning", LightningAttention)
 register_mixer("time_mix", TimeMix)
 register_mixer("gated_delta", HeadDelta)
 register_mixer("decay_attention", DecayAttention)

@@ -34,7 +34,7 @@ import torch
 
 from ..errors import ConfigError
 from .base import BuildEnv, CacheRequest, Part, TensorSpec, build_part, register_mixer
-from .linear import linear, pack_rows
+from .linear import linear, linear_to_stream, pack_rows
 
 DEFAULT_NAMES = {"dq": "dq", "dq_norm": "dq.norm", "uq": "uq", "dkv": "dkv", "dkv_norm": "dkv.norm", "uk": "uk", "uv": "uv",
                  "sink": "sink", "o": "o", "gate": "g"}
@@ -45,6 +45,7 @@ _MATRIX_CORE_RANKS = (64, 128)     # latents of these sizes in bfloat16 go throu
 class LatentAttention(Part):
     graph_safe = True
     plan_safe = True
+    leaves_terms = True
 
     def __init__(self, params: Dict, env: BuildEnv):
         self.env = env
@@ -169,7 +170,7 @@ class LatentAttention(Part):
         o = torch.empty((t, self.heads * self.vdim), dtype=dt, device=h.device)
         # the latent's part of every head's sum through the head's value matrix, the head's gate on the way out
         lib.heads_linear_part(ol, r, self.w_uv, o, self.vdim, gate=down if self.has_gate else None, gate_col=self.gate_col)
-        return linear(lib, o, self.w_o, torch.float32)
+        return linear_to_stream(lib, o, self.w_o, None, next_norm)
 
 
 register_mixer("latent_attention", LatentAttention)

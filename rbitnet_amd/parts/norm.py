@@ -23,8 +23,9 @@ from typing import Dict, Optional
 
 import torch
 
+from ..errors import ConfigError
 from .base import BuildEnv, Part, TensorSpec, register_norm
-from .stream import GainedRows, ScaledSum, StreamsUpdate  # noqa: F401  (GainedRows: its old home; importers find it here too)
+from .stream import ExpertPairs, GainedRows, NormedTerm, ScaledSum, StreamsUpdate  # noqa: F401  (GainedRows: its old home; importers find it here too)
 
 
 class RMSNorm(Part):
@@ -125,5 +126,59 @@ class LayerNorm(Part):
         return out
 
 
+class TanhNorm(Part):
+    """tanh(alpha x) * weight + bias, number by number, in float32: a norm without statistics, alpha being one number.
+    Parameters: size, names ({"weight": ..., "bias": ..., "alpha": ...}: the tensors' names below the part's prefix; an empty
+    name is the prefix itself).
+
+    It may stand in front of a sublayer or on its output (`add_normed`).  Where the two stand next to each other, behind one
+    sublayer and in front of the next, one kernel does the first, the residual sum and the second (delta a `NormedTerm`)."""
+    graph_safe = True
+    plan_safe = True
+    adds_terms = True
+    adds_normed_terms = True
+
+    def __init__(self, params: Dict, env: BuildEnv):
+        self.size = int(params["size"])
+        self.names = dict({"weight": "weight", "bias": "bias", "alpha": "alpha"}, **(params.get("names") or {}))
+        self.env = env
+        self.params = None          # (alpha, weight, bias)
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        return {self.names["weight"]: TensorSpec((self.size,), role="gain", init="ones_normal"),
+                self.names["bias"]: TensorSpec((self.size,), role="gain", init="normal"),
+                self.names["alpha"]: TensorSpec((), role="gain", init="ones_normal")}
+
+    def tensor_names(self, base: str) -> Dict[str, str]:
+        """full name -> the part's own name, for an owner that stores the norm under `base`."""
+        return {".".join(p for p in (base, name) if p): name for name in self.tensor_specs()}
+
+    def load(self, tensors: Dict[str, torch.Tensor]) -> None:
+        self.params = (tensors[self.names["alpha"]].reshape(1), tensors[self.names["weight"]], tensors[self.names["bias"]])
+
+    @staticmethod
+    def _term(y):
+        return (y.outputs, y.weights) if isinstance(y, ExpertPairs) else (y, None)
+
+    def add_normed(self, x: torch.Tensor, y, h_out: Optional[torch.Tensor] = None) -> None:
+        """x [T, E] float32 <- x + norm(y)."""
+        if h_out is not None:
+            raise ConfigError("a tanh norm on a sublayer's output does not leave the stream's rows")
+        y, weights = self._term(y)
+        self.env.lib.tanh_norm(x, y, self.params, None, None, None, weights=weights)
+
+    def forward(self, x: torch.Tensor, delta=None, rows: Optional[torch.Tensor] = None,
+                out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
+        n = x.shape[0] if rows is None else rows.shape[0]
+        out = torch.empty((n, self.size), dtype=out_dtype or self.env.dtype, device=x.device)
+        after, weights = None, None
+        if isinstance(delta, NormedTerm):
+            after = delta.norm.params
+            delta, weights = self._term(delta.y)
+        self.env.lib.tanh_norm(x, delta, after, self.params, rows, out, weights=weights)
+        return out
+
+
 register_norm("rmsnorm", RMSNorm)
+register_norm("tanh", TanhNorm)
 register_norm("layernorm", LayerNorm)

@@ -31,7 +31,11 @@ def rope_inverse_frequencies(head_dim: int, theta: float, scaling: Optional[Dict
     """float64 [D/2].  `scaling` None or {"rope_type": "llama3", factor, low_freq_factor,
     high_freq_factor, original_max_position_embeddings}: wavelengths shorter than
     original/high keep their frequency, longer than original/low have it divided by
-    factor, and those between are blended linearly in original/wavelength."""
+    factor, and those between are blended linearly in original/wavelength.
+    {"rope_type": "yarn", factor, original, fast, slow}: with index(t) = D ln(original / (2 pi t)) / (2 ln theta), the pair
+    index that turns t times over `original` positions, lo = max(floor(index(fast)), 0) and hi = min(ceil(index(slow)), D - 1),
+    pair i goes over from its own frequency to that divided by factor with the ramp clamp((i - lo) / max(hi - lo, 0.001), 0, 1);
+    its cosines and sines also carry a factor (`rope_amplitude`)."""
     i = torch.arange(head_dim // 2, dtype=torch.float64)
     inv = torch.pow(torch.tensor(float(theta), dtype=torch.float64), -2.0 * i / head_dim)
     if not scaling:
@@ -39,9 +43,16 @@ def rope_inverse_frequencies(head_dim: int, theta: float, scaling: Optional[Dict
     kind = scaling.get("rope_type", "default")
     if kind == "default":
         return inv
-    if kind != "llama3":
+    if kind not in ("llama3", "yarn"):
         raise ConfigError(f"unsupported rope scaling {kind!r}")
     factor = float(scaling["factor"])
+    if kind == "yarn":
+        def index(turns: float) -> float:
+            return head_dim * math.log(float(scaling["original"]) / (2.0 * math.pi * turns)) / (2.0 * math.log(float(theta)))
+        lo = max(math.floor(index(float(scaling["fast"]))), 0)
+        hi = min(math.ceil(index(float(scaling["slow"]))), head_dim - 1)
+        ramp = torch.clamp((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+        return inv / factor * ramp + inv * (1.0 - ramp)
     low = float(scaling["low_freq_factor"])
     high = float(scaling["high_freq_factor"])
     orig = float(scaling["original_max_position_embeddings"])
@@ -51,6 +62,13 @@ def rope_inverse_frequencies(head_dim: int, theta: float, scaling: Optional[Dict
     out = torch.where(wavelength > orig / low, inv / factor, mixed)
     out = torch.where(wavelength < orig / high, inv, out)
     return out
+
+
+def rope_amplitude(scaling: Optional[Dict]) -> float:
+    """The factor on every cosine and sine: 0.1 ln(factor) + 1 with the "yarn" scaling, else 1."""
+    if scaling and scaling.get("rope_type") == "yarn":
+        return 0.1 * math.log(float(scaling["factor"])) + 1.0
+    return 1.0
 
 
 class Rope(Part):
@@ -78,8 +96,9 @@ class Rope(Part):
                    self.max_positions, str(env.device))
             if key not in env.shared:
                 angles = torch.arange(self.max_positions, dtype=torch.float64)[:, None] * inv[None, :]
-                env.shared[key] = (torch.cos(angles).to(torch.float32).to(env.device).contiguous(),
-                                   torch.sin(angles).to(torch.float32).to(env.device).contiguous())
+                m = rope_amplitude(params.get("scaling"))
+                env.shared[key] = ((torch.cos(angles) * m).to(torch.float32).to(env.device).contiguous(),
+                                   (torch.sin(angles) * m).to(torch.float32).to(env.device).contiguous())
             self.cos, self.sin = env.shared[key]
 
     def rotation_tables(self):

@@ -21,7 +21,9 @@ A second family of routers is served by the same launches, each choice a paramet
     limit        None: no clamps, and the plain gate: expert(x) = Wd (silu(Wg x) * (Wu x))
     shared       None, or {"intermediate_size": f}: an expert of the plain gated form (tensors "shared.gate", "shared.up",
                  "shared.down") that every token uses, added times sigmoid(w . h), w the tensor "shared.sg" [1, E]
-The weights of the chosen are never renormalised.  Router logits, scores, the choice and all sums are float32.
+    bias         True: the tensor "router_bias" (one number per output) is added to the router's logits
+With score "chosen" the choice goes by the logits and the weights are the softmax over the chosen logits alone; otherwise the
+weights of the chosen are never renormalised.  Router logits, scores, the choice and all sums are float32.
 """
 from __future__ import annotations
 
@@ -33,10 +35,12 @@ from ..errors import ConfigError
 from .base import BuildEnv, Part, TensorSpec, register_feed_forward
 from .feed_forward import SwiGLU
 from .linear import linear, pack_rows
+from .stream import ExpertPairs
 
 DEFAULT_NAMES = {"router": "router", "expert": "e{i}", "gate": "gate", "up": "up", "down": "down", "correction": "correction",
-                 "shared": "shared", "shared_gate": "shared.sg"}
+                 "shared": "shared", "shared_gate": "shared.sg", "router_bias": "router.b"}
 MAX_EXPERTS = 1024
+MAX_CHOSEN = 64            # of the softmax over the chosen logits
 
 
 class RoutedExperts(Part):
@@ -56,9 +60,12 @@ class RoutedExperts(Part):
                               f"not supported (at most {MAX_EXPERTS} outputs)")
         if self.ff <= 0 or (self.limit is not None and not self.limit > 0):
             raise ConfigError("routed experts: sizes and the limit must be positive")
-        self.score = {"sigmoid": 0, "softmax": 1}.get(str(params.get("score", "sigmoid")))
+        self.score = {"sigmoid": 0, "softmax": 1, "chosen": 2}.get(str(params.get("score", "sigmoid")))
         if self.score is None:
-            raise ConfigError(f"routed experts: score {params.get('score')!r} not supported (sigmoid, softmax)")
+            raise ConfigError(f"routed experts: score {params.get('score')!r} not supported (sigmoid, softmax, chosen)")
+        if self.score == 2 and self.top > MAX_CHOSEN:
+            raise ConfigError(f"routed experts: the softmax over the chosen takes at most {MAX_CHOSEN} of them, not {self.top}")
+        self.has_bias = bool(params.get("bias"))
         self.has_correction = bool(params.get("correction"))
         if self.has_correction and self.score != 1:
             raise ConfigError("routed experts: a correction of the choice goes with the softmax")
@@ -77,7 +84,10 @@ class RoutedExperts(Part):
             base = self.names["shared"]
             self.shared = SwiGLU({"intermediate_size": int(shared["intermediate_size"]),
                                   "names": {"gate": f"{base}.gate", "up": f"{base}.up", "down": f"{base}.down"}}, env)
-        self.plain = self.score == 0 and self.weight_on == "input" and not self.identity and self.shared is None
+        self.plain = (self.score == 0 and self.weight_on == "input" and not self.identity and self.shared is None
+                      and not self.has_bias)
+        # the sum over a token's experts may be left to whoever reads it, where it is nothing but that
+        self.leaves_pairs = self.weight_on == "output" and not self.identity and self.shared is None
 
     def _name(self, i: int, what: str) -> str:
         return f"{self.names['expert'].format(i=i)}.{self.names[what]}"
@@ -86,6 +96,8 @@ class RoutedExperts(Part):
         out = {self.names["router"]: TensorSpec((self.n_outputs, self.hidden))}
         if self.has_correction:
             out[self.names["correction"]] = TensorSpec((self.n_outputs,), role="gain", init="normal")
+        if self.has_bias:
+            out[self.names["router_bias"]] = TensorSpec((self.n_outputs,), role="gain", init="normal")
         if self.shared is not None:
             out.update(self.shared.tensor_specs())
             out[self.names["shared_gate"]] = TensorSpec((1, self.hidden))
@@ -105,6 +117,7 @@ class RoutedExperts(Part):
         rows = r.shape[0] + len(pieces) - 1
         self.w_router = pack_rows(lib, pieces, rows, r.shape[1], r.dtype, r.device, allowed)
         self.correction = tensors[self.names["correction"]].contiguous() if self.has_correction else None
+        self.bias = tensors[self.names["router_bias"]].contiguous() if self.has_bias else None
         # all experts' matrices in one tensor each; for the matrix cores (bfloat16, sizes that are multiples of 32) every
         # expert's matrix fragment-major, so that a wave's load is 1 KB in a row
         self.frag = bool(allowed and r.dtype == torch.bfloat16 and self.hidden % 32 == 0 and self.ff % 32 == 0)
@@ -118,24 +131,29 @@ class RoutedExperts(Part):
 
         self.w_gate, self.w_up, self.w_down = stack("gate"), stack("up"), stack("down")
 
-    def forward(self, h: torch.Tensor, ctx=None, stream: Optional[torch.Tensor] = None, next_norm=None) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, ctx=None, stream: Optional[torch.Tensor] = None, next_norm=None, pairs: bool = False):
+        """-> float32 [T, E], or, with pairs=True (where `leaves_pairs`), the `ExpertPairs` of the step."""
         lib, t, dev = self.env.lib, h.shape[0], h.device
         z = linear(lib, h, self.w_router, torch.float32)
-        pairs = t * self.top
+        n_pairs = t * self.top
         max_rows = lib.routed_rows(t, self.top, self.n_experts)
-        sel = torch.empty(pairs, dtype=torch.int32, device=dev)
-        weight = torch.empty(pairs, dtype=torch.float32, device=dev)
+        sel = torch.empty(n_pairs, dtype=torch.int32, device=dev)
+        weight = torch.empty(n_pairs, dtype=torch.float32, device=dev)
         row_pair = torch.empty(max_rows, dtype=torch.int32, device=dev)
         tile_expert = torch.empty(2 * (max_rows // 16), dtype=torch.int32, device=dev)      # experts, then positions in their runs
         if self.plain:
             lib.route_top(z, self.n_experts, self.top, sel, weight, row_pair, tile_expert)
         else:
             lib.route_choose(z, self.n_outputs, self.n_experts, self.top, self.score, self.correction, sel, weight, row_pair,
-                             tile_expert)
+                             tile_expert, bias=self.bias)
         y = torch.empty((max_rows, self.ff + self.hidden), dtype=h.dtype, device=dev)         # scratch: gated units, scaled inputs
-        out = torch.empty((pairs, self.hidden), dtype=torch.float32, device=dev)
+        out = torch.empty((n_pairs, self.hidden), dtype=torch.float32, device=dev)
         lib.routed_experts(h, weight if self.weight_on == "input" else None, self.top, row_pair, tile_expert, self.w_gate,
                            self.w_up, self.w_down, y, out, self.limit or 0.0, self.alpha, w_frag=self.frag)
+        if pairs:
+            if not self.leaves_pairs:
+                raise ConfigError("routed experts: only a plain weighted sum of the experts' outputs can be left to its reader")
+            return ExpertPairs(out, weight)
         if self.weight_on == "output":
             total = torch.empty((t, self.hidden), dtype=torch.float32, device=dev)
             both = None if self.shared is None else self.shared.forward(h, ctx)

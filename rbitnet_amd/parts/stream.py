@@ -19,6 +19,9 @@ prepared for the norm that follows, `GainedRows`).  What a sublayer has not yet 
     StreamCopy      nothing to add, and the stream's rows as they are in the compute dtype: what the sublayers of a layer
                     whose norms stand on the sublayers' outputs read; only a block that says `takes_stream_copy` gets it
                     (`run_blocks` drops it before any other block and before the head)
+    NormedTerm      norm(y) still to be added, y a sublayer's output and norm the one that stands on it: a norm that says
+                    `adds_normed_terms` does both, and its own work, in one pass over the rows.  y may be [P, T, E], the K
+                    slices of a product, or `ExpertPairs`, the outputs of every token's experts before they are added up
 
 A mixer may hand back `WeightedTerms` (sa * a + sb * b, not yet added up) to a block that asks for them: the norm on the
 sublayer's output then adds them up in its own pass.
@@ -30,6 +33,9 @@ returns plain tensors, a norm without any does every sum and every normalisation
     part.adds_to_stream       forward takes stream=x and next_norm, and may return any form above
     part.takes_gained_rows    forward's input may be GainedRows instead of a tensor
     norm.adds_terms           forward's delta may be [P, T, E]
+    norm.adds_normed_terms    forward's delta may be a NormedTerm whose norm is of the same kind
+    part.leaves_terms         forward takes next_norm (stream None) and may return [P, T, E] to one that `adds_terms`
+    part.leaves_pairs         forward takes pairs=True and then returns `ExpertPairs`
     norm.folds_into_products  the norm is x * weight / sqrt(mean x^2 + eps) with `weight`, `eps`
                               and `size`, so that products may do its work (GainedRows)
     block.takes_next_norm     forward takes next_norm: the first norm of whatever runs after it
@@ -113,6 +119,24 @@ class WeightedTerms:
 
     def __init__(self, a: torch.Tensor, sa: float, b: torch.Tensor, sb: float):
         self.a, self.sa, self.b, self.sb = a, float(sa), b, float(sb)
+
+
+class ExpertPairs:
+    """The outputs [T * top, E] of every token's chosen experts and their weights [T * top]: the sum over a token's experts,
+    weight times output, is still to be done."""
+
+    def __init__(self, outputs: torch.Tensor, weights: torch.Tensor):
+        self.outputs, self.weights = outputs, weights
+
+
+class NormedTerm:
+    """norm(y) that is still to be added to the stream x [T, E]; norm offers `add_normed`."""
+
+    def __init__(self, norm, y):
+        self.norm, self.y = norm, y
+
+    def apply(self, x: torch.Tensor) -> None:
+        self.norm.add_normed(x, self.y)
 
 
 def normed_for(part, norm, x: torch.Tensor, pending, rows: Optional[torch.Tensor] = None):
