@@ -397,9 +397,35 @@ def menerax_config(width: int, layers: int, heads: int, kv_heads: int, ff: int, 
     return {"architecture": "Menerax", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "layers": out}
 
 
+def lilevik_config(width: int, layers: int, heads: int, kv_heads: int, ff: int, vocab: int, experts: int = 16, top: int = 4,
+                   chunk: int = 1024, head: int = 64) -> dict:
+    """Groups of four layers with norms in front of and behind every sublayer: attention in chunks with sigmoid weights (heads
+    of `head` numbers, half of each rotated), lightning attention (heads of 128), attention through a latent (128 numbers a
+    token in the cache: a latent of 96 and a rotated part of 32), and attention in chunks again; routed experts whose `top`
+    chosen ones are together as wide as a dense feed-forward of `ff`."""
+    soft = {"heads": heads, "kv_heads": kv_heads, "dim": head, "vdim": head, "scale": head ** -0.5, "mask": {"size": chunk},
+            "rot": {"base": 500000.0, "dims": head // 2, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    n = max(1, width // 128)
+    light = {"heads": n, "dim": 128, "vdim": 128, "decay": [2.0 ** (-8.0 * (i + 1) / n) for i in range(n)]}
+    light["decay"] = [1.0 - 0.5 * d for d in light["decay"]]
+    latent = {"heads": heads, "dim": 64, "rot_dim": 32, "vdim": 64, "q_rank": max(256, width * 3 // 8), "kv_rank": 96, "scale": 96 ** -0.5,
+              "rot": {"base": 10000.0, "dims": 32}}
+    kinds = [("attention", soft), ("lightning", light), ("latent_attention", latent), ("attention", soft)]
+    moe = {"kind": "moe", "expert": {"ff": ff // top}, "router": {"experts": experts, "top": top}}
+    out = [{"type": kinds[i % 4][0], "mixer": dict(kinds[i % 4][1]), "mlp": dict(moe)} for i in range(layers)]
+    return {"architecture": "Lilevik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "layers": out}
+
+
 # size -> (the design's configuration, then the shapes beside it: the Llama shape of equal width, depth and feed-forward
 # width, and for Pulunex the Tigutar model of those sizes too, whose routed experts and attention kernels are the like ones)
 DESIGN_SIZES = {
+    # Lilevik beside the Tigutar model (routed experts, a linear recurrence), the Menerax model (latents, heads prepared in front
+    # of attention, norms on the outputs) and the Llama shape of those sizes
+    "lilevik_w1024": (lilevik_config(1024, 12, 16, 4, 4096, 32000), tigutar_config(1024, 12, 16, 4, 4096, 32000, experts=16),
+                      menerax_config(1024, 12, 16, 4, 4096, 32000), _other(1024, 4096, 16, 4, 64, 12, vocab=32000)),
+    "lilevik_w2048": (lilevik_config(2048, 16, 32, 8, 8192, 128256), tigutar_config(2048, 16, 32, 8, 8192, 128256, experts=16),
+                      menerax_config(2048, 16, 32, 8, 8192, 128256), _other(2048, 8192, 32, 8, 64, 16)),
+    "lilevik_w4096": (lilevik_config(4096, 8, 32, 8, 14336, 128256, head=128), dict(LLAMA3_8B, num_hidden_layers=8)),
     # Menerax beside the Tigutar model of those sizes (gated attention, windowed attention beside a linear recurrence) and the Llama shape
     "menerax_w1024": (menerax_config(1024, 12, 16, 4, 4096, 32000), tigutar_config(1024, 12, 16, 4, 4096, 32000, experts=16),
                       _other(1024, 4096, 16, 4, 64, 12, vocab=32000)),
@@ -531,8 +557,8 @@ def main(argv=None) -> int:
                     help="no benchmark line: the named shape's decode products of 8 tokens beside a kernel that only "
                          "reads as many bytes")
     ap.add_argument("--design", default="", metavar="SIZE",
-                    help=f"no benchmark line: a Bagonex, Tigutar, Pulunex or Menerax model of this size ({', '.join(sorted(DESIGN_SIZES))}) beside the Llama "
-                         "shape of equal width, depth and feed-forward width (Pulunex: beside Tigutar too): prefill and decode throughput, and the time per kernel")
+                    help=f"no benchmark line: a Bagonex, Tigutar, Pulunex, Menerax or Lilevik model of this size ({', '.join(sorted(DESIGN_SIZES))}) beside the Llama "
+                         "shape of equal width, depth and feed-forward width (some beside other designs too): prefill and decode throughput, and the time per kernel")
     ap.add_argument("--tokens", default="1,8,64,512,2048", help="token counts of --planner-sweep")
     ap.add_argument("--sweep-detail", default=None, help="--planner-sweep: a file for every candidate's time")
     ap.add_argument("--prefill-tokens", type=int, default=PREFILL_TOKENS,

@@ -361,6 +361,13 @@ int rb_tanh_norm(float* x, const float* y, int n_terms, long long term_stride, l
 int rb_lightning_recurrence(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride, const float* decay,
                             float* state, const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs, int n_tokens,
                             int n_heads, int dim, int vdim, void* stream);
+// The same for steps of several tokens a sequence, in chunks of 64 tokens on the matrix cores (float32 products and sums), for
+// heads whose sizes are multiples of 4 up to 128 (rb_lightning_chunks_ok).  powers float32 [H][65]: decay^0 .. decay^64.
+// q, k and v are overwritten.
+int rb_lightning_chunks_ok(int dim, int vdim);
+int rb_lightning_chunks(float* q, float* k, long long qk_stride, float* v, long long v_stride, const float* powers, float* state,
+                        const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs, int n_tokens, int n_heads, int dim,
+                        int vdim, void* stream);
 // rb_gated_rmsnorm_act with ONE norm over the whole row (all heads together); weight [width].
 int rb_gated_rmsnorm_rows(const float* o, const float* weight, const float* gate, long long gate_stride, int act, float eps, void* out,
                           int out_dtype, int n_tokens, int width, void* stream);

@@ -105,7 +105,7 @@ class KernelTimes:
         return "\n".join(lines)
 
 
-TIMED_OPS = ("tanh_norm", "heads_prepare", "lightning_recurrence", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
+TIMED_OPS = ("tanh_norm", "heads_prepare", "lightning_recurrence", "lightning_chunks", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
              "route_top", "routed_experts", "pairs_sum", "embed_streams", "streams_layernorm", "streams_update", "xielu", "tanh_cap", "short_conv",
              "delta_prep", "delta_rule", "gated_rmsnorm", "latent_norm_store", "heads_linear", "attention_sinks", "embed_gather", "add_rmsnorm", "rope_kv_write", "swiglu", "gemm_generic", "gemm_bf16", "gemm_bf16_terms",
              "gemm_bf16_few", "attention_generic", "attention_prefill_bf16", "attention_decode_bf16",
@@ -202,6 +202,8 @@ class Kernels:
             "rb_heads_prepare": [_P, _L, _P, _P, _I, _I, _P, _P, _I, _F, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
             "rb_tanh_norm": [_P, _P, _I, _L, _L, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _I, _P],
             "rb_lightning_recurrence": [_P, _P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P],
+            "rb_lightning_chunks_ok": [_I, _I],
+            "rb_lightning_chunks": [_P, _P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P],
             "rb_gated_rmsnorm_rows": [_P, _P, _P, _L, _I, _F, _P, _I, _I, _I, _P],
             "rb_route_choose_bias": [_P, _L, _P, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
             "rb_attention_mixed": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P, _I, _I, _P],
@@ -1396,6 +1398,30 @@ class Kernels:
         self._ok(self._lib.rb_lightning_recurrence(base, base + 4 * nq, width, base + 8 * nq, width, _ptr(decay), _ptr(state),
                                                    _ptr(ctx.cu_seqlens), _ptr(ctx.slots), _ptr(out), ctx.n_seqs, n, n_heads, dim, vdim,
                                                    self._stream()))
+
+    def lightning_chunks_ok(self, dim: int, vdim: int, width: int) -> bool:
+        """Whether `lightning_chunks` takes heads of these sizes in rows of `width` numbers."""
+        return bool(self._lib.rb_lightning_chunks_ok(int(dim), int(vdim))) and width % 4 == 0
+
+    def lightning_chunks(self, qkv: torch.Tensor, dim: int, n_heads: int, vdim: int, powers: torch.Tensor, state: torch.Tensor, ctx,
+                         out: torch.Tensor) -> None:
+        """`lightning_recurrence` in chunks of 64 tokens on the matrix cores; powers float32 [H, 65] (decay^0 .. decay^64);
+        the q, k and v columns of qkv are overwritten."""
+        n, width = qkv.shape
+        _check(qkv, "qkv", torch.float32)
+        if width < n_heads * (2 * dim + vdim):
+            raise KernelError("lightning_chunks: rows too short for q, k and v")
+        _check(powers, "powers", torch.float32, (n_heads, 65))
+        _check(state, "state", torch.float32)
+        if tuple(state.shape[1:]) != (n_heads, vdim, dim):
+            raise KernelError(f"lightning_chunks: state of shape {tuple(state.shape)}, expected [*, {n_heads}, {vdim}, {dim}]")
+        _check(out, "out", torch.float32, (n, n_heads * vdim))
+        if ctx.n_tokens != n:
+            raise KernelError("lightning_chunks: the step's tokens and the rows differ")
+        base, nq = qkv.data_ptr(), n_heads * dim
+        self._ok(self._lib.rb_lightning_chunks(base, base + 4 * nq, width, base + 8 * nq, width, _ptr(powers), _ptr(state),
+                                               _ptr(ctx.cu_seqlens), _ptr(ctx.slots), _ptr(out), ctx.n_seqs, n, n_heads, dim, vdim,
+                                               self._stream()))
 
     def gated_rmsnorm_rows(self, o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, gate_col: int, act: int, eps: float,
                            out: torch.Tensor) -> None:

@@ -358,7 +358,8 @@ class LightningAttention(Part):
         q, k = silu(Wq h), silu(Wk h)  (heads x dim each);  v = silu(Wv h)  (heads x vdim)
         S <- decay[head] S + k v^T;  o = S^T q          (no other scale)
         out = Wo (o / sqrt(mean(o^2) + eps) * norm * sigmoid(Wg h)),   the mean over all heads together, norm [heads * vdim]
-    All four projections are one product; silu is applied as the recurrence reads q, k and v; the state
+    All four projections are one product; silu is applied as the recurrence reads q, k and v.  Steps of several tokens a
+    sequence run in chunks on the matrix cores (in float32), single tokens one after another; the state
     (`view.states["lightning"]`, [slots, heads, vdim, dim] float32) lives in the cache's per-slot storage.
     Parameters: heads, dim, vdim, decay (a number per head), eps, names."""
     graph_safe = True
@@ -398,7 +399,9 @@ class LightningAttention(Part):
         self.norm = tensors[n["norm"]]
         o = tensors[n["o"]]
         self.w_o = pack_rows(lib, [(o, 0, None, None)], o.shape[0], o.shape[1], o.dtype, o.device, allowed)
-        self.decay_t = torch.tensor(self.decay, dtype=torch.float32, device=first.device)
+        d = torch.tensor(self.decay, dtype=torch.float64)
+        self.decay_t = d.to(torch.float32).to(first.device)
+        self.powers = torch.stack([d ** i for i in range(65)], dim=1).to(torch.float32).to(first.device).contiguous()
 
     def cache_requests(self) -> List[CacheRequest]:
         return [CacheRequest("state", state_shape=(self.heads, self.vdim, self.dim), state_init=0.0, name="lightning")]
@@ -410,7 +413,10 @@ class LightningAttention(Part):
         lib, t = self.env.lib, h.shape[0]
         proj = linear(lib, h, self.w_in, torch.float32)                       # [T, q | k | v | gate]
         o = torch.empty((t, self.n_v), dtype=torch.float32, device=h.device)
-        lib.lightning_recurrence(proj, self.dim, self.heads, self.vdim, self.decay_t, view.states["lightning"], ctx, o)
+        if ctx.max_q_len > 1 and lib.lightning_chunks_ok(self.dim, self.vdim, proj.shape[1]):
+            lib.lightning_chunks(proj, self.dim, self.heads, self.vdim, self.powers, view.states["lightning"], ctx, o)
+        else:                                # single tokens, and sizes off the matrix cores' grid: one token after another
+            lib.lightning_recurrence(proj, self.dim, self.heads, self.vdim, self.decay_t, view.states["lightning"], ctx, o)
         on = torch.empty((t, self.n_v), dtype=self.env.dtype, device=h.device)
         lib.gated_rmsnorm_rows(o, self.norm, proj, 2 * self.n_qk + self.n_v, 0, self.eps, on)
         return linear_to_stream(lib, on, self.w_o, None, next_norm)
