@@ -247,6 +247,10 @@ int rb_route_top(const float* z, long long z_stride, int n_experts, int top, int
 int rb_routed_experts(const void* h, int dtype, const float* weight, int top, const int32_t* row_pair, const int32_t* tile_expert,
                       int max_rows, const void* w_gate, const void* w_up, const void* w_down, int w_layout, void* y, float* out,
                       int n_experts, int width, int ff, float limit, float alpha, void* stream);
+// The same for a step of at most 64 tokens with fragment-major experts: the same sums, bit for bit, in two launches.
+int rb_routed_experts_few(const void* h, const float* weight, int top, const int32_t* row_pair, const int32_t* tile_expert, int max_rows,
+                          const void* w_gate, const void* w_up, const void* w_down, void* y, float* out, int n_tokens, int n_experts,
+                          int width, int ff, float limit, float alpha, void* stream);
 // rb_route_top with its choices spelled out.  The router has n_outputs outputs, of which the first n_experts are experts
 // with matrices; a pair whose output lies behind them belongs to no run (rb_experts_combine gives it the token's input).
 // score 0: weight = sigmoid(z) of the chosen, chosen by z.  score 1: weight = softmax(z) over all outputs, chosen by

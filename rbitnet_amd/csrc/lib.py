@@ -112,6 +112,9 @@ TIMED_OPS = ("tanh_norm", "heads_prepare", "lightning_recurrence", "lightning_ch
              "attention_decode_fused_bf16", "sample")
 
 
+ROUTED_FEW_TOKENS = 64         # steps of up to so many tokens run their experts in the kernels for few tokens
+
+
 class Kernels:
     """The loaded library.  Methods check operand shapes on the host before a launch, so
     that a kernel never sees sizes other than the ones its grid assumes."""
@@ -175,6 +178,7 @@ class Kernels:
             "rb_pair_norm_mean": [_P, _P, _P, _P, _F, _P, _I, _I, _P],
             "rb_route_top": [_P, _L, _I, _I, _P, _P, _P, _P, _I, _I, _P],
             "rb_routed_experts": [_P, _I, _P, _I, _P, _P, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _F, _F, _P],
+            "rb_routed_experts_few": [_P, _P, _I, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _F, _F, _P],
             "rb_pairs_sum": [_P, _I, _P, _I, _I, _P],
             "rb_route_choose": [_P, _L, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
             "rb_experts_combine": [_P, _P, _P, _I, _I, _P, _I, _P, _P, _L, _P, _I, _I, _P],
@@ -848,6 +852,11 @@ class Kernels:
         _check(w_down, "w_down", h.dtype, (n_experts, width, ff))
         _check(y, "y", h.dtype, (max_rows, ff + width))
         _check(out, "out", torch.float32, (n * top, width))
+        if w_frag and n <= ROUTED_FEW_TOKENS:
+            self._ok(self._lib.rb_routed_experts_few(_ptr(h), _ptr(weight), top, _ptr(row_pair), _ptr(tile_expert), max_rows, _ptr(w_gate),
+                                                     _ptr(w_up), _ptr(w_down), _ptr(y), _ptr(out), n, n_experts, width, ff, float(limit),
+                                                     float(alpha), self._stream()))
+            return
         self._ok(self._lib.rb_routed_experts(_ptr(h), dtype_code(h.dtype), _ptr(weight), top, _ptr(row_pair), _ptr(tile_expert),
                                              max_rows, _ptr(w_gate), _ptr(w_up), _ptr(w_down), int(bool(w_frag)), _ptr(y), _ptr(out),
                                              n_experts, width, ff, float(limit), float(alpha), self._stream()))

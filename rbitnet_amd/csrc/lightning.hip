@@ -138,8 +138,8 @@ __global__ __launch_bounds__(256) void lightning_inner_kernel(float* __restrict_
 // ---------------------------------------------------------------- from chunk to chunk
 // A workgroup of 4 waves holds 16 columns (value channels) of a head's state: wave w rows 16 RT w .. of it in its
 // accumulators (RT tiles of 16 rows; with two, row r of tile i is number 32 w + 2 r + i of the head, so that a lane's operand
-// of both tiles is 8 bytes in a row), and all of them in LDS, twice, for every wave's read-out.  The operands of the next chunk
-// are asked for while this one's products run.
+// of both tiles is 8 bytes in a row), and all of them in LDS, twice, for every wave's read-out.  A chunk's operands are asked
+// for two chunks ahead.
 template <int DK>
 __global__ __launch_bounds__(256) void lightning_carry_kernel(const float* __restrict__ q, const float* __restrict__ k, size_t qk_stride,
                                                               const float* __restrict__ v, size_t v_stride,
@@ -176,62 +176,68 @@ __global__ __launch_bounds__(256) void lightning_carry_kernel(const float* __res
 #pragma unroll
       for (int e = 0; e < 4; ++e) acc[i][e] = own[RT * e + i];
   }
+  // Loads are unconditional, from an address inside the step where a token, row or column lies outside, so that they are all in
+  // flight together: a query or column that is not there gives a result that nobody stores; a token that is not there must not
+  // reach the state (its v becomes 0 at use), nor a row of the head beyond dim the read-out (its q becomes 0 at use).
   struct Chunk {
     float4 q[DK / 16];        // query 16 w + c16: rows 16 s + 4 g ..
     float k[16][RT];          // token 4 s + g: rows of this wave's tiles
     float v[16];              // token 4 s + g: this lane's column
     float o[4];               // queries 16 w + 4 g + i: what the first launch left
   };
+  const int k_row = 16 * RT * wave + RT * c16;
+  const float* q_base = q + (size_t)h * dim;
+  const float* k_base = k + (size_t)h * dim + (k_row < dim ? k_row : 0);
+  const float* v_base = v + (size_t)h * vdim + (col_on ? col : 0);
+  const size_t o_base = (size_t)h * vdim + (col_on ? col : 0), o_stride = (size_t)n_heads * vdim;
   auto fetch = [&](Chunk& x, int at) {
     const int len = n - at < LN_CHUNK ? n - at : LN_CHUNK;
-    const int row0 = seq0 + at;
+    const size_t row0 = (size_t)(seq0 + at);
     const int qi = 16 * wave + c16;
-    const float* qrow = q + (size_t)(row0 + (qi < len ? qi : 0)) * qk_stride + (size_t)h * dim;
+    const float* qrow = q_base + (row0 + (qi < len ? qi : 0)) * qk_stride;
 #pragma unroll
     for (int s = 0; s < DK / 16; ++s) {
       const int d = 16 * s + 4 * g;
-      x.q[s] = (qi < len && d < dim) ? *reinterpret_cast<const float4*>(qrow + d) : make_float4(0.f, 0.f, 0.f, 0.f);
+      x.q[s] = *reinterpret_cast<const float4*>(qrow + (d < dim ? d : 0));
     }
-    const int r = 16 * RT * wave + RT * c16;
 #pragma unroll
     for (int s = 0; s < 16; ++s) {
-      const int t = 4 * s + g;
-      const bool on = t < len;
-      const float* krow = k + (size_t)(row0 + (on ? t : 0)) * qk_stride + (size_t)h * dim + (r < dim ? r : 0);
+      const size_t t = row0 + (4 * s + g < len ? 4 * s + g : 0);
       if (RT == 2) {
-        const float2 two = (on && r < dim) ? *reinterpret_cast<const float2*>(krow) : make_float2(0.f, 0.f);
+        const float2 two = *reinterpret_cast<const float2*>(k_base + t * qk_stride);
         x.k[s][0] = two.x;
         x.k[s][RT - 1] = two.y;
       } else {
-        x.k[s][0] = (on && r < dim) ? *krow : 0.f;
+        x.k[s][0] = k_base[t * qk_stride];
       }
-      x.v[s] = (on && col_on) ? v[(size_t)(row0 + t) * v_stride + (size_t)h * vdim + col] : 0.f;
+      x.v[s] = v_base[t * v_stride];
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int t = 16 * wave + 4 * g + i;
-      x.o[i] = (t < len && col_on) ? out[((size_t)(row0 + t) * n_heads + h) * vdim + col] : 0.f;
+      x.o[i] = out[(row0 + (t < len ? t : 0)) * o_stride + o_base];
     }
+    __builtin_amdgcn_sched_barrier(0);            // asked for here, not where the scheduler would sink them: at their use
   };
-  Chunk cur, next;
-  fetch(cur, 0);
   int buf = 0;
-  for (int at = 0; at < n; at += LN_CHUNK, buf ^= 1) {
+  // chunk at token `at` from `cur`, while the chunk two further on is fetched into `later`
+  auto work = [&](Chunk& cur, Chunk& later, int at) {
     const int len = n - at < LN_CHUNK ? n - at : LN_CHUNK;
     const bool more = at + LN_CHUNK < n;
     __syncthreads();                              // the state of all waves' rows is there
-    if (more) fetch(next, at + LN_CHUNK);
-    __builtin_amdgcn_sched_barrier(0);            // asked for here, not where the scheduler would sink them: at their use
+    if (at + 2 * LN_CHUNK < n) fetch(later, at + 2 * LN_CHUNK);
     const float dl = powers[(size_t)h * LN_POWERS + len];
-    f32x4_t oa = {cur.o[0], cur.o[1], cur.o[2], cur.o[3]}, ob = {0.f, 0.f, 0.f, 0.f};
+    if (dim < DK) {
 #pragma unroll
-    for (int s = 0; s < DK / 16; ++s) {
-      const float4 sf = *reinterpret_cast<const float4*>(&st[buf][c16 * SLD + 16 * s + 4 * g]);
-      oa = mfma16_f32(cur.q[s].x, sf.x, oa);
-      ob = mfma16_f32(cur.q[s].y, sf.y, ob);
-      oa = mfma16_f32(cur.q[s].z, sf.z, oa);
-      ob = mfma16_f32(cur.q[s].w, sf.w, ob);
+      for (int s = 0; s < DK / 16; ++s)
+        if (16 * s + 4 * g >= dim) cur.q[s] = make_float4(0.f, 0.f, 0.f, 0.f);
     }
+    if (len < LN_CHUNK) {
+#pragma unroll
+      for (int s = 0; s < 16; ++s)
+        if (4 * s + g >= len) cur.v[s] = 0.f;
+    }
+    f32x4_t oa = {cur.o[0], cur.o[1], cur.o[2], cur.o[3]}, ob = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < RT; ++i)
 #pragma unroll
@@ -240,6 +246,14 @@ __global__ __launch_bounds__(256) void lightning_carry_kernel(const float* __res
     for (int s = 0; s < 16; ++s)
 #pragma unroll
       for (int i = 0; i < RT; ++i) acc[i] = mfma16_f32(cur.k[s][i], cur.v[s], acc[i]);
+#pragma unroll
+    for (int s = 0; s < DK / 16; ++s) {
+      const float4 sf = *reinterpret_cast<const float4*>(&st[buf][c16 * SLD + 16 * s + 4 * g]);
+      oa = mfma16_f32(cur.q[s].x, sf.x, oa);
+      ob = mfma16_f32(cur.q[s].y, sf.y, ob);
+      oa = mfma16_f32(cur.q[s].z, sf.z, oa);
+      ob = mfma16_f32(cur.q[s].w, sf.w, ob);
+    }
     if (more) {
       float own[4 * RT];
 #pragma unroll
@@ -253,9 +267,18 @@ __global__ __launch_bounds__(256) void lightning_carry_kernel(const float* __res
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int t = 16 * wave + 4 * g + i;
-      if (t < len && col_on) out[((size_t)(seq0 + at + t) * n_heads + h) * vdim + col] = oa[i] + ob[i];
+      if (t < len && col_on) out[(size_t)(seq0 + at + t) * o_stride + o_base] = oa[i] + ob[i];
     }
-    if (more) cur = next;
+    buf ^= 1;
+  };
+  // three chunks' operands in registers: the one at work and two on their way
+  Chunk x0, x1, x2;
+  fetch(x0, 0);
+  if (LN_CHUNK < n) fetch(x1, LN_CHUNK);
+  for (int at = 0; at < n; at += 3 * LN_CHUNK) {
+    work(x0, x2, at);
+    if (at + LN_CHUNK < n) work(x1, x0, at + LN_CHUNK);
+    if (at + 2 * LN_CHUNK < n) work(x2, x1, at + 2 * LN_CHUNK);
   }
   if (!col_on) return;
   float own[4 * RT];

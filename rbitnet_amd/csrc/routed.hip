@@ -23,6 +23,7 @@
 
 #define RT_TILE 16
 #define RT_MAX_EXPERTS 1024
+#define RT_FEW_MOST 64         // tokens of a step whose experts run in the kernels for few tokens
 
 // ---------------------------------------------------------------- route
 // score 0: sigmoid(z) of the chosen logit.  score 1: the softmax of z over all outputs; the choice then goes by the
@@ -277,22 +278,154 @@ __global__ void routed_down_generic_kernel(const T* __restrict__ y, const int32_
 // rows it touched 16 lines a fixed 2 * K bytes apart, and the kernels ran at a tenth of this speed.  The experts'
 // matrices are stored so at load time; the step's rows are written so here, and the gated units by the kernel below.
 // The rows of the step, scaled by their weights and rounded to bfloat16, in sorted order: xs[row] = bf16(weight h[token]).
-__global__ void routed_gather_kernel(const bf16_t* __restrict__ h, const float* __restrict__ weight, int top,
-                                     const int32_t* __restrict__ row_pair, bf16_t* __restrict__ xs, int width) {
-  const int row = blockIdx.x;
-  const int p = row_pair[row];
-  if (p < 0) return;
-  const float wt = weight ? weight[p] : 1.0f;
-  const bf16_t* x = h + (size_t)(p / top) * width;
-  bf16_t* dst = xs + (size_t)(row / RT_TILE) * RT_TILE * width + 8 * (row % RT_TILE);
-  for (int k = 8 * threadIdx.x; k < width; k += 8 * blockDim.x) {
-    const uint4 raw = load16(x + k);
-    *reinterpret_cast<uint4*>(dst + (size_t)(k / 32) * 512 + 128 * ((k % 32) / 8)) =
-        make_uint4(pack_bf16x2(bf16_bits_to_f32(raw.x & 0xffffu) * wt, bf16_bits_to_f32(raw.x >> 16) * wt),
-                   pack_bf16x2(bf16_bits_to_f32(raw.y & 0xffffu) * wt, bf16_bits_to_f32(raw.y >> 16) * wt),
-                   pack_bf16x2(bf16_bits_to_f32(raw.z & 0xffffu) * wt, bf16_bits_to_f32(raw.z >> 16) * wt),
-                   pack_bf16x2(bf16_bits_to_f32(raw.w & 0xffffu) * wt, bf16_bits_to_f32(raw.w >> 16) * wt));
+// A workgroup a tile: a wave reads 64 bytes of each of the 16 rows and writes 1 KB in a row.
+__device__ __forceinline__ uint4 scaled16(const uint4& raw, float wt) {
+  return make_uint4(pack_bf16x2(bf16_bits_to_f32(raw.x & 0xffffu) * wt, bf16_bits_to_f32(raw.x >> 16) * wt),
+                    pack_bf16x2(bf16_bits_to_f32(raw.y & 0xffffu) * wt, bf16_bits_to_f32(raw.y >> 16) * wt),
+                    pack_bf16x2(bf16_bits_to_f32(raw.z & 0xffffu) * wt, bf16_bits_to_f32(raw.z >> 16) * wt),
+                    pack_bf16x2(bf16_bits_to_f32(raw.w & 0xffffu) * wt, bf16_bits_to_f32(raw.w >> 16) * wt));
+}
+__global__ __launch_bounds__(256) void routed_gather_kernel(const bf16_t* __restrict__ h, const float* __restrict__ weight, int top,
+                                                            const int32_t* __restrict__ row_pair, const int32_t* __restrict__ tile_expert,
+                                                            bf16_t* __restrict__ xs, int width) {
+  const int tile = blockIdx.x;
+  if (tile_expert[tile] < 0) return;
+  const int lane = threadIdx.x & (RB_WAVE - 1), wave = threadIdx.x / RB_WAVE, n_waves = blockDim.x / RB_WAVE;
+  const int p = row_pair[tile * RT_TILE + (lane & 15)];
+  const float wt = (weight && p >= 0) ? weight[p] : 1.0f;
+  const bf16_t* x = h + (size_t)(p >= 0 ? p / top : 0) * width + 8 * (lane >> 4);      // a row of padding: any row, nobody stores what comes of it
+  bf16_t* dst = xs + (size_t)tile * RT_TILE * width + 8 * lane;
+  const int n_blocks = width / 32;
+  constexpr int AHEAD = 4;
+  for (int k0 = wave; k0 < n_blocks; k0 += AHEAD * n_waves) {
+    uint4 raw[AHEAD];
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) raw[u] = load16(x + 32 * (size_t)(k0 + u * n_waves < n_blocks ? k0 + u * n_waves : k0));
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      const int k = k0 + u * n_waves;
+      if (k < n_blocks) *reinterpret_cast<uint4*>(dst + 512 * (size_t)k) = weight ? scaled16(raw[u], wt) : raw[u];
+    }
   }
+}
+
+// ---- steps of few tokens.  An expert's run is then NT tiles at most, an expert's matrices are read once, and what counts is how
+// many loads are on their way: a wave takes 16 channels (gate and up) or 16 of the model's channels (down) for all of the
+// run's tiles, walks the depth alone, in the order of the kernels below (so that a row's sums are the same bits), and asks for
+// RT_AHEAD steps at once, the experts' matrices past the caches.  The rows are read where they lie (no gathered copy).
+#define RT_AHEAD 8
+template <int NT, bool WEIGHTED>
+__global__ __launch_bounds__(256) void routed_up_few_kernel(const bf16_t* __restrict__ h, const float* __restrict__ weight, int top,
+                                                            const int32_t* __restrict__ row_pair, const int32_t* __restrict__ tile_expert,
+                                                            const int32_t* __restrict__ tile_pos, const bf16_t* __restrict__ w_gate,
+                                                            const bf16_t* __restrict__ w_up, bf16_t* __restrict__ y, int width, int ff,
+                                                            float limit, float alpha, int n_tiles) {
+  const int t0 = blockIdx.y, e = tile_expert[t0];
+  if (e < 0 || tile_pos[t0] % NT != 0) return;
+  const int lane = threadIdx.x & (RB_WAVE - 1), wave = threadIdx.x / RB_WAVE;
+  const int c0 = (blockIdx.x * 4 + wave) * 16;
+  if (c0 >= ff) return;
+  int nt = 1;
+  while (nt < NT && t0 + nt < n_tiles && tile_expert[t0 + nt] == e) ++nt;
+  const int r = lane & 15, grp = lane >> 4;
+  const bf16_t* xr[NT];
+  float wt[NT];
+  bool on[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) {
+    const int p = j < nt ? row_pair[(t0 + j) * RT_TILE + r] : -1;
+    on[j] = p >= 0;
+    wt[j] = (WEIGHTED && p >= 0) ? weight[p] : 1.0f;
+    xr[j] = h + (size_t)(p >= 0 ? p / top : 0) * width + 8 * grp;
+  }
+  const bf16_t* gr = w_gate + ((size_t)e * ff + c0) * width + 8 * lane;
+  const bf16_t* ur = w_up + ((size_t)e * ff + c0) * width + 8 * lane;
+  f32x4_t ag[NT], au[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) ag[j] = au[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const int n_steps = width / 32;
+  auto steps = [&](int s0, int cnt) {
+    Frag8 fg[RT_AHEAD], fu[RT_AHEAD], fx[RT_AHEAD][NT];
+#pragma unroll
+    for (int u = 0; u < RT_AHEAD; ++u) {
+      const size_t s = (size_t)(s0 + (u < cnt ? u : 0));
+      fg[u].u = load16_stream(gr + 512 * s);
+      fu[u].u = load16_stream(ur + 512 * s);
+#pragma unroll
+      for (int j = 0; j < NT; ++j) fx[u][j].u = load16(xr[j] + 32 * s);
+    }
+    __builtin_amdgcn_sched_barrier(0);            // all of them are on their way before the first is waited for
+#pragma unroll
+    for (int u = 0; u < RT_AHEAD; ++u) {
+      if (u >= cnt) break;
+#pragma unroll
+      for (int j = 0; j < NT; ++j) {
+        if (WEIGHTED) fx[u][j].u = scaled16(fx[u][j].u, wt[j]);
+        ag[j] = mfma16(fg[u], fx[u][j], ag[j]);
+        au[j] = mfma16(fu[u], fx[u][j], au[j]);
+      }
+    }
+  };
+  int s0 = 0;
+  for (; s0 + RT_AHEAD <= n_steps; s0 += RT_AHEAD) steps(s0, RT_AHEAD);
+  if (s0 < n_steps) steps(s0, n_steps - s0);
+#pragma unroll
+  for (int j = 0; j < NT; ++j) {
+    if (!on[j]) continue;
+    const int c = c0 + 4 * grp;
+    bf16_t* dst = y + (size_t)(t0 + j) * RT_TILE * ff + (size_t)(c / 32) * 512 + 8 * (16 * ((c % 32) / 8) + r) + c % 8;
+    const f32x4_t g = ag[j], u = au[j];
+    *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(gated_unit(g[0], u[0], limit, alpha), gated_unit(g[1], u[1], limit, alpha)),
+                                                pack_bf16x2(gated_unit(g[2], u[2], limit, alpha), gated_unit(g[3], u[3], limit, alpha)));
+  }
+}
+
+template <int NT>
+__global__ __launch_bounds__(256) void routed_down_few_kernel(const bf16_t* __restrict__ y, const int32_t* __restrict__ row_pair,
+                                                              const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ tile_pos,
+                                                              const bf16_t* __restrict__ w_down, float* __restrict__ out, int width, int ff,
+                                                              int n_tiles) {
+  const int t0 = blockIdx.y, e = tile_expert[t0];
+  if (e < 0 || tile_pos[t0] % NT != 0) return;
+  const int lane = threadIdx.x & (RB_WAVE - 1), wave = threadIdx.x / RB_WAVE;
+  const int c0 = (blockIdx.x * 4 + wave) * 16;
+  if (c0 >= width) return;
+  int nt = 1;
+  while (nt < NT && t0 + nt < n_tiles && tile_expert[t0 + nt] == e) ++nt;
+  const int r = lane & 15, grp = lane >> 4;
+  int pair[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) pair[j] = j < nt ? row_pair[(t0 + j) * RT_TILE + r] : -1;
+  const bf16_t* dr = w_down + ((size_t)e * width + c0) * ff + 8 * lane;
+  const bf16_t* yr = y + (size_t)t0 * RT_TILE * ff + 8 * lane;
+  f32x4_t acc[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) acc[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const int n_steps = ff / 32;
+  auto steps = [&](int s0, int cnt) {
+    Frag8 fd[RT_AHEAD], fy[RT_AHEAD][NT];
+#pragma unroll
+    for (int u = 0; u < RT_AHEAD; ++u) {
+      const size_t s = (size_t)(s0 + (u < cnt ? u : 0));
+      fd[u].u = load16_stream(dr + 512 * s);
+#pragma unroll
+      for (int j = 0; j < NT; ++j) fy[u][j].u = load16(yr + (size_t)(j < nt ? j : 0) * RT_TILE * ff + 512 * s);
+    }
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int u = 0; u < RT_AHEAD; ++u) {
+      if (u >= cnt) break;
+#pragma unroll
+      for (int j = 0; j < NT; ++j) acc[j] = mfma16(fd[u], fy[u][j], acc[j]);
+    }
+  };
+  int s0 = 0;
+  for (; s0 + RT_AHEAD <= n_steps; s0 += RT_AHEAD) steps(s0, RT_AHEAD);
+  if (s0 < n_steps) steps(s0, n_steps - s0);
+#pragma unroll
+  for (int j = 0; j < NT; ++j)
+    if (pair[j] >= 0)
+      *reinterpret_cast<float4*>(out + (size_t)pair[j] * width + c0 + 4 * grp) = make_float4(acc[j][0], acc[j][1], acc[j][2], acc[j][3]);
 }
 
 // A workgroup of 8 waves takes up to RT_SPAN tiles of 16 rows that follow one another in an expert's run (the
@@ -445,8 +578,7 @@ extern "C" int rb_routed_experts(const void* h, int dtype, const float* weight, 
     RB_REQUIRE(aligned(h) && aligned(w_gate) && aligned(w_up) && aligned(w_down) && aligned(y) && aligned(out),
                "rb_routed_experts: the matrix-core kernels need 16-byte aligned operands");
     bf16_t* xs = (bf16_t*)y + (size_t)max_rows * ff;
-    const int threads = width / 8 >= 256 ? 256 : 64;
-    routed_gather_kernel<<<max_rows, threads, 0, s>>>((const bf16_t*)h, weight, top, row_pair, xs, width);
+    routed_gather_kernel<<<tiles, 256, 0, s>>>((const bf16_t*)h, weight, top, row_pair, tile_expert, xs, width);
     routed_up_mfma_kernel<<<dim3((ff + 63) / 64, tiles), RT_THREADS, 0, s>>>(xs, row_pair, tile_expert, tile_expert + tiles,
                                                                         (const bf16_t*)w_gate, (const bf16_t*)w_up, (bf16_t*)y, width,
                                                                         ff, limit, alpha, tiles);
@@ -465,6 +597,45 @@ extern "C" int rb_routed_experts(const void* h, int dtype, const float* weight, 
     routed_down_generic_kernel<float><<<dim3(tiles, (width + 3) / 4 < 64 ? (width + 3) / 4 : 64), 256, 0, s>>>(
         (const float*)y, row_pair, tile_expert, (const float*)w_down, out, width, ff);
   }
+  RB_LAUNCH_CHECK();
+  return 0;
+}
+
+// rb_routed_experts for a step of at most 64 tokens with fragment-major experts (bfloat16, sizes that are multiples of 32): the
+// same sums in the same order, two launches whose waves keep more of the experts' matrices on their way.  n_tokens: rows of h.
+extern "C" int rb_routed_experts_few(const void* h, const float* weight, int top, const int32_t* row_pair, const int32_t* tile_expert,
+                                     int max_rows, const void* w_gate, const void* w_up, const void* w_down, void* y, float* out,
+                                     int n_tokens, int n_experts, int width, int ff, float limit, float alpha, void* stream) {
+  RB_RECORDED(rb_routed_experts_few(h, weight, top, row_pair, tile_expert, max_rows, w_gate, w_up, w_down, y, out, n_tokens, n_experts, width,
+                                    ff, limit, alpha, stream));
+  RB_REQUIRE(n_tokens >= 0 && n_tokens <= RT_FEW_MOST, "rb_routed_experts_few: %d tokens (at most %d)", n_tokens, RT_FEW_MOST);
+  RB_REQUIRE(max_rows >= 0 && max_rows % RT_TILE == 0 && max_rows / RT_TILE <= 65535 && n_experts > 0 && width > 0 && ff > 0 && top > 0 &&
+                 width % 32 == 0 && ff % 32 == 0,
+             "rb_routed_experts_few: bad sizes rows=%d experts=%d width=%d ff=%d", max_rows, n_experts, width, ff);
+  auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  RB_REQUIRE(aligned(h) && aligned(w_gate) && aligned(w_up) && aligned(w_down) && aligned(y) && aligned(out),
+             "rb_routed_experts_few: operands must be 16-byte aligned");
+  if (max_rows == 0 || n_tokens == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  const int tiles = max_rows / RT_TILE;
+  const dim3 gu((ff + 63) / 64, tiles), gd((width + 63) / 64, tiles);
+#define RT_UP(NT, WEIGHTED)                                                                                                           \
+  routed_up_few_kernel<NT, WEIGHTED><<<gu, 256, 0, s>>>((const bf16_t*)h, weight, top, row_pair, tile_expert, tile_expert + tiles,    \
+                                                        (const bf16_t*)w_gate, (const bf16_t*)w_up, (bf16_t*)y, width, ff, limit, alpha, tiles)
+#define RT_DOWN(NT)                                                                                                       \
+  routed_down_few_kernel<NT><<<gd, 256, 0, s>>>((const bf16_t*)y, row_pair, tile_expert, tile_expert + tiles,             \
+                                                (const bf16_t*)w_down, out, width, ff, tiles)
+  if (n_tokens <= RT_TILE) {                  // a token chooses an expert once: no run is longer than the step's tokens
+    if (weight) RT_UP(1, true);
+    else RT_UP(1, false);
+    RT_DOWN(1);
+  } else {
+    if (weight) RT_UP(4, true);
+    else RT_UP(4, false);
+    RT_DOWN(4);
+  }
+#undef RT_UP
+#undef RT_DOWN
   RB_LAUNCH_CHECK();
   return 0;
 }
