@@ -92,7 +92,7 @@ def test_errors_name_the_key(edit, match):
 
 
 @pytest.mark.parametrize("dims,base,scaling", [
-    (32, 5e4, {"factor": 4.0, "original": 1000, "fast": 32.0, "slow": 1.0}),
+    (24, 3e4, {"factor": 5.0, "original": 900, "fast": 24.0, "slow": 1.5}),
     (64, 1e4, {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}),
     (4, 10.0, {"factor": 2.0, "original": 8, "fast": 4.0, "slow": 0.5}),
     (2, 100.0, {"factor": 3.0, "original": 50, "fast": 1.0, "slow": 1.0}),

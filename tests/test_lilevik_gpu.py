@@ -245,7 +245,7 @@ def test_what_the_cache_holds_are_normed_rotated_keys_and_normed_values(lib):
 
 
 @pytest.mark.parametrize("dtype", BOTH)
-@pytest.mark.parametrize("chunk,dim,vdim", [(36, 16, 12), (64, 64, 64), (65, 64, 128), (7, 8, 12), (130, 128, 32)])
+@pytest.mark.parametrize("chunk,dim,vdim", [(36, 16, 12), (64, 64, 64), (65, 64, 128), (7, 8, 12), (130, 128, 48)])
 def test_a_key_that_stands_out_at_every_edge_of_a_chunk(lib, dtype, chunk, dim, vdim):
     """One earlier token has the query's own input, keys are made from the matrix that makes queries, and the number added to
     the scores is so low that hardly any other key has a weight: seen as the first and the last but one of the query's chunk,
@@ -370,7 +370,7 @@ def _lat(heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, base):
 
 LATENTS = [_lat(3, 8, 4, 6, 12, 10, 0.3, 100.0), _lat(4, 32, 32, 16, 48, 96, 0.1, 1e4), _lat(16, 16, 16, 24, 32, 40, 0.15, 5e5),
            _lat(1, 5, 2, 7, 3, 9, 0.5, 7.0), _lat(20, 24, 8, 8, 64, 64, 0.12, 300.0), _lat(2, 64, 64, 64, 128, 192, 0.08, 1e4),
-           _lat(5, 48, 16, 80, 40, 112, 0.1, 1e4), _lat(4, 16, 0, 16, 24, 64, 0.2, 1.0), _lat(6, 64, 64, 128, 96, 64, 0.09, 1e5)]
+           _lat(5, 48, 16, 72, 40, 112, 0.1, 1e4), _lat(4, 16, 0, 16, 24, 64, 0.2, 1.0), _lat(6, 64, 64, 128, 96, 64, 0.09, 1e5)]
 
 
 @pytest.mark.parametrize("dtype", BOTH)
@@ -403,7 +403,7 @@ def test_a_far_token_through_the_latent(lib, dtype):
 
 
 # ---------------------------------------------------------------------------- lightning attention
-LIGHTNINGS = [dict(heads=2, dim=32, vdim=48, decay=[0.6, 0.999]), dict(heads=3, dim=12, vdim=20, decay=[0.0, 1.0, 0.9]),
+LIGHTNINGS = [dict(heads=2, dim=32, vdim=48, decay=[0.55, 0.998]), dict(heads=3, dim=12, vdim=20, decay=[0.0, 1.0, 0.9]),
               dict(heads=1, dim=64, vdim=64, decay=[0.97]), dict(heads=6, dim=5, vdim=7, decay=[0.5, 0.6, 0.7, 0.8, 0.9, 0.99]),
               dict(heads=2, dim=128, vdim=24, decay=[0.95, 0.3]), dict(heads=2, dim=20, vdim=128, decay=[0.999, 0.9999]),
               dict(heads=2, dim=100, vdim=100, decay=[0.99, -0.5]), dict(heads=1, dim=160, vdim=16, decay=[0.9]),
@@ -490,7 +490,7 @@ def test_what_the_first_token_wrote_is_read_much_later_beside_another_sequence(l
 
 # ---------------------------------------------------------------------------- routed experts
 EXPERTS = [(64, 32, 4, 2, 70), (48, 24, 7, 3, 33), (32, 16, 1, 1, 9), (128, 64, 16, 4, 300), (50, 31, 5, 5, 20), (64, 96, 130, 6, 40),
-           (256, 64, 12, 3, 1), (96, 64, 9, 2, 32), (64, 32, 70, 64, 5)]
+           (224, 96, 11, 3, 1), (96, 64, 9, 2, 32), (64, 32, 70, 64, 5)]
 
 
 @pytest.mark.parametrize("dtype", BOTH)
@@ -710,7 +710,7 @@ def _random_config(rng):
         if kind == "lightning":
             h = rng.choice([1, 2, 3, 4, 6])
             return dict(heads=h, dim=rng.choice([8, 12, 16, 32, 64, 96, 128]), vdim=rng.choice([8, 16, 20, 32, 64, 128]),
-                        decay=[rng.choice([0.3, 0.6065, 0.9, 0.98, 0.999]) for _ in range(h)])
+                        decay=[rng.choice([0.3, 0.62, 0.9, 0.98, 0.9995]) for _ in range(h)])
         if kind == "attention":
             dim, kvh, group = rng.choice([8, 16, 32, 48, 64, 96, 128]), rng.choice([1, 2, 3, 4]), rng.choice([1, 2, 3, 4, 8, 20])
             out = dict(heads=kvh * group, kv_heads=kvh, dim=dim, vdim=rng.choice([8, 16, 32, 48, 64, 128]), scale=rng.choice([0.05, 0.125, 0.3]), rot=rotation(dim))
@@ -718,8 +718,8 @@ def _random_config(rng):
                 out["mask"] = {"size": rng.choice([1, 7, 16, 36, 64, 65, 100, 128, 200])}
             return out
         rot = rng.choice([0, 2, 4, 8, 16, 32, 64])
-        out = _lat(rng.choice([1, 2, 3, 4, 8, 16, 24, 32]), rng.choice([8, 16, 32, 64, 128]), rot, rng.choice([8, 16, 32, 64, 80]),
-                   rng.choice([16, 24, 64, 80, 128]), rng.choice([8, 24, 32, 48, 64, 96, 112, 128]), rng.choice([0.05, 0.125, 0.2]), rng.choice([100.0, 1e4, 5e5]))
+        out = _lat(rng.choice([1, 2, 3, 4, 8, 16, 24, 32]), rng.choice([8, 16, 32, 64, 128]), rot, rng.choice([8, 16, 32, 64, 72]),
+                   rng.choice([16, 24, 64, 88, 128]), rng.choice([8, 24, 32, 48, 64, 96, 112, 128]), rng.choice([0.05, 0.125, 0.2]), rng.choice([100.0, 1e4, 5e5]))
         return out
 
     layers = []
