@@ -18,6 +18,7 @@ from typing import Any, Dict, Iterable, Optional, Tuple
 
 from ..errors import ConfigError
 from .bagonex import BagonexConfig
+from .goperax import GoperaxConfig
 from .lilevik import LilevikConfig
 from .llama import LlamaConfig
 from .menerax import MeneraxConfig
@@ -103,3 +104,4 @@ register_architecture("Tigutar", TigutarConfig)
 register_architecture("Pulunex", PulunexConfig)
 register_architecture("Menerax", MeneraxConfig)
 register_architecture("Lilevik", LilevikConfig)
+register_architecture("Goperax", GoperaxConfig)

@@ -165,9 +165,23 @@ int rb_streams_update_layernorm(float* x, int n_streams, long long stream_stride
                                 const float* y, const float* scale, const float* coef, const float* delta, const float* weight,
                                 const float* bias, float eps, const int32_t* rows, int n_rows, int width, void* out,
                                 int out_dtype, void* stream);      // rb_streams_update (mix null: none), then the norm, in one pass
+// rb_embed_streams with x[s][t, :] = table[ids[t], :] * scale + wave(tok_pos[t]): number 2i of wave(p) is sin(p inv[i]), number 2i + 1
+// cos(p inv[i]); inv float64 [(width + 1) / 2], null: no wave.
+int rb_embed_streams_waves(const void* table, int table_dtype, const int32_t* ids, float scale, const double* inv, const int32_t* tok_pos,
+                           float* x, int n_streams, long long stream_stride, int n_tokens, int width, void* stream);
+// RMS norm of a stream in several copies, behind the update that may still be to be done (mix null: none), in one pass:
+//   x'[t] = sum_s mix[s, t] x[s] + out_coef[t] * y;  u = sum_s coef[s] x'[s][src];  out[r] = u / sqrt(mean(u^2) + eps) * gain,
+// src = rows ? rows[r] : r; with rows the copies stay as they are.  y of row src is the sum over k < n_terms of
+// (weights ? weights[src * n_terms + k] : 1) * y[src * row_stride + k * term_stride + :], plus, where `extra` is given, the sum over
+// k < n_extra of extra[src * width + k * extra_stride + :].
+int rb_streams_rmsnorm(float* x, int n_streams, long long stream_stride, const float* mix, const float* out_coef, const float* y,
+                       int n_terms, long long term_stride, long long row_stride, const float* weights, const float* extra, int n_extra,
+                       long long extra_stride, const float* coef, const float* gain, float eps, const int32_t* rows, int n_rows,
+                       int width, void* out, int out_dtype, void* stream);
 int rb_streams_update(float* x, int n_streams, long long stream_stride, const float* mix, const float* out_coef, const float* y,
                       const float* scale, int n_tokens, int width, void* stream);
-// out = z > 0 ? softplus(act[0]) z^2 + z/2 : (1/2 + softplus(act[1])) (exp(z) - 1 - z) + z/2; act[0] NaN: the tanh form of GELU
+// out = z > 0 ? softplus(act[0]) z^2 + z/2 : (1/2 + softplus(act[1])) (exp(z) - 1 - z) + z/2; act[0] NaN: the tanh form of
+// GELU (act[1] 0) or the squared relu max(z, 0)^2 (act[1] 1)
 int rb_xielu(const float* z, const float* act, void* out, int out_dtype, long long n, void* stream);
 // x <- cap * tanh(x / cap)
 int rb_tanh_cap(float* x, float cap, long long n, void* stream);
@@ -212,6 +226,22 @@ int rb_linear_recurrence(const float* q, const float* k, long long qk_stride, co
 int rb_gated_rmsnorm_act(const float* o, const float* weight, const float* gate, long long gate_stride, int act, float eps, void* out,
                          int out_dtype, int n_tokens, int n_heads, int vdim, void* stream);
 
+// rb_short_conv_bias with a bias on the convolution's result too (bias_out float32 [C], null: none; not with residual).
+int rb_short_conv_biases(const float* x, long long x_stride, const float* bias, const float* bias_out, const float* w, int taps, float* state,
+                         const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens, const int32_t* slots, void* out,
+                         long long out_stride, int out_dtype, int residual, int act, int n_tokens, int n_seqs, int channels, void* stream);
+// A selective scan, token after token, on the state S kept column by column as [slots, H, vdim, dim]; with
+// dt = softplus(dt_in[t * dt_stride + h] + dt_bias[h]):
+//   S <- exp(-exp(a_log[h]) dt) S + dt k v^T;  out[t, h, :] = S^T q + d[h] v      (head h reads the q and k of group h / (H / G))
+int rb_selective_scan(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride, const float* dt_in,
+                      long long dt_stride, const float* dt_bias, const float* a_log, const float* d, float* state,
+                      const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs, int n_tokens, int n_heads, int n_groups,
+                      int dim, int vdim, void* stream);
+// The gate in front of the norm, the row in `parts` equal parts with a norm each: g = o * silu(gate[t * gate_stride + :]);
+// out[part] = g[part] / sqrt(mean(g[part]^2) + eps) * weight[part]; o [T, width], weight [width].
+int rb_gate_rmsnorm_parts(const float* o, const float* weight, const float* gate, long long gate_stride, float eps, void* out,
+                          int out_dtype, int n_tokens, int width, int parts, void* stream);
+
 // ---- a plain stream with layer norm (streams.hip)
 // v = x[src] + dscale * (delta[src] + (delta2 ? delta2[src] : 0)), src = rows ? rows[r] : r; without rows x[src] = v too;
 // out[r] = (v - mean) / sqrt(var + eps) * weight + bias.  delta null: the norm alone.
@@ -222,6 +252,7 @@ int rb_layernorm_residual(float* x, const float* delta, const float* delta2, flo
 // rb_rope_kv_write for heads whose keys and values differ in size and of which only the first `rot` numbers are rotated
 // (i paired with i + rot / 2; cos, sin [positions, rot / 2]).  A row of qkv (row_width floats apart) holds Hq and Hk
 // heads of `dim` and Hk heads of `vdim`; q_out [T, Hq, pad] and the pages [*, Hk, 64, pad] get them padded with zeros.
+// (v_pages null: the row holds no values, the keys serve as values too.)
 int rb_rope_store(const float* qkv, long long row_width, const float* cos, const float* sin, int rot, void* q_out, void* k_pages,
                   void* v_pages, int cache_dtype, const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* block_table,
                   int bt_stride, int n_tokens, int n_heads, int n_kv_heads, int dim, int vdim, int pad, void* stream);
@@ -257,10 +288,10 @@ int rb_routed_experts_few(const void* h, const float* weight, int top, const int
 // softmax + correction (float32 [n_outputs], null: nothing added).
 int rb_route_choose(const float* z, long long z_stride, int n_outputs, int n_experts, int top, int score, const float* correction,
                     int32_t* sel, float* weight, int32_t* row_pair, int32_t* tile_expert, int max_rows, int n_tokens, void* stream);
-// rb_routed_experts takes weight null (the input is not scaled) and limit <= 0 (no clamps, the plain gate:
+// rb_routed_experts takes weight null (the input is not scaled), w_gate null (experts without a gate: out[p] = Wd max(Wu x, 0)^2) and limit <= 0 (no clamps, the plain gate:
 // out[p] = Wd (silu(Wg x) * (Wu x))).
 // out[t] = sum over k of weight[p] * (sel[p] < n_experts ? pairs[p] : h[t]), p = t * top + k, in the order of k; with
-// shared (float32 [T, width]) also + sigmoid(gate[t * gate_stride]) * shared[t].  h of h_dtype [T, width].
+// shared (float32 [T, width]) also + sigmoid(gate[t * gate_stride]) * shared[t] (gate null: + shared[t]).  h of h_dtype [T, width].
 int rb_experts_combine(const float* pairs, const int32_t* sel, const float* weight, int top, int n_experts, const void* h,
                        int h_dtype, const float* shared, const float* gate, long long gate_stride, float* out, int n_tokens,
                        int width, void* stream);

@@ -105,7 +105,7 @@ class KernelTimes:
         return "\n".join(lines)
 
 
-TIMED_OPS = ("tanh_norm", "heads_prepare", "lightning_recurrence", "lightning_chunks", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
+TIMED_OPS = ("embed_streams_waves", "streams_rmsnorm", "selective_scan", "gate_rmsnorm_parts", "tanh_norm", "heads_prepare", "lightning_recurrence", "lightning_chunks", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
              "route_top", "routed_experts", "pairs_sum", "embed_streams", "streams_layernorm", "streams_update", "xielu", "tanh_cap", "short_conv",
              "delta_prep", "delta_rule", "gated_rmsnorm", "latent_norm_store", "heads_linear", "attention_sinks", "embed_gather", "add_rmsnorm", "rope_kv_write", "swiglu", "gemm_generic", "gemm_bf16", "gemm_bf16_terms",
              "gemm_bf16_few", "attention_generic", "attention_prefill_bf16", "attention_decode_bf16",
@@ -161,6 +161,11 @@ class Kernels:
             "rb_streams_layernorm": [_P, _I, _L, _P, _P, _P, _P, _F, _P, _I, _I, _P, _I, _P],
             "rb_streams_update_layernorm": [_P, _I, _L, _P, _P, _P, _P, _P, _P, _P, _P, _F, _P, _I, _I, _P, _I, _P],
             "rb_streams_update": [_P, _I, _L, _P, _P, _P, _P, _I, _I, _P],
+            "rb_embed_streams_waves": [_P, _I, _P, _F, _P, _P, _P, _I, _L, _I, _I, _P],
+            "rb_streams_rmsnorm": [_P, _I, _L, _P, _P, _P, _I, _L, _L, _P, _P, _I, _L, _P, _P, _F, _P, _I, _I, _P, _I, _P],
+            "rb_short_conv_biases": [_P, _L, _P, _P, _P, _I, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _P],
+            "rb_selective_scan": [_P, _P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
+            "rb_gate_rmsnorm_parts": [_P, _P, _P, _L, _F, _P, _I, _I, _I, _I, _P],
             "rb_xielu": [_P, _P, _P, _I, _L, _P],
             "rb_tanh_cap": [_P, _F, _L, _P],
             "rb_short_conv": [_P, _L, _P, _I, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _P],
@@ -583,6 +588,65 @@ class Kernels:
         self._ok(self._lib.rb_streams_update(_ptr(x), s_, n * width, _ptr(mix), _ptr(out_coef), _ptr(y), _ptr(scale), n, width,
                                              self._stream()))
 
+    def embed_streams_waves(self, table: torch.Tensor, ids: torch.Tensor, scale: float, inv: Optional[torch.Tensor],
+                            tok_pos: torch.Tensor, x: torch.Tensor) -> None:
+        """`embed_streams` with table[ids[t]] * scale + wave(tok_pos[t]): numbers 2i and 2i + 1 of wave(p) are the sine and the
+        cosine of p inv[i] (inv float64 [(E + 1) // 2]; None: no wave)."""
+        s_, n, width = x.shape
+        _check(table, "table")
+        _check(ids, "ids", torch.int32, (n,))
+        _check(tok_pos, "tok_pos", torch.int32, (n,))
+        _check(x, "x", torch.float32)
+        if table.shape[1] != width:
+            raise KernelError("embedding width mismatch")
+        if inv is not None:
+            _check(inv, "inv", torch.float64, ((width + 1) // 2,))
+        self._ok(self._lib.rb_embed_streams_waves(_ptr(table), dtype_code(table.dtype), _ptr(ids), float(scale), _ptr(inv),
+                                                  _ptr(tok_pos), _ptr(x), s_, n * width, n, width, self._stream()))
+
+    def streams_rmsnorm(self, x: torch.Tensor, coef: Optional[torch.Tensor], weight: torch.Tensor, eps: float,
+                        rows: Optional[torch.Tensor], out: torch.Tensor, update=None) -> None:
+        """x [S, T, E] float32; out [rows or T, E]: the RMS norm of sum_s coef[s] x[s] (coef None: the plain sum).
+        update (mix [S, S], out_coef [S], y, weights, extra): x[t] <- sum_s mix[s, t] x[s] + out_coef[t] * y first, in the same
+        pass (with rows only for them, and x stays as it is).  y: [T, E]; [P, T, E], terms that are added up; or, with weights
+        float32 [T * k], the outputs [T * k, E] of every token's k experts, each times its weight.  extra (or None): [T, E] or
+        [P, T, E], added to that."""
+        s_, n, width = x.shape
+        _check(x, "x", torch.float32)
+        if coef is not None:
+            _check(coef, "coef", torch.float32, (s_,))
+        _check(weight, "weight", torch.float32, (width,))
+        n_rows = n
+        if rows is not None:
+            n_rows = rows.shape[0]
+            _check(rows, "rows", torch.int32, (n_rows,))
+        _check(out, "out", None, (n_rows, width))
+        mix = out_coef = y = weights = extra = None
+        n_terms, term_stride, row_stride, n_extra, extra_stride = 1, 0, width, 1, 0
+        if update is not None:
+            mix, out_coef, y, weights, extra = update
+            _check(mix, "mix", torch.float32, (s_, s_))
+            _check(out_coef, "out_coef", torch.float32, (s_,))
+            if weights is not None:
+                n_terms, term_stride = y.shape[0] // max(1, n), width
+                row_stride = n_terms * width
+                _check(y, "y", torch.float32, (n * n_terms, width))
+                _check(weights, "weights", torch.float32, (n * n_terms,))
+            elif y.dim() == 3:
+                n_terms, term_stride = y.shape[0], n * width
+                _check(y, "y", torch.float32, (n_terms, n, width))
+            else:
+                _check(y, "y", torch.float32, (n, width))
+            if extra is not None:
+                if extra.dim() == 3:
+                    n_extra, extra_stride = extra.shape[0], n * width
+                    _check(extra, "extra", torch.float32, (n_extra, n, width))
+                else:
+                    _check(extra, "extra", torch.float32, (n, width))
+        self._ok(self._lib.rb_streams_rmsnorm(_ptr(x), s_, n * width, _ptr(mix), _ptr(out_coef), _ptr(y), n_terms, term_stride, row_stride,
+                                              _ptr(weights), _ptr(extra), n_extra, extra_stride, _ptr(coef), _ptr(weight), float(eps),
+                                              _ptr(rows), n_rows, width, _ptr(out), dtype_code(out.dtype), self._stream()))
+
     def xielu(self, z: torch.Tensor, act: torch.Tensor, out: torch.Tensor) -> None:
         _check(z, "z", torch.float32)
         _check(act, "act", torch.float32, (2,))
@@ -779,10 +843,11 @@ class Kernels:
                 raise KernelError("angle table width mismatch")
         need = n_heads * dim
         if k_pages is not None:
-            need += n_kv * (dim + vdim)
+            need += n_kv * (dim + (vdim if v_pages is not None else 0))          # without v pages the keys serve as values too
             _check(block_table, "block_table", torch.int32)
             _check(k_pages, "k_pages", q_out.dtype)
-            _check(v_pages, "v_pages", q_out.dtype, k_pages.shape)
+            if v_pages is not None:
+                _check(v_pages, "v_pages", q_out.dtype, k_pages.shape)
             if tuple(k_pages.shape[1:]) != (n_kv, self.page_size, pad):
                 raise KernelError(f"cache pages have shape {tuple(k_pages.shape)}, expected [*, {n_kv}, {self.page_size}, {pad}]")
         if width < need:
@@ -836,18 +901,20 @@ class Kernels:
                                         _ptr(tile_expert), max_rows, n, self._stream()))
 
     def routed_experts(self, h: torch.Tensor, weight: torch.Tensor, top: int, row_pair: torch.Tensor, tile_expert: torch.Tensor,
-                       w_gate: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, y: torch.Tensor, out: torch.Tensor,
+                       w_gate: Optional[torch.Tensor], w_up: torch.Tensor, w_down: torch.Tensor, y: torch.Tensor, out: torch.Tensor,
                        limit: float, alpha: float, w_frag: bool = False) -> None:
-        """w_frag: every expert's matrices are stored fragment-major (`place_rows(..., frag=True)` on each)."""
+        """w_frag: every expert's matrices are stored fragment-major (`place_rows(..., frag=True)` on each).  w_gate None: experts
+        without a gate, Wd max(Wu x, 0)^2."""
         n, width = h.shape
-        n_experts, ff, _ = w_gate.shape
+        n_experts, ff, _ = w_up.shape
         max_rows = row_pair.shape[0]
         _check(h, "h")
         if weight is not None:                   # None: the experts' inputs are not scaled
             _check(weight, "weight", torch.float32, (n * top,))
         _check(row_pair, "row_pair", torch.int32)
         _check(tile_expert, "tile_expert", torch.int32, (2 * (max_rows // 16),))
-        _check(w_gate, "w_gate", h.dtype, (n_experts, ff, width))
+        if w_gate is not None:
+            _check(w_gate, "w_gate", h.dtype, (n_experts, ff, width))
         _check(w_up, "w_up", h.dtype, (n_experts, ff, width))
         _check(w_down, "w_down", h.dtype, (n_experts, width, ff))
         _check(y, "y", h.dtype, (max_rows, ff + width))
@@ -890,7 +957,7 @@ class Kernels:
                         h: torch.Tensor, shared: Optional[torch.Tensor], gate: Optional[torch.Tensor], gate_col: int,
                         out: torch.Tensor) -> None:
         """out[t] = sum_k weight * (the pair's expert output, or h[t] for an output behind the experts), plus
-        sigmoid(gate[t, gate_col]) * shared[t] when there is a shared expert."""
+        sigmoid(gate[t, gate_col]) * shared[t] (gate None: shared[t]) when there is a shared expert."""
         n, width = out.shape
         _check(pairs, "pairs", torch.float32, (n * top, width))
         _check(sel, "sel", torch.int32, (n * top,))
@@ -900,6 +967,7 @@ class Kernels:
         gate_ptr, stride = None, 0
         if shared is not None:
             _check(shared, "shared", torch.float32, (n, width))
+        if shared is not None and gate is not None:
             _check(gate, "gate", torch.float32)
             if gate.shape[0] != n or not 0 <= gate_col < gate.shape[1]:
                 raise KernelError("experts_combine: the gate's column lies outside its rows")
@@ -1184,14 +1252,18 @@ class Kernels:
                                         _ptr(ctx.tok_seq), _ptr(ctx.slots), n, ctx.n_seqs, width, self._stream()))
 
     def short_conv_bias(self, x: torch.Tensor, col0: int, channels: int, bias: Optional[torch.Tensor], w: torch.Tensor,
-                        state: Optional[torch.Tensor], ctx, out: torch.Tensor, residual: bool, act: int) -> None:
-        """`short_conv` on x + bias (float32 [channels]); the state holds the inputs with their bias."""
+                        state: Optional[torch.Tensor], ctx, out: torch.Tensor, residual: bool, act: int,
+                        bias_out: Optional[torch.Tensor] = None) -> None:
+        """`short_conv` on x + bias (float32 [channels]); the state holds the inputs with their bias.  bias_out (float32
+        [channels], not with residual) is added to the result, in front of the activation."""
         n, width = x.shape
         taps = w.shape[1]
         _check(x, "x", torch.float32)
         _check(w, "w", torch.float32, (channels, taps))
         if bias is not None:
             _check(bias, "bias", torch.float32, (channels,))
+        if bias_out is not None:
+            _check(bias_out, "bias_out", torch.float32, (channels,))
         if col0 < 0 or col0 + channels > width:
             raise KernelError("short_conv: the columns lie outside the rows")
         if taps > 1:
@@ -1200,10 +1272,10 @@ class Kernels:
                 raise KernelError(f"short_conv: state of shape {tuple(state.shape)}, expected [*, {taps - 1}, {channels}]")
         _check(out, "out", None, (n, channels))
         _check(ctx.tok_pos, "tok_pos", torch.int32, (n,))
-        self._ok(self._lib.rb_short_conv_bias(x.data_ptr() + 4 * col0, width, _ptr(bias), _ptr(w), taps,
-                                              _ptr(state) if taps > 1 else None, _ptr(ctx.tok_pos), _ptr(ctx.tok_seq),
-                                              _ptr(ctx.cu_seqlens), _ptr(ctx.slots), _ptr(out), channels, dtype_code(out.dtype),
-                                              int(bool(residual)), int(act), n, ctx.n_seqs, channels, self._stream()))
+        self._ok(self._lib.rb_short_conv_biases(x.data_ptr() + 4 * col0, width, _ptr(bias), _ptr(bias_out), _ptr(w), taps,
+                                                _ptr(state) if taps > 1 else None, _ptr(ctx.tok_pos), _ptr(ctx.tok_seq),
+                                                _ptr(ctx.cu_seqlens), _ptr(ctx.slots), _ptr(out), channels, dtype_code(out.dtype),
+                                                int(bool(residual)), int(act), n, ctx.n_seqs, channels, self._stream()))
 
     def time_mix_recurrence(self, r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, bonus: torch.Tensor,
                             state: torch.Tensor, ctx, out: torch.Tensor, n_heads: int, dim: int, vdim: int) -> None:
@@ -1444,6 +1516,54 @@ class Kernels:
         _check(out, "out", None, (n, width))
         self._ok(self._lib.rb_gated_rmsnorm_rows(_ptr(o), _ptr(weight), gate.data_ptr() + 4 * gate_col, gate.shape[1], int(act), float(eps),
                                                  _ptr(out), dtype_code(out.dtype), n, width, self._stream()))
+
+    # ------------------------------------------------------------------ selective scans
+    def _scan_operands(self, what: str, xkq: torch.Tensor, dim: int, n_groups: int, n_heads: int, vdim: int, dt_in: torch.Tensor,
+                       dt_col: int, dt_bias: torch.Tensor, a_log: torch.Tensor, d: torch.Tensor, state: torch.Tensor, ctx,
+                       out: torch.Tensor) -> None:
+        n, width = xkq.shape
+        if width < n_heads * vdim + 2 * n_groups * dim or n_heads % n_groups:
+            raise KernelError(f"{what}: rows too short for x, k and q, or heads that do not share the groups")
+        _check(dt_in, "dt_in", torch.float32)
+        if dt_in.shape[0] != n or dt_col < 0 or dt_col + n_heads > dt_in.shape[1]:
+            raise KernelError(f"{what}: the step sizes' columns lie outside the rows")
+        for name, t in (("dt_bias", dt_bias), ("a_log", a_log), ("d", d)):
+            _check(t, name, torch.float32, (n_heads,))
+        _check(state, "state", torch.float32)
+        if tuple(state.shape[1:]) != (n_heads, vdim, dim):
+            raise KernelError(f"{what}: state of shape {tuple(state.shape)}, expected [*, {n_heads}, {vdim}, {dim}]")
+        _check(out, "out", torch.float32, (n, n_heads * vdim))
+        if ctx.n_tokens != n:
+            raise KernelError(f"{what}: the step's tokens and the rows differ")
+
+    def selective_scan(self, xkq: torch.Tensor, dim: int, n_groups: int, n_heads: int, vdim: int, dt_in: torch.Tensor, dt_col: int,
+                       dt_bias: torch.Tensor, a_log: torch.Tensor, d: torch.Tensor, state: torch.Tensor, ctx, out: torch.Tensor) -> None:
+        """xkq rows [x: H vdim | k: G dim | q: G dim | ...] float32; with dt = softplus(dt_in[t, dt_col + h] + dt_bias[h]):
+        S <- exp(-exp(a_log[h]) dt) S + dt k x^T, out = S^T q + d[h] x, token after token; state [slots, H, vdim, dim] float32."""
+        _check(xkq, "xkq", torch.float32)
+        self._scan_operands("selective_scan", xkq, dim, n_groups, n_heads, vdim, dt_in, dt_col, dt_bias, a_log, d, state, ctx, out)
+        n, width = xkq.shape
+        base = xkq.data_ptr()
+        k = base + 4 * n_heads * vdim
+        self._ok(self._lib.rb_selective_scan(k + 4 * n_groups * dim, k, width, base, width, dt_in.data_ptr() + 4 * dt_col, dt_in.shape[1],
+                                             _ptr(dt_bias), _ptr(a_log), _ptr(d), _ptr(state), _ptr(ctx.cu_seqlens), _ptr(ctx.slots),
+                                             _ptr(out), ctx.n_seqs, n, n_heads, n_groups, dim, vdim, self._stream()))
+
+    def gate_rmsnorm_parts(self, o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, gate_col: int, parts: int, eps: float,
+                           out: torch.Tensor) -> None:
+        """g = o * silu(gate[:, gate_col ..]); out: each of `parts` equal parts of g's rows divided by its root mean square, times
+        weight [width]."""
+        n, width = o.shape
+        _check(o, "o", torch.float32)
+        _check(weight, "weight", torch.float32, (width,))
+        _check(gate, "gate", torch.float32)
+        if gate.shape[0] != n or gate_col < 0 or gate_col + width > gate.shape[1]:
+            raise KernelError("gate_rmsnorm_parts: the gate's columns lie outside the rows")
+        if parts <= 0 or width % parts:
+            raise KernelError(f"gate_rmsnorm_parts: rows of {width} numbers in {parts} parts")
+        _check(out, "out", None, (n, width))
+        self._ok(self._lib.rb_gate_rmsnorm_parts(_ptr(o), _ptr(weight), gate.data_ptr() + 4 * gate_col, gate.shape[1], float(eps), _ptr(out),
+                                                 dtype_code(out.dtype), n, width, int(parts), self._stream()))
 
     # ------------------------------------------------------------------ recorded steps
     def plan_begin(self) -> int:

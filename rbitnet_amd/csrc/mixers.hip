@@ -123,8 +123,9 @@ extern "C" int rb_rope_store(const float* qkv, long long row_width, const float*
              "rb_rope_store: bad sizes T=%d Hq=%d Hk=%d dim=%d vdim=%d pad=%d", n_tokens, n_heads, n_kv_heads, dim, vdim, pad);
   RB_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dim, "rb_rope_store: %d rotated numbers in a head of %d", rot, dim);
   RB_REQUIRE(rot == 0 || (cos != nullptr && sin != nullptr), "rb_rope_store: a rotation needs its tables");
-  RB_REQUIRE((k_pages == nullptr) == (v_pages == nullptr), "rb_rope_store: k and v pages go together");
-  const long long need = (long long)n_heads * dim + (k_pages ? (long long)n_kv_heads * (dim + vdim) : 0);
+  // k pages without v pages: the row holds no values (the keys serve as values too)
+  RB_REQUIRE(k_pages != nullptr || v_pages == nullptr, "rb_rope_store: v pages need k pages");
+  const long long need = (long long)n_heads * dim + (k_pages ? (long long)n_kv_heads * (dim + (v_pages ? vdim : 0)) : 0);
   RB_REQUIRE(row_width >= need, "rb_rope_store: rows of %lld numbers, %lld needed", row_width, need);
   if (n_tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;

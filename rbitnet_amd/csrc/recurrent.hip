@@ -22,7 +22,7 @@ __device__ __forceinline__ float rb_softplus(float v) { return v > 20.0f ? v : l
 #define SC_TILE 16             // rows of the step that a workgroup walks
 template <typename TO>
 __global__ void short_conv_kernel(const float* __restrict__ x, size_t x_stride, const float* __restrict__ bias,
-                                  const float* __restrict__ w, int taps,
+                                  const float* __restrict__ bias_out, const float* __restrict__ w, int taps,
                                   float* __restrict__ state, const int32_t* __restrict__ tok_pos,
                                   const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ cu_seqlens,
                                   const int32_t* __restrict__ slots, TO* __restrict__ out, size_t out_stride,
@@ -42,7 +42,7 @@ __global__ void short_conv_kernel(const float* __restrict__ x, size_t x_stride, 
         wt[j] = j < keep ? w[(size_t)c * taps + j] : 0.f;
       }
       const float w_cur = w[(size_t)c * taps + keep];
-      const float bc = bias ? bias[c] : 0.f;
+      const float bc = bias ? bias[c] : 0.f, bo = bias_out ? bias_out[c] : 0.f;
       bool have = false;
       for (int t = r0; t < r1; ++t) {
         if (t - cu_seqlens[tok_seq[t]] < keep) {             // the sequence's workgroup takes it
@@ -56,7 +56,7 @@ __global__ void short_conv_kernel(const float* __restrict__ x, size_t x_stride, 
           have = true;
         }
         const float cur = x[(size_t)t * x_stride + c] + bc;
-        float acc = residual ? cur : 0.f;
+        float acc = residual ? cur : bo;
         acc = fmaf(w_cur, cur, acc);
 #pragma unroll
         for (int j = 0; j < SC_MAX_TAPS; ++j) acc = fmaf(wt[j], win[j], acc);
@@ -83,13 +83,13 @@ __global__ void short_conv_kernel(const float* __restrict__ x, size_t x_stride, 
       wt[j] = j < keep ? w[(size_t)c * taps + j] : 0.f;
     }
     const float w_cur = w[(size_t)c * taps + keep];
-    const float bc = bias ? bias[c] : 0.f;
+    const float bc = bias ? bias[c] : 0.f, bo = bias_out ? bias_out[c] : 0.f;
     float nxt = first > 0 ? x[(size_t)row0 * x_stride + c] + bc : 0.f;
     __builtin_amdgcn_sched_barrier(0);                       // state, weights and the first row: one trip to memory together
     for (int i = 0; i < first; ++i) {
       const float cur = nxt;
       if (i + 1 < first) nxt = x[(size_t)(row0 + i + 1) * x_stride + c] + bc;
-      float acc = residual ? cur : 0.f;
+      float acc = residual ? cur : bo;
       acc = fmaf(w_cur, cur, acc);
 #pragma unroll
       for (int j = 0; j < SC_MAX_TAPS; ++j) acc = fmaf(wt[j], win[j], acc);
@@ -125,6 +125,19 @@ extern "C" int rb_short_conv_bias(const float* x, long long x_stride, const floa
                                   int act, int n_tokens, int n_seqs, int channels, void* stream) {
   RB_RECORDED(rb_short_conv_bias(x, x_stride, bias, w, taps, state, tok_pos, tok_seq, cu_seqlens, slots, out, out_stride, out_dtype,
                                  residual, act, n_tokens, n_seqs, channels, stream));
+  return rb_short_conv_biases(x, x_stride, bias, nullptr, w, taps, state, tok_pos, tok_seq, cu_seqlens, slots, out, out_stride, out_dtype,
+                              residual, act, n_tokens, n_seqs, channels, stream);
+}
+
+// The same with a bias on the convolution's result as well (bias_out float32 [C], null: none; not with residual), in front of the
+// activation; the state knows nothing of it.
+extern "C" int rb_short_conv_biases(const float* x, long long x_stride, const float* bias, const float* bias_out, const float* w, int taps,
+                                    float* state, const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens,
+                                    const int32_t* slots, void* out, long long out_stride, int out_dtype, int residual, int act,
+                                    int n_tokens, int n_seqs, int channels, void* stream) {
+  RB_RECORDED(rb_short_conv_biases(x, x_stride, bias, bias_out, w, taps, state, tok_pos, tok_seq, cu_seqlens, slots, out, out_stride,
+                                   out_dtype, residual, act, n_tokens, n_seqs, channels, stream));
+  RB_REQUIRE(bias_out == nullptr || !residual, "rb_short_conv: a bias on the result goes without the residual");
   RB_REQUIRE(n_tokens >= 0 && n_seqs >= 0 && channels > 0 && taps >= 1 && taps - 1 <= SC_MAX_TAPS,
              "rb_short_conv: bad sizes T=%d B=%d C=%d taps=%d (at most %d)", n_tokens, n_seqs, channels, taps, SC_MAX_TAPS + 1);
   RB_REQUIRE(x_stride >= channels && out_stride >= channels, "rb_short_conv: a row stride is shorter than the channels");
@@ -135,10 +148,10 @@ extern "C" int rb_short_conv_bias(const float* x, long long x_stride, const floa
   dim3 grid(n_tiles + (taps > 1 ? n_seqs : 0), (channels + 255) / 256 < 64 ? (channels + 255) / 256 : 64);
   hipStream_t s = (hipStream_t)stream;
   if (out_dtype == RB_F32)
-    short_conv_kernel<float><<<grid, 256, 0, s>>>(x, (size_t)x_stride, bias, w, taps, state, tok_pos, tok_seq, cu_seqlens, slots,
+    short_conv_kernel<float><<<grid, 256, 0, s>>>(x, (size_t)x_stride, bias, bias_out, w, taps, state, tok_pos, tok_seq, cu_seqlens, slots,
                                                   (float*)out, (size_t)out_stride, residual, act, channels, n_tokens, n_tiles);
   else if (out_dtype == RB_BF16)
-    short_conv_kernel<bf16_t><<<grid, 256, 0, s>>>(x, (size_t)x_stride, bias, w, taps, state, tok_pos, tok_seq, cu_seqlens, slots,
+    short_conv_kernel<bf16_t><<<grid, 256, 0, s>>>(x, (size_t)x_stride, bias, bias_out, w, taps, state, tok_pos, tok_seq, cu_seqlens, slots,
                                                    (bf16_t*)out, (size_t)out_stride, residual, act, channels, n_tokens, n_tiles);
   else
     RB_REQUIRE(false, "rb_short_conv: unknown dtype %d", out_dtype);
@@ -245,19 +258,27 @@ __device__ __forceinline__ float lanes_sum(float v) {
   return v;
 }
 
-// MODE 0: as above; 1: the read before the write, with a bonus (see below); 2: q, k and v go through silu as they are fetched.
+// MODE 0: as above; 1: the read before the write, with a bonus (see below); 2: q, k and v go through silu as they are fetched;
+// 3: a selective scan: every token has a step size dt = softplus(dt_in + dt_bias[h]) per head, from which the decay and the
+// weight of the write come, and its value passes to the read-out with a weight of the head:
+//   S <- exp(-exp(a_log[h]) dt) S + dt k v^T;  o = S^T q + d[h] v
+struct SelectiveArgs {
+  const float* dt_in;
+  size_t dt_stride;
+  const float *dt_bias, *a_log, *d;
+};
 template <int DKL, int RG, int CH, int MODE>
 __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
     const float* __restrict__ q, const float* __restrict__ k, size_t qk_stride, const float* __restrict__ v,
     size_t v_stride, const float* __restrict__ g, size_t g_stride, const float* __restrict__ beta, float* __restrict__ state,
     const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ slots, float* __restrict__ out, int n_heads,
-    int n_kv, int dim, int vdim, int g_per_head, const float* __restrict__ bonus) {
-  constexpr bool BONUS = MODE == 1;
+    int n_kv, int dim, int vdim, int g_per_head, const float* __restrict__ bonus, SelectiveArgs sel) {
+  constexpr bool BONUS = MODE == 1, SELECTIVE = MODE == 3;
   constexpr int COLS = RB_WAVE / RG;
   constexpr int DK = DKL * RG;               // rows held, >= dim; rows beyond dim stay zero
   constexpr int NQ = DK * CH / RB_WAVE;      // q (or k, or g) values of a chunk per lane
   constexpr int NV = (COLS * CH + RB_WAVE - 1) / RB_WAVE;
-  __shared__ float sq[CH][DK], sk[CH][DK], sg[CH][DK], sv[CH][COLS], so[CH][COLS], sb[CH];
+  __shared__ float sq[CH][DK], sk[CH][DK], sg[SELECTIVE ? 1 : CH][SELECTIVE ? CH : DK], sv[CH][COLS], so[CH][COLS], sb[CH];
   const int b = blockIdx.x, h = blockIdx.y;
   const int lane = threadIdx.x;
   const int col0 = blockIdx.z * COLS;
@@ -296,7 +317,8 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
     const int r = rg * DKL + i;
     ub[i] = (BONUS && r < dim) ? bonus[(size_t)h * dim + r] : 0.f;
   }
-  float rq[NQ], rk[NQ], rgt[NQ], rv[NV], rb = 0.f;
+  float rq[NQ], rk[NQ], rgt[SELECTIVE ? 1 : NQ], rv[NV], rb = 0.f;
+  const float rate = SELECTIVE ? expf(sel.a_log[h]) : 0.f, dt_bias = SELECTIVE ? sel.dt_bias[h] : 0.f, pass = SELECTIVE ? sel.d[h] : 0.f;
   auto fetch = [&](int t0) {
     const int nt = n - t0 < CH ? n - t0 : CH;
 #pragma unroll
@@ -306,7 +328,7 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
       const size_t t = (size_t)(row0 + t0 + tt);
       rq[j] = in ? q[t * qk_stride + (size_t)kvh * dim + i] : 0.f;
       rk[j] = in ? k[t * qk_stride + (size_t)kvh * dim + i] : 0.f;
-      rgt[j] = in ? (g_per_head ? g[t * g_stride + h] : g[t * g_stride + (size_t)h * dim + i]) : 0.f;
+      if (!SELECTIVE) rgt[j] = in ? (g_per_head ? g[t * g_stride + h] : g[t * g_stride + (size_t)h * dim + i]) : 0.f;
       if (MODE == 2) {
         rq[j] *= rb_sigmoid(rq[j]);
         rk[j] *= rb_sigmoid(rk[j]);
@@ -318,7 +340,10 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
       rv[j] = (tt < nt && col0 + c < vdim) ? v[(size_t)(row0 + t0 + tt) * v_stride + (size_t)h * vdim + col0 + c] : 0.f;
       if (MODE == 2) rv[j] *= rb_sigmoid(rv[j]);
     }
-    rb = (beta && lane < nt) ? beta[(size_t)(row0 + t0 + lane) * n_heads + h] : 0.f;
+    if (SELECTIVE)                                     // the step's raw number: what it becomes is made when the chunk goes to LDS
+      rb = lane < nt ? sel.dt_in[(size_t)(row0 + t0 + lane) * sel.dt_stride + h] : 0.f;
+    else
+      rb = (beta && lane < nt) ? beta[(size_t)(row0 + t0 + lane) * n_heads + h] : 0.f;
   };
   if (n > 0) fetch(0);
   for (int t0 = 0; t0 < n; t0 += CH) {
@@ -329,14 +354,22 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
       const int e = lane + RB_WAVE * j, tt = e / DK, i = e - tt * DK;
       sq[tt][i] = rq[j];
       sk[tt][i] = rk[j];
-      sg[tt][i] = rgt[j];
+      if (!SELECTIVE) sg[tt][i] = rgt[j];
     }
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int e = lane + RB_WAVE * j;
       if (e < COLS * CH) sv[e / COLS][e % COLS] = rv[j];
     }
-    if (lane < CH) sb[lane] = rb;
+    if (SELECTIVE) {
+      if (lane < CH) {
+        const float dt = rb_softplus(rb + dt_bias);
+        sb[lane] = dt;
+        sg[0][lane] = expf(-rate * dt);
+      }
+    } else if (lane < CH) {
+      sb[lane] = rb;
+    }
     __syncthreads();
     if (t0 + CH < n) fetch(t0 + CH);                   // in flight while this chunk is computed
     __builtin_amdgcn_sched_barrier(0);                 // (issued here, not where the scheduler would sink them: at their use)
@@ -346,6 +379,7 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
     auto token = [&](int tt) {
       const float vv = sv[tt][lane / RG];
       const float bt = sb[tt];
+      const float gt = SELECTIVE ? sg[0][tt] : 0.f;
       float kv0 = 0.f, kv1 = 0.f, dq0 = 0.f, dq1 = 0.f, kq0 = 0.f, kq1 = 0.f;
 #pragma unroll
       for (int i = 0; i < DKL; i += 2) {
@@ -360,6 +394,15 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
           s[i + 1] *= sg[tt][rg * DKL + i + 1];
           continue;
         }
+        if (SELECTIVE) {
+          s[i] *= gt;
+          s[i + 1] *= gt;
+          dq0 = fmaf(s[i], q0, dq0);
+          dq1 = fmaf(s[i + 1], q1, dq1);
+          kq0 = fmaf(k0, q0, kq0);
+          kq1 = fmaf(k1, q1, kq1);
+          continue;
+        }
         s[i] *= sg[tt][rg * DKL + i];
         s[i + 1] *= sg[tt][rg * DKL + i + 1];
         kv0 = fmaf(s[i], k0, kv0);
@@ -369,13 +412,14 @@ __global__ __launch_bounds__(RB_WAVE) void delta_rule_kernel(
         kq0 = fmaf(k0, q0, kq0);
         kq1 = fmaf(k1, q1, kq1);
       }
-      const float kv = BONUS ? 0.f : lanes_sum<RG>(kv0 + kv1);
+      const float kv = (BONUS || SELECTIVE) ? 0.f : lanes_sum<RG>(kv0 + kv1);
       const float dq = lanes_sum<RG>(dq0 + dq1);
       const float kq = lanes_sum<RG>(kq0 + kq1);
-      const float u = (!BONUS && beta) ? bt * (vv - kv) : vv;       // without beta: the plain rule, S <- diag(g) S + k v^T
+      // without beta: the plain rule, S <- diag(g) S + k v^T
+      const float u = SELECTIVE ? bt * vv : (!BONUS && beta) ? bt * (vv - kv) : vv;
 #pragma unroll
       for (int i = 0; i < DKL; ++i) s[i] = fmaf(sk[tt][rg * DKL + i], u, s[i]);
-      if (rg == 0) so[tt][lane / RG] = fmaf(u, kq, dq);
+      if (rg == 0) so[tt][lane / RG] = SELECTIVE ? fmaf(pass, vv, fmaf(u, kq, dq)) : fmaf(u, kq, dq);
     };
     if (nt == CH) {
       // a whole chunk as straight code, so that a token's reads from LDS are issued while the one before is computed
@@ -409,12 +453,12 @@ template <int DKL, int RG, int CH, int MODE>
 static void launch_delta_rule(const float* q, const float* k, size_t qk_stride, const float* v, size_t v_stride,
                               const float* g, size_t g_stride, const float* beta, float* state, const int32_t* cu_seqlens,
                               const int32_t* slots, float* out, int n_seqs, int n_heads, int n_kv, int dim, int vdim,
-                              int g_per_head, const float* bonus, hipStream_t s) {
+                              int g_per_head, const float* bonus, const SelectiveArgs& sel, hipStream_t s) {
   constexpr int COLS = RB_WAVE / RG;
   static_assert((DKL * RG * CH) % RB_WAVE == 0 && CH <= RB_WAVE && DKL % 4 == 0, "a chunk's values are dealt evenly to the lanes");
   dim3 grid(n_seqs, n_heads, (vdim + COLS - 1) / COLS);
   delta_rule_kernel<DKL, RG, CH, MODE><<<grid, RB_WAVE, 0, s>>>(q, k, qk_stride, v, v_stride, g, g_stride, beta, state, cu_seqlens,
-                                                                 slots, out, n_heads, n_kv, dim, vdim, g_per_head, bonus);
+                                                                 slots, out, n_heads, n_kv, dim, vdim, g_per_head, bonus, sel);
 }
 
 extern "C" int rb_delta_rule(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride,
@@ -441,7 +485,7 @@ extern "C" int rb_linear_recurrence(const float* q, const float* k, long long qk
 static int linear_recurrence_launch(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride,
                                     const float* g, long long g_stride, int g_per_head, const float* beta, const float* bonus,
                                     int silu_in, float* state, const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs,
-                                    int n_tokens, int n_heads, int n_kv_heads, int dim, int vdim, void* stream);
+                                    int n_tokens, int n_heads, int n_kv_heads, int dim, int vdim, const SelectiveArgs* sel, void* stream);
 
 // bonus (float32 [H, dim], null: rb_linear_recurrence): the plain rule read BEFORE the token's write, with the token's own
 // k v^T weighted per key channel:  out = (S + diag(bonus) k v^T)^T q;  S <- diag(g) S + k v^T.  Goes without beta.
@@ -453,7 +497,7 @@ extern "C" int rb_linear_recurrence_bonus(const float* q, const float* k, long l
   RB_RECORDED(rb_linear_recurrence_bonus(q, k, qk_stride, v, v_stride, g, g_stride, g_per_head, beta, bonus, state, cu_seqlens, slots,
                                          out, n_seqs, n_tokens, n_heads, n_kv_heads, dim, vdim, stream));
   return linear_recurrence_launch(q, k, qk_stride, v, v_stride, g, g_stride, g_per_head, beta, bonus, 0, state, cu_seqlens, slots, out,
-                                  n_seqs, n_tokens, n_heads, n_kv_heads, dim, vdim, stream);
+                                  n_seqs, n_tokens, n_heads, n_kv_heads, dim, vdim, nullptr, stream);
 }
 
 // The plain rule with one constant decay per head (decay float32 [H]) and silu on q, k and v as they are read:
@@ -464,14 +508,31 @@ extern "C" int rb_lightning_recurrence(const float* q, const float* k, long long
   RB_RECORDED(rb_lightning_recurrence(q, k, qk_stride, v, v_stride, decay, state, cu_seqlens, slots, out, n_seqs, n_tokens, n_heads, dim,
                                       vdim, stream));
   return linear_recurrence_launch(q, k, qk_stride, v, v_stride, decay, 0, 1, nullptr, nullptr, 1, state, cu_seqlens, slots, out, n_seqs,
-                                  n_tokens, n_heads, n_heads, dim, vdim, stream);
+                                  n_tokens, n_heads, n_heads, dim, vdim, nullptr, stream);
+}
+
+// A selective scan, token after token: with dt = softplus(dt_in[t * dt_stride + h] + dt_bias[h]),
+//   S <- exp(-exp(a_log[h]) dt) S + dt k v^T;  out[t, h, :] = S^T q + d[h] v      (head h reads the q and k of group h / (H / G))
+extern "C" int rb_selective_scan(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride, const float* dt_in,
+                                 long long dt_stride, const float* dt_bias, const float* a_log, const float* d, float* state,
+                                 const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs, int n_tokens, int n_heads,
+                                 int n_groups, int dim, int vdim, void* stream) {
+  RB_RECORDED(rb_selective_scan(q, k, qk_stride, v, v_stride, dt_in, dt_stride, dt_bias, a_log, d, state, cu_seqlens, slots, out, n_seqs,
+                                n_tokens, n_heads, n_groups, dim, vdim, stream));
+  RB_REQUIRE(dt_stride >= n_heads && dt_in != nullptr && dt_bias != nullptr && a_log != nullptr && d != nullptr,
+             "rb_selective_scan: the step sizes' rows are too short, or a tensor is missing");
+  const SelectiveArgs sel = {dt_in, (size_t)dt_stride, dt_bias, a_log, d};
+  return linear_recurrence_launch(q, k, qk_stride, v, v_stride, nullptr, n_heads, 1, nullptr, nullptr, 0, state, cu_seqlens, slots, out,
+                                  n_seqs, n_tokens, n_heads, n_groups, dim, vdim, &sel, stream);
 }
 
 // silu_in: q, k and v go through silu as they are read; g_stride 0 (with g_per_head): the same decays for every token.
 static int linear_recurrence_launch(const float* q, const float* k, long long qk_stride, const float* v, long long v_stride,
                                     const float* g, long long g_stride, int g_per_head, const float* beta, const float* bonus,
                                     int silu_in, float* state, const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs,
-                                    int n_tokens, int n_heads, int n_kv_heads, int dim, int vdim, void* stream) {
+                                    int n_tokens, int n_heads, int n_kv_heads, int dim, int vdim, const SelectiveArgs* selective,
+                                    void* stream) {
+  const SelectiveArgs sel = selective ? *selective : SelectiveArgs{nullptr, 0, nullptr, nullptr, nullptr};
   RB_REQUIRE(bonus == nullptr || beta == nullptr, "rb_linear_recurrence: a bonus goes with the plain rule (no beta)");
   RB_REQUIRE(n_seqs >= 0 && n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0 && dim > 0 && vdim > 0,
              "rb_linear_recurrence: bad sizes H=%d Hk=%d dim=%d vdim=%d", n_heads, n_kv_heads, dim, vdim);
@@ -488,24 +549,30 @@ static int linear_recurrence_launch(const float* q, const float* k, long long qk
 #define DR_GO(DKL, RG, CH)                                                                                                  \
   do {                                                                                                                      \
     constexpr int CH1 = (DKL * RG >= RB_WAVE) ? 1 : RB_WAVE / (DKL * RG);                                                   \
-    if (single && silu_in)                                                                                                  \
+    if (single && selective)                                                                                                \
+      launch_delta_rule<DKL, RG, CH1, 3>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,        \
+                                         n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, sel, s);                \
+    else if (selective)                                                                                                     \
+      launch_delta_rule<DKL, RG, CH, 3>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,         \
+                                        n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, sel, s);                 \
+    else if (single && silu_in)                                                                                                  \
       launch_delta_rule<DKL, RG, CH1, 2>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,        \
-                                         n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                     \
+                                         n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, sel, s);                   \
     else if (silu_in)                                                                                                       \
       launch_delta_rule<DKL, RG, CH, 2>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,         \
-                                        n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                      \
+                                        n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, sel, s);                    \
     else if (single && bonus)                                                                                               \
       launch_delta_rule<DKL, RG, CH1, 1>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,     \
-                                            n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                  \
+                                            n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, sel, s);                \
     else if (single)                                                                                                        \
       launch_delta_rule<DKL, RG, CH1, 0>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,    \
-                                             n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                 \
+                                             n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, sel, s);               \
     else if (bonus)                                                                                                         \
       launch_delta_rule<DKL, RG, CH, 1>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,      \
-                                           n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                   \
+                                           n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, sel, s);                 \
     else                                                                                                                    \
       launch_delta_rule<DKL, RG, CH, 0>(q, k, qs, v, vs, g, (size_t)g_stride, beta, state, cu_seqlens, slots, out,     \
-                                            n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, s);                  \
+                                            n_seqs, n_heads, n_kv_heads, dim, vdim, g_per_head, bonus, sel, s);                \
   } while (0)
   // Rows of a column over RG lanes, chunks as long as the registers that hold the next one allow.  A token's time is
   // its lane's share of the column, so while the waves do not fill the GPU's SIMDs a column goes to more lanes
@@ -617,6 +684,84 @@ extern "C" int rb_gated_rmsnorm_rows(const float* o, const float* weight, const 
     else RB_GR(bf16_t, false);
   }
 #undef RB_GR
+  RB_LAUNCH_CHECK();
+  return 0;
+}
+
+// The gate in front of the norm, and the row in equal parts with a norm each: with g = o * silu(gate),
+//   out[t, part] = g[part] / sqrt(mean(g[part]^2) + eps) * weight[part].      A workgroup a token and part.
+template <typename TO, bool VEC>
+__global__ __launch_bounds__(1024) void gate_rmsnorm_parts_kernel(const float* __restrict__ o, const float* __restrict__ weight,
+                                                                  const float* __restrict__ gate, size_t gate_stride, float eps,
+                                                                  TO* __restrict__ out, int width, int part) {
+  __shared__ float scratch[16];
+  const size_t t = blockIdx.x;
+  const int c0 = blockIdx.y * part;
+  const float* p = o + t * width + c0;
+  const float* gp = gate + t * gate_stride + c0;
+  const float* wp = weight + c0;
+  TO* op = out + t * width + c0;
+  auto gated = [](float v, float g) { return v * g * rb_sigmoid(g); };
+  float ss = 0.f;
+  if (VEC) {
+    const int j0 = 4 * threadIdx.x;
+    auto quad = [&](int j) {
+      const float4 v = *reinterpret_cast<const float4*>(p + j), g = *reinterpret_cast<const float4*>(gp + j);
+      return make_float4(gated(v.x, g.x), gated(v.y, g.y), gated(v.z, g.z), gated(v.w, g.w));
+    };
+    float4 keep = make_float4(0.f, 0.f, 0.f, 0.f), w0 = keep;
+    for (int j = j0; j < part; j += 4 * blockDim.x) {
+      const float4 v = quad(j);
+      if (j == j0) {
+        keep = v;
+        w0 = *reinterpret_cast<const float4*>(wp + j);
+      }
+      ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+    }
+    const float f = 1.0f / sqrtf(block_sum(ss, scratch) / (float)part + eps);
+    for (int j = j0; j < part; j += 4 * blockDim.x) {
+      const float4 v = j == j0 ? keep : quad(j);
+      const float4 w = j == j0 ? w0 : *reinterpret_cast<const float4*>(wp + j);
+      const float a = v.x * f * w.x, b = v.y * f * w.y, c = v.z * f * w.z, d = v.w * f * w.w;
+      if (sizeof(TO) == 4)
+        *reinterpret_cast<float4*>(op + j) = make_float4(a, b, c, d);
+      else
+        *reinterpret_cast<uint2*>(op + j) = make_uint2(pack_bf16x2(a, b), pack_bf16x2(c, d));
+    }
+  } else {
+    for (int j = threadIdx.x; j < part; j += blockDim.x) {
+      const float v = gated(p[j], gp[j]);
+      ss = fmaf(v, v, ss);
+    }
+    const float f = 1.0f / sqrtf(block_sum(ss, scratch) / (float)part + eps);
+    for (int j = threadIdx.x; j < part; j += blockDim.x) Num<TO>::store(op + j, gated(p[j], gp[j]) * f * wp[j]);
+  }
+}
+
+extern "C" int rb_gate_rmsnorm_parts(const float* o, const float* weight, const float* gate, long long gate_stride, float eps, void* out,
+                                     int out_dtype, int n_tokens, int width, int parts, void* stream) {
+  RB_RECORDED(rb_gate_rmsnorm_parts(o, weight, gate, gate_stride, eps, out, out_dtype, n_tokens, width, parts, stream));
+  RB_REQUIRE(n_tokens >= 0 && width > 0 && parts > 0 && parts <= 65535 && width % parts == 0 && gate_stride >= width,
+             "rb_gate_rmsnorm_parts: bad sizes T=%d width=%d parts=%d", n_tokens, width, parts);
+  RB_REQUIRE(out_dtype == RB_F32 || out_dtype == RB_BF16, "rb_gate_rmsnorm_parts: unknown dtype %d", out_dtype);
+  if (n_tokens == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const int part = width / parts;
+  const bool vec = part % 4 == 0 && gate_stride % 4 == 0 && aligned(o) && aligned(weight) && aligned(gate) && aligned(out);
+  int threads = ((part / (vec ? 4 : 1) + RB_WAVE - 1) / RB_WAVE) * RB_WAVE;
+  threads = threads > 1024 ? 1024 : (threads < RB_WAVE ? RB_WAVE : threads);
+  const dim3 grid(n_tokens, parts);
+#define RB_GP(TO, VEC) \
+  gate_rmsnorm_parts_kernel<TO, VEC><<<grid, threads, 0, s>>>(o, weight, gate, (size_t)gate_stride, eps, (TO*)out, width, part)
+  if (out_dtype == RB_F32) {
+    if (vec) RB_GP(float, true);
+    else RB_GP(float, false);
+  } else {
+    if (vec) RB_GP(bf16_t, true);
+    else RB_GP(bf16_t, false);
+  }
+#undef RB_GP
   RB_LAUNCH_CHECK();
   return 0;
 }

@@ -218,6 +218,12 @@ __device__ __forceinline__ float gated_unit(float g, float u, float limit, float
   return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
 }
 
+// Experts may have no gate (w_gate null): y[row] = max(u, 0)^2 with u = Wu x.
+template <bool GATED>
+__device__ __forceinline__ float expert_unit(float g, float u, float limit, float alpha) {
+  return GATED ? gated_unit(g, u, limit, alpha) : squared_relu(u);
+}
+
 // ---------------------------------------------------------------- vector units: a wave per output
 template <typename T>
 __global__ void routed_up_generic_kernel(const T* __restrict__ h, const float* __restrict__ weight, int top,
@@ -234,17 +240,17 @@ __global__ void routed_up_generic_kernel(const T* __restrict__ h, const float* _
     const T* x = h + (size_t)(p / top) * width;
     const float wt = weight ? weight[p] : 1.0f;
     for (int j = blockIdx.y * n_waves + wave; j < ff; j += gridDim.y * n_waves) {
-      const T* gr = w_gate + ((size_t)e * ff + j) * width;
+      const T* gr = w_gate ? w_gate + ((size_t)e * ff + j) * width : nullptr;
       const T* ur = w_up + ((size_t)e * ff + j) * width;
       float g = 0.f, u = 0.f;
       for (int k = lane; k < width; k += RB_WAVE) {
         const float xv = Num<T>::load(x + k) * wt;
-        g = fmaf(Num<T>::load(gr + k), xv, g);
+        if (gr) g = fmaf(Num<T>::load(gr + k), xv, g);
         u = fmaf(Num<T>::load(ur + k), xv, u);
       }
-      g = wave_sum(g);
+      if (gr) g = wave_sum(g);
       u = wave_sum(u);
-      if (lane == 0) Num<T>::store(y + (size_t)row * ff + j, gated_unit(g, u, limit, alpha));
+      if (lane == 0) Num<T>::store(y + (size_t)row * ff + j, gr ? gated_unit(g, u, limit, alpha) : squared_relu(u));
     }
   }
 }
@@ -314,7 +320,7 @@ __global__ __launch_bounds__(256) void routed_gather_kernel(const bf16_t* __rest
 // run's tiles, walks the depth alone, in the order of the kernels below (so that a row's sums are the same bits), and asks for
 // RT_AHEAD steps at once, the experts' matrices past the caches.  The rows are read where they lie (no gathered copy).
 #define RT_AHEAD 8
-template <int NT, bool WEIGHTED>
+template <int NT, bool WEIGHTED, bool GATED>
 __global__ __launch_bounds__(256) void routed_up_few_kernel(const bf16_t* __restrict__ h, const float* __restrict__ weight, int top,
                                                             const int32_t* __restrict__ row_pair, const int32_t* __restrict__ tile_expert,
                                                             const int32_t* __restrict__ tile_pos, const bf16_t* __restrict__ w_gate,
@@ -338,7 +344,7 @@ __global__ __launch_bounds__(256) void routed_up_few_kernel(const bf16_t* __rest
     wt[j] = (WEIGHTED && p >= 0) ? weight[p] : 1.0f;
     xr[j] = h + (size_t)(p >= 0 ? p / top : 0) * width + 8 * grp;
   }
-  const bf16_t* gr = w_gate + ((size_t)e * ff + c0) * width + 8 * lane;
+  const bf16_t* gr = GATED ? w_gate + ((size_t)e * ff + c0) * width + 8 * lane : nullptr;
   const bf16_t* ur = w_up + ((size_t)e * ff + c0) * width + 8 * lane;
   f32x4_t ag[NT], au[NT];
 #pragma unroll
@@ -349,7 +355,7 @@ __global__ __launch_bounds__(256) void routed_up_few_kernel(const bf16_t* __rest
 #pragma unroll
     for (int u = 0; u < RT_AHEAD; ++u) {
       const size_t s = (size_t)(s0 + (u < cnt ? u : 0));
-      fg[u].u = load16_stream(gr + 512 * s);
+      if (GATED) fg[u].u = load16_stream(gr + 512 * s);
       fu[u].u = load16_stream(ur + 512 * s);
 #pragma unroll
       for (int j = 0; j < NT; ++j) fx[u][j].u = load16(xr[j] + 32 * s);
@@ -361,7 +367,7 @@ __global__ __launch_bounds__(256) void routed_up_few_kernel(const bf16_t* __rest
 #pragma unroll
       for (int j = 0; j < NT; ++j) {
         if (WEIGHTED) fx[u][j].u = scaled16(fx[u][j].u, wt[j]);
-        ag[j] = mfma16(fg[u], fx[u][j], ag[j]);
+        if (GATED) ag[j] = mfma16(fg[u], fx[u][j], ag[j]);
         au[j] = mfma16(fu[u], fx[u][j], au[j]);
       }
     }
@@ -375,8 +381,9 @@ __global__ __launch_bounds__(256) void routed_up_few_kernel(const bf16_t* __rest
     const int c = c0 + 4 * grp;
     bf16_t* dst = y + (size_t)(t0 + j) * RT_TILE * ff + (size_t)(c / 32) * 512 + 8 * (16 * ((c % 32) / 8) + r) + c % 8;
     const f32x4_t g = ag[j], u = au[j];
-    *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(gated_unit(g[0], u[0], limit, alpha), gated_unit(g[1], u[1], limit, alpha)),
-                                                pack_bf16x2(gated_unit(g[2], u[2], limit, alpha), gated_unit(g[3], u[3], limit, alpha)));
+    *reinterpret_cast<uint2*>(dst) =
+        make_uint2(pack_bf16x2(expert_unit<GATED>(g[0], u[0], limit, alpha), expert_unit<GATED>(g[1], u[1], limit, alpha)),
+                   pack_bf16x2(expert_unit<GATED>(g[2], u[2], limit, alpha), expert_unit<GATED>(g[3], u[3], limit, alpha)));
   }
 }
 
@@ -437,6 +444,7 @@ __global__ __launch_bounds__(256) void routed_down_few_kernel(const bf16_t* __re
 #define RT_GROUP 4
 #define RT_SPAN 16
 #define RT_THREADS 512
+template <bool GATED>
 __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t* __restrict__ xs, const int32_t* __restrict__ row_pair,
                                                              const int32_t* __restrict__ tile_expert,
                                                              const int32_t* __restrict__ tile_pos,
@@ -456,7 +464,7 @@ __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t
   if (c0 >= ff) return;
   const int r = lane & 15, grp = lane >> 4;
   const bf16_t* xr = xs + (size_t)t0 * RT_TILE * width + 8 * lane;
-  const bf16_t* gr = w_gate + ((size_t)e * ff + c0) * width + 8 * lane;
+  const bf16_t* gr = GATED ? w_gate + ((size_t)e * ff + c0) * width + 8 * lane : nullptr;
   const bf16_t* ur = w_up + ((size_t)e * ff + c0) * width + 8 * lane;
   const size_t blk = (size_t)16 * width;               // 16 rows further: the next block of channels, the next tile
   f32x4_t ag[RT_GROUP][2], au[RT_GROUP][2];
@@ -468,7 +476,7 @@ __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t
     Frag8 fg[2], fu[2], fx[RT_GROUP];
 #pragma unroll
     for (int cb = 0; cb < 2; ++cb) {
-      fg[cb].u = load16(gr + cb * blk + k);
+      if (GATED) fg[cb].u = load16(gr + cb * blk + k);
       fu[cb].u = load16(ur + cb * blk + k);
     }
 #pragma unroll
@@ -478,7 +486,7 @@ __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t
       if (j < nt) {
 #pragma unroll
         for (int cb = 0; cb < 2; ++cb) {
-          ag[j][cb] = mfma16(fg[cb], fx[j], ag[j][cb]);
+          if (GATED) ag[j][cb] = mfma16(fg[cb], fx[j], ag[j][cb]);
           au[j][cb] = mfma16(fu[cb], fx[j], au[j][cb]);
         }
       }
@@ -495,8 +503,9 @@ __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t
       const int c = c0 + 16 * cb + 4 * grp;
       bf16_t* dst = y + (size_t)(t0 + j) * RT_TILE * ff + (size_t)(c / 32) * 512 + 8 * (16 * ((c % 32) / 8) + r) + c % 8;
       const f32x4_t g = ag[j][cb], u = au[j][cb];
-      *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(gated_unit(g[0], u[0], limit, alpha), gated_unit(g[1], u[1], limit, alpha)),
-                                                  pack_bf16x2(gated_unit(g[2], u[2], limit, alpha), gated_unit(g[3], u[3], limit, alpha)));
+      *reinterpret_cast<uint2*>(dst) =
+          make_uint2(pack_bf16x2(expert_unit<GATED>(g[0], u[0], limit, alpha), expert_unit<GATED>(g[1], u[1], limit, alpha)),
+                     pack_bf16x2(expert_unit<GATED>(g[2], u[2], limit, alpha), expert_unit<GATED>(g[3], u[3], limit, alpha)));
     }
   }
 }
@@ -579,9 +588,9 @@ extern "C" int rb_routed_experts(const void* h, int dtype, const float* weight, 
                "rb_routed_experts: the matrix-core kernels need 16-byte aligned operands");
     bf16_t* xs = (bf16_t*)y + (size_t)max_rows * ff;
     routed_gather_kernel<<<tiles, 256, 0, s>>>((const bf16_t*)h, weight, top, row_pair, tile_expert, xs, width);
-    routed_up_mfma_kernel<<<dim3((ff + 63) / 64, tiles), RT_THREADS, 0, s>>>(xs, row_pair, tile_expert, tile_expert + tiles,
-                                                                        (const bf16_t*)w_gate, (const bf16_t*)w_up, (bf16_t*)y, width,
-                                                                        ff, limit, alpha, tiles);
+    auto up = w_gate ? routed_up_mfma_kernel<true> : routed_up_mfma_kernel<false>;
+    up<<<dim3((ff + 63) / 64, tiles), RT_THREADS, 0, s>>>(xs, row_pair, tile_expert, tile_expert + tiles, (const bf16_t*)w_gate,
+                                                          (const bf16_t*)w_up, (bf16_t*)y, width, ff, limit, alpha, tiles);
     routed_down_mfma_kernel<<<dim3((width + 127) / 128, tiles), RT_THREADS, 0, s>>>((const bf16_t*)y, row_pair, tile_expert,
                                                                              tile_expert + tiles, (const bf16_t*)w_down, out, width,
                                                                              ff, tiles);
@@ -620,7 +629,7 @@ extern "C" int rb_routed_experts_few(const void* h, const float* weight, int top
   const int tiles = max_rows / RT_TILE;
   const dim3 gu((ff + 63) / 64, tiles), gd((width + 63) / 64, tiles);
 #define RT_UP(NT, WEIGHTED)                                                                                                           \
-  routed_up_few_kernel<NT, WEIGHTED><<<gu, 256, 0, s>>>((const bf16_t*)h, weight, top, row_pair, tile_expert, tile_expert + tiles,    \
+  (w_gate ? routed_up_few_kernel<NT, WEIGHTED, true> : routed_up_few_kernel<NT, WEIGHTED, false>)<<<gu, 256, 0, s>>>((const bf16_t*)h, weight, top, row_pair, tile_expert, tile_expert + tiles,    \
                                                         (const bf16_t*)w_gate, (const bf16_t*)w_up, (bf16_t*)y, width, ff, limit, alpha, tiles)
 #define RT_DOWN(NT)                                                                                                       \
   routed_down_few_kernel<NT><<<gd, 256, 0, s>>>((const bf16_t*)y, row_pair, tile_expert, tile_expert + tiles,             \
@@ -663,13 +672,14 @@ extern "C" int rb_pairs_sum(const float* pairs, int top, float* out, int n_token
 
 // out[t] = sum over k of weight[p] * (sel[p] < n_experts ? pairs[p] : h[t]), p = t * top + k, in the order of k: the score
 // multiplies the expert's OUTPUT, and an output of the router behind the experts stands for the token's own input.
-// With `shared` (float32 [T, width], what an expert that every token uses gave): + sigmoid(gate[t * gate_stride]) * shared[t].
+// With `shared` (float32 [T, width], what an expert that every token uses gave): + sigmoid(gate[t * gate_stride]) * shared[t]
+// (gate null: + shared[t]).
 template <typename T>
 __global__ void experts_combine_kernel(const float* __restrict__ pairs, const int32_t* __restrict__ sel, const float* __restrict__ weight,
                                        int top, int n_experts, const T* __restrict__ h, const float* __restrict__ shared,
                                        const float* __restrict__ gate, size_t gate_stride, float* __restrict__ out, int width) {
   const int t = blockIdx.x;
-  const float sg = shared ? 1.0f / (1.0f + expf(-gate[(size_t)t * gate_stride])) : 0.f;
+  const float sg = !shared ? 0.f : gate ? 1.0f / (1.0f + expf(-gate[(size_t)t * gate_stride])) : 1.0f;
   for (int j = threadIdx.x; j < width; j += blockDim.x) {
     float v = 0.f;
     for (int k = 0; k < top; ++k) {
@@ -687,7 +697,6 @@ extern "C" int rb_experts_combine(const float* pairs, const int32_t* sel, const 
                                   int width, void* stream) {
   RB_RECORDED(rb_experts_combine(pairs, sel, weight, top, n_experts, h, h_dtype, shared, gate, gate_stride, out, n_tokens, width, stream));
   RB_REQUIRE(n_tokens >= 0 && width > 0 && top > 0 && n_experts >= 0, "rb_experts_combine: bad sizes");
-  RB_REQUIRE(shared == nullptr || gate != nullptr, "rb_experts_combine: a shared expert comes with its gate");
   if (n_tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   const int threads = width >= 256 ? 256 : 64;

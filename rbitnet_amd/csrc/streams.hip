@@ -1,6 +1,7 @@
 // A residual stream kept as several copies (hyper-connections), layer norm with weight and bias, and two small
 // element-wise functions: the xIELU activation and the tanh cap of logits.  float32 arithmetic throughout.
 //
+// (The kernels for RMS norms of such streams take an update's term as a sum of terms as well.)
 // The streams are x [S, T, E], stream_stride floats from one copy to the next.  A sublayer reads the mixture
 // u = sum_s coef[s] x[s], and afterwards every copy is rebuilt from all the old ones:
 //   x'[j] = sum_s mix[s, j] x[s] + out[j] * (scale * y)
@@ -318,6 +319,234 @@ extern "C" int rb_embed_streams(const void* table, int table_dtype, const int32_
     embed_streams_kernel<bf16_t><<<n_tokens, 256, 0, s>>>((const bf16_t*)table, ids, x, n_streams, (size_t)stream_stride, width);
   else
     RB_REQUIRE(false, "rb_embed_streams: unknown dtype %d", table_dtype);
+  RB_LAUNCH_CHECK();
+  return 0;
+}
+
+// The same with what a model may do to an embedding's row: x[s][t, :] = table[ids[t], :] * scale + wave(pos[t]), where number 2i of
+// wave(p) is sin(p inv[i]) and number 2i + 1 is cos(p inv[i]) (inv float64 [(width + 1) / 2]; null: no wave).  The angle is
+// made and brought into one turn in float64, so that a late position's sine is as good as an early one's.
+template <typename T>
+__global__ void embed_streams_waves_kernel(const T* __restrict__ table, const int32_t* __restrict__ ids, float scale,
+                                           const double* __restrict__ inv, const int32_t* __restrict__ tok_pos, float* __restrict__ x,
+                                           int n_streams, size_t stream_stride, int width) {
+  const int t = blockIdx.x;
+  const T* row = table + (size_t)ids[t] * width;
+  const double pos = (double)tok_pos[t];
+  const int n_pairs = (width + 1) / 2;
+  for (int i = threadIdx.x; i < n_pairs; i += blockDim.x) {
+    float sn = 0.f, cs = 0.f;
+    if (inv) {
+      const double angle = pos * inv[i];
+      const double turns = rint(angle * 0.15915494309189535);
+      sincosf((float)fma(-turns, 6.283185307179586, angle), &sn, &cs);
+    }
+    const float a = fmaf(Num<T>::load(row + 2 * i), scale, sn);
+    const bool two = 2 * i + 1 < width;
+    const float b = two ? fmaf(Num<T>::load(row + 2 * i + 1), scale, cs) : 0.f;
+    for (int s = 0; s < n_streams; ++s) {
+      float* xr = x + (size_t)s * stream_stride + (size_t)t * width + 2 * i;
+      xr[0] = a;
+      if (two) xr[1] = b;
+    }
+  }
+}
+
+extern "C" int rb_embed_streams_waves(const void* table, int table_dtype, const int32_t* ids, float scale, const double* inv,
+                                      const int32_t* tok_pos, float* x, int n_streams, long long stream_stride, int n_tokens, int width,
+                                      void* stream) {
+  RB_RECORDED(rb_embed_streams_waves(table, table_dtype, ids, scale, inv, tok_pos, x, n_streams, stream_stride, n_tokens, width, stream));
+  RB_REQUIRE(n_tokens >= 0 && width > 0 && n_streams >= 1 && stream_stride >= 0, "rb_embed_streams_waves: bad sizes");
+  RB_REQUIRE(inv == nullptr || tok_pos != nullptr, "rb_embed_streams_waves: a wave needs the tokens' positions");
+  if (n_tokens == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  if (table_dtype == RB_F32)
+    embed_streams_waves_kernel<float><<<n_tokens, 256, 0, s>>>((const float*)table, ids, scale, inv, tok_pos, x, n_streams,
+                                                               (size_t)stream_stride, width);
+  else if (table_dtype == RB_BF16)
+    embed_streams_waves_kernel<bf16_t><<<n_tokens, 256, 0, s>>>((const bf16_t*)table, ids, scale, inv, tok_pos, x, n_streams,
+                                                                (size_t)stream_stride, width);
+  else
+    RB_REQUIRE(false, "rb_embed_streams_waves: unknown dtype %d", table_dtype);
+  RB_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---------------------------------------------------------------- RMS norm of a stream in several copies
+// out[r] = u / sqrt(mean(u^2) + eps) * gain, u = sum_s coef[s] x[s][src], src = rows ? rows[r] : r (coef null: the plain sum).
+// With an update that was still to be done (mix not null) the copies are first rebuilt from all the old ones,
+//   x[t] <- sum_s mix[s, t] x[s] + out_coef[t] * y,
+// in the same pass; with rows the copies stay as they are (nobody reads them again).  y of a row is a sum of terms:
+//   y = sum_k (weights ? weights[src * n_terms + k] : 1) y[src * row_stride + k * term_stride]  +  sum_k extra[src * width + k * extra_stride]
+// (the K slices of a product; the outputs of a token's experts and what a shared expert adds).  NS copies, or, NS 0, n_streams.
+struct StreamsNormArgs {
+  int n_streams;
+  size_t stream_stride;
+  int n_terms;
+  size_t term_stride, row_stride;
+  int n_extra;
+  size_t extra_stride;
+  float eps;
+  int width;
+};
+template <int V>
+struct Piece {
+  float v[V];
+};
+template <int V>
+__device__ __forceinline__ Piece<V> load_piece(const float* p) {
+  Piece<V> r;
+  if (V == 4) {
+    const float4 q = ld4(p);
+    r.v[0] = q.x;
+    r.v[V > 1 ? 1 : 0] = q.y;
+    r.v[V > 2 ? 2 : 0] = q.z;
+    r.v[V - 1] = q.w;
+  } else {
+    r.v[0] = *p;
+  }
+  return r;
+}
+template <int V>
+__device__ __forceinline__ void store_piece_f32(float* p, const Piece<V>& r) {
+  if (V == 4) st4(p, r.v[0], r.v[V > 1 ? 1 : 0], r.v[V > 2 ? 2 : 0], r.v[V - 1]);
+  else *p = r.v[0];
+}
+template <int V>
+__device__ __forceinline__ void add_terms(Piece<V>& acc, const float* p, int n_terms, size_t stride, const float* w) {
+  int k = 0;
+  for (; k + 3 < n_terms; k += 4) {                 // four terms in flight
+    Piece<V> e[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) e[u] = load_piece<V>(p + (size_t)(k + u) * stride);
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const float f = w ? w[k + u] : 1.0f;
+#pragma unroll
+      for (int i = 0; i < V; ++i) acc.v[i] = fmaf(f, e[u].v[i], acc.v[i]);
+    }
+  }
+  for (; k < n_terms; ++k) {
+    const Piece<V> e = load_piece<V>(p + (size_t)k * stride);
+    const float f = w ? w[k] : 1.0f;
+#pragma unroll
+    for (int i = 0; i < V; ++i) acc.v[i] = fmaf(f, e.v[i], acc.v[i]);
+  }
+}
+
+template <typename TO, int V, int NS>
+__global__ __launch_bounds__(1024) void streams_rmsnorm_kernel(StreamsNormArgs p, float* __restrict__ x, const float* __restrict__ mix,
+                                                               const float* __restrict__ out_coef, const float* __restrict__ y,
+                                                               const float* __restrict__ weights, const float* __restrict__ extra,
+                                                               const float* __restrict__ coef, const float* __restrict__ gain,
+                                                               const int32_t* __restrict__ rows, TO* __restrict__ out) {
+  extern __shared__ float u[];
+  __shared__ float scratch[16];
+  constexpr int MOST = NS > 0 ? NS : ST_MAX_STREAMS;
+  const int n = NS > 0 ? NS : p.n_streams;
+  const int r = blockIdx.x;
+  const size_t src = rows ? (size_t)rows[r] : (size_t)r;
+  const bool write_back = mix != nullptr && rows == nullptr;
+  float ss = 0.f;
+  for (int j = V * threadIdx.x; j < p.width; j += V * blockDim.x) {
+    Piece<V> old[MOST], v, yv;
+#pragma unroll
+    for (int s = 0; s < MOST; ++s)
+      if (s < n) old[s] = load_piece<V>(x + (size_t)s * p.stream_stride + src * p.width + j);
+#pragma unroll
+    for (int i = 0; i < V; ++i) v.v[i] = yv.v[i] = 0.f;
+    if (mix) {
+      add_terms<V>(yv, y + src * p.row_stride + j, p.n_terms, p.term_stride, weights ? weights + src * p.n_terms : nullptr);
+      if (extra) add_terms<V>(yv, extra + src * p.width + j, p.n_extra, p.extra_stride, nullptr);
+#pragma unroll
+      for (int t = 0; t < MOST; ++t) {
+        if (t < n) {
+          const float oc = out_coef[t], ic = coef ? coef[t] : 1.0f;
+          Piece<V> nv;
+#pragma unroll
+          for (int i = 0; i < V; ++i) nv.v[i] = oc * yv.v[i];
+#pragma unroll
+          for (int s = 0; s < MOST; ++s)
+            if (s < n) {
+              const float m = mix[s * n + t];
+#pragma unroll
+              for (int i = 0; i < V; ++i) nv.v[i] = fmaf(m, old[s].v[i], nv.v[i]);
+            }
+          if (write_back) store_piece_f32<V>(x + (size_t)t * p.stream_stride + src * p.width + j, nv);
+#pragma unroll
+          for (int i = 0; i < V; ++i) v.v[i] = fmaf(ic, nv.v[i], v.v[i]);
+        }
+      }
+    } else {
+#pragma unroll
+      for (int s = 0; s < MOST; ++s)
+        if (s < n) {
+          const float ic = coef ? coef[s] : 1.0f;
+#pragma unroll
+          for (int i = 0; i < V; ++i) v.v[i] = fmaf(ic, old[s].v[i], v.v[i]);
+        }
+    }
+    store_piece_f32<V>(u + j, v);
+#pragma unroll
+    for (int i = 0; i < V; ++i) ss = fmaf(v.v[i], v.v[i], ss);
+  }
+  // the gain of this thread's first numbers is asked for now, so that it arrives under the reduction
+  const int j0 = V * threadIdx.x;
+  Piece<V> g0;
+#pragma unroll
+  for (int i = 0; i < V; ++i) g0.v[i] = 0.f;
+  if (j0 < p.width) g0 = load_piece<V>(gain + j0);
+  __builtin_amdgcn_sched_barrier(0);
+  const float f = 1.0f / sqrtf(block_sum(ss, scratch) / (float)p.width + p.eps);
+  TO* orow = out + (size_t)r * p.width;
+  for (int j = j0; j < p.width; j += V * blockDim.x) {
+    const Piece<V> v = load_piece<V>(u + j), g = j == j0 ? g0 : load_piece<V>(gain + j);
+    if (V == 4)
+      st4(orow + j, v.v[0] * f * g.v[0], v.v[V > 1 ? 1 : 0] * f * g.v[V > 1 ? 1 : 0], v.v[V > 2 ? 2 : 0] * f * g.v[V > 2 ? 2 : 0],
+          v.v[V - 1] * f * g.v[V - 1]);
+    else
+      Num<TO>::store(orow + j, v.v[0] * f * g.v[0]);
+  }
+}
+
+extern "C" int rb_streams_rmsnorm(float* x, int n_streams, long long stream_stride, const float* mix, const float* out_coef, const float* y,
+                                  int n_terms, long long term_stride, long long row_stride, const float* weights, const float* extra,
+                                  int n_extra, long long extra_stride, const float* coef, const float* gain, float eps,
+                                  const int32_t* rows, int n_rows, int width, void* out, int out_dtype, void* stream) {
+  RB_RECORDED(rb_streams_rmsnorm(x, n_streams, stream_stride, mix, out_coef, y, n_terms, term_stride, row_stride, weights, extra, n_extra,
+                                 extra_stride, coef, gain, eps, rows, n_rows, width, out, out_dtype, stream));
+  RB_REQUIRE(n_rows >= 0 && width > 0 && width <= 16384, "rb_streams_rmsnorm: bad sizes %d x %d (width at most 16384)", n_rows, width);
+  RB_REQUIRE(n_streams >= 1 && n_streams <= ST_MAX_STREAMS && stream_stride >= 0, "rb_streams_rmsnorm: %d streams (1 to %d)", n_streams,
+             ST_MAX_STREAMS);
+  RB_REQUIRE(mix == nullptr || (out_coef != nullptr && y != nullptr && n_terms >= 1 && term_stride >= 0 && row_stride >= width),
+             "rb_streams_rmsnorm: an update needs out_coef and the terms of y");
+  RB_REQUIRE(extra == nullptr || (mix != nullptr && n_extra >= 1 && extra_stride >= 0), "rb_streams_rmsnorm: more terms go with an update");
+  RB_REQUIRE(out_dtype == RB_F32 || out_dtype == RB_BF16, "rb_streams_rmsnorm: unknown dtype %d", out_dtype);
+  if (n_rows == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  const size_t lds = (size_t)width * sizeof(float);
+  auto aligned = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
+  const bool vec = width % 4 == 0 && stream_stride % 4 == 0 && term_stride % 4 == 0 && row_stride % 4 == 0 && extra_stride % 4 == 0 &&
+                   aligned(x) && aligned(y) && aligned(extra) && aligned(gain) && aligned(out);
+  const StreamsNormArgs p = {n_streams, (size_t)stream_stride, n_terms, (size_t)term_stride, (size_t)row_stride, n_extra,
+                             (size_t)extra_stride, eps, width};
+  int threads = vec ? ((width / 4 + RB_WAVE - 1) / RB_WAVE) * RB_WAVE : 256;
+  if (threads > 1024) threads = 1024;
+#define ST_GO(TO, V, NS) \
+  streams_rmsnorm_kernel<TO, V, NS><<<n_rows, threads, lds, s>>>(p, x, mix, out_coef, y, weights, extra, coef, gain, rows, (TO*)out)
+#define ST_BY_COPIES(TO)                    \
+  do {                                      \
+    if (!vec) ST_GO(TO, 1, 0);              \
+    else if (n_streams == 1) ST_GO(TO, 4, 1); \
+    else if (n_streams == 2) ST_GO(TO, 4, 2); \
+    else if (n_streams == 3) ST_GO(TO, 4, 3); \
+    else if (n_streams == 4) ST_GO(TO, 4, 4); \
+    else ST_GO(TO, 4, 0);                   \
+  } while (0)
+  if (out_dtype == RB_F32) ST_BY_COPIES(float);
+  else ST_BY_COPIES(bf16_t);
+#undef ST_BY_COPIES
+#undef ST_GO
   RB_LAUNCH_CHECK();
   return 0;
 }

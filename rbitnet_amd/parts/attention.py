@@ -28,7 +28,7 @@ and four more, each of which sends the layer through the kernels that take all h
   chunk       None, or c: a query at position i sees the keys j <= i with i // c == j // c only, chunks being counted
               from the sequence's first position, whatever a step brings.
 These go without a rotation (position "none") and without a sink.  (A chunk also goes with everything below.)
-Eight more send the layer through a third way, in which q, k and v are prepared by kernels of their own in front of attention
+Ten more send the layer through a third way, in which q, k and v are prepared by kernels of their own in front of attention
 (biases and a norm with a weight belong to it too, and a rotation is welcome):
   conv        None, or the taps of a short causal convolution over time on every channel of q, k and v (tensors "q_conv",
               "k_conv", "v_conv" [channels, taps], no bias), directly behind the projection and its bias; the last taps - 1
@@ -42,6 +42,8 @@ Eight more send the layer through a third way, in which q, k and v are prepared 
   value_norm  None, or e: every value head is divided by sqrt(mean(head^2) + e) (no weight) and cached so;
   weights     "sigmoid": a visible key's weight is sigmoid(score + b[head]) by itself, not normalised over the keys, b the
               tensor "score_bias" [heads] (float32); "softmax" otherwise;
+  values      "keys": the values are the keys as they are cached (no value matrix, value_dim is head_dim, one set of pages);
+  sink        "one": the softmax's denominator is one plus the sum, which is a sink of exactly 0 for every head, without a tensor;
   gate        "elementwise": the concatenated heads are multiplied number by number with sigmoid(Wg h) (tensor "gate"
               [heads * value_dim, E]) before the output matrix.
 A position part that rotates only the first numbers of a head says so with its own head_dim
@@ -101,7 +103,14 @@ class Attention(Part):
         self.value_dim = int(params.get("value_dim") or self.head_dim)
         if not 0 < self.value_dim <= 512:
             raise ConfigError(f"attention: value_dim {self.value_dim} not supported (1 to 512)")
+        self.one_sink = params.get("sink") == "one"
         self.has_sink, self.has_gate = bool(params.get("sink")), bool(params.get("head_gate"))
+        values = str(params.get("values") or "own")
+        if values not in ("own", "keys"):
+            raise ConfigError(f"attention: unknown values {values!r} (own, keys)")
+        self.own_values = values == "own"
+        if not self.own_values and self.value_dim != self.head_dim:
+            raise ConfigError(f"attention: values that are the keys have the keys' size {self.head_dim}, not {self.value_dim}")
         self.scale = float(params.get("scale") or self.head_dim ** -0.5)
         self.window = params.get("window")
         if self.window is not None and int(self.window) <= 0:
@@ -153,7 +162,11 @@ class Attention(Part):
         if self.keep_first < 0 or (self.keep_first and self.window is None):
             raise ConfigError("attention: kept first tokens go with a window")
         self.prepared = bool(self.taps is not None or self.qk_weight or self.softcap is not None or self.keep_first
-                             or self.gate_kind == "elementwise" or self.value_eps is not None or self.sigmoid)
+                             or self.gate_kind == "elementwise" or self.value_eps is not None or self.sigmoid or not self.own_values
+                             or self.one_sink)
+        if not self.own_values and (self.taps is not None or params.get("bias") or self.qk_eps is not None or self.value_eps is not None
+                                    or params.get("cache_from") is not None):
+            raise ConfigError("attention: values that are the keys go without convolutions, biases, norms and another layer's cache")
         if self.prepared and self.has_talk:
             raise ConfigError("attention: mixed heads go without a convolution, weighted norms, capped scores, "
                               "kept first tokens, an elementwise gate, norms of the values and sigmoid weights")
@@ -164,7 +177,7 @@ class Attention(Part):
             if self.cache_from is None:
                 n_ch += self.n_kv * (self.head_dim + self.value_dim)
             self.conv = ShortConv(n_ch, self.taps or 1, env, residual=False, act=ACT_NONE)
-        if self.prepared and (self.sigmoid or self.whole_norm) and env.dtype == torch.bfloat16 and not getattr(env, "generic_only", False):
+        if self.prepared and (self.sigmoid or self.whole_norm or not self.own_values) and env.dtype == torch.bfloat16 and not getattr(env, "generic_only", False):
             # a head size of the matrix cores' kernels where one is near (zeros cost cache, not correctness)
             for size in _MATRIX_CORE_HEAD_DIMS:
                 if self.pad <= size and 2 * self.pad >= size:
@@ -194,7 +207,8 @@ class Attention(Part):
                  self.names["o"]: TensorSpec((self.hidden, self.n_heads * self.value_dim))}
         if self.cache_from is None:
             specs[self.names["k"]] = TensorSpec((kd, self.hidden))
-            specs[self.names["v"]] = TensorSpec((self.n_kv * self.value_dim, self.hidden))
+            if self.own_values:
+                specs[self.names["v"]] = TensorSpec((self.n_kv * self.value_dim, self.hidden))
         if self.has_bias:
             specs[self.names["q_bias"]] = TensorSpec((qd,), role="gain", init="normal")
             if self.cache_from is None:
@@ -202,7 +216,7 @@ class Attention(Part):
                 specs[self.names["v_bias"]] = TensorSpec((self.n_kv * self.value_dim,), role="gain", init="normal")
         if self.has_talk:
             specs[self.names["talk"]] = TensorSpec((self.n_heads, self.n_heads), role="gain", init="eye_normal")
-        if self.has_sink:
+        if self.has_sink and not self.one_sink:
             specs[self.names["sink"]] = TensorSpec((self.n_heads,), role="gain", init="normal")
         if self.has_gate:
             rows = self.n_heads * (self.value_dim if self.gate_kind == "elementwise" else 1)
@@ -225,7 +239,7 @@ class Attention(Part):
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         # q, k and v rows in one matrix: one product per step instead of three
         lib, allowed = self.env.lib, not getattr(self.env, "generic_only", False)
-        names = ("q", "k", "v") if self.cache_from is None else ("q",)
+        names = ("q",) if self.cache_from is not None else ("q", "k", "v") if self.own_values else ("q", "k")
         pieces, row = [], 0
         for n in names:
             t = tensors[self.names[n]]
@@ -249,7 +263,9 @@ class Attention(Part):
                                           and self.pad in _MATRIX_CORE_HEAD_DIMS and self.n_heads <= MIXED_MATRIX_CORE_HEADS)
         if self.mixed_on_matrix_cores and self.talk is None:
             self.talk = torch.eye(self.n_heads, dtype=torch.float32, device=o.device)
-        if self.has_sink:
+        if self.one_sink:
+            self.sink = torch.zeros(self.n_heads, dtype=torch.float32, device=o.device)
+        elif self.has_sink:
             self.sink = tensors[self.names["sink"]]
         if self.gate_kind == "head":
             # rows up to a multiple of 16 (zeros), so that the product's kernels find whole tiles
@@ -287,7 +303,8 @@ class Attention(Part):
     def cache_request(self) -> Optional[CacheRequest]:
         if self.cache_from is not None:
             return None
-        return CacheRequest("kv", heads=self.n_kv, head_dim=self.pad, window=self.reach, keep_first=self.keep_first)
+        return CacheRequest("kv", heads=self.n_kv, head_dim=self.pad, window=self.reach, keep_first=self.keep_first,
+                            values=self.own_values)
 
     def cache_requests(self):
         out = [r for r in (self.cache_request(),) if r is not None]
@@ -327,8 +344,8 @@ class Attention(Part):
             lib.norm_rope_store(qkv, cos, sin, self.rot, self.q_norm_w, self.k_norm_w, self.qk_eps, q, k_pages, v_pages,
                                 ctx.tok_pos, ctx.tok_seq, view.block_table, hq, hk, self.head_dim, self.value_dim, d)
         else:
-            lib.rope_store(qkv, cos, sin, self.rot, q, k_pages, v_pages, ctx.tok_pos, ctx.tok_seq, view.block_table, hq, hk,
-                           self.head_dim, self.value_dim, d)
+            lib.rope_store(qkv, cos, sin, self.rot, q, k_pages, v_pages if self.own_values else None, ctx.tok_pos, ctx.tok_seq,
+                           view.block_table, hq, hk, self.head_dim, self.value_dim, d)
         attn = torch.empty((t, hq * d), dtype=self.env.dtype, device=h.device)
         window = int(self.window) if self.window is not None else 0
         fast = (self.env.dtype == torch.bfloat16 and d in _MATRIX_CORE_HEAD_DIMS and not getattr(self.env, "generic_only", False))

@@ -10,7 +10,9 @@ embedding "table" (crates/bitnet-core/src/llama/model.rs:229-232): x[t, :] = tab
     Parameters: name, vocab_size, streams (None: the stream is [T, E]; n: n equal copies [n, T, E], for
     blocks that keep the residual stream in several copies), scale (None, or c: the rows are multiplied by c),
     positions (None, or {"name": tensor, "max_positions": n}: a learned vector per absolute position [n, E], added
-    to the scaled row as it is): x[t, :] = table[id[t], :] * c + positions[pos[t], :]; norm (None, or a PartSpec of a norm
+    to the scaled row as it is): x[t, :] = table[id[t], :] * c + positions[pos[t], :]; waves (None, or b: a fixed vector per
+    absolute position p is added, whose numbers 2i and 2i + 1 are the sine and the cosine of p b^(-2i / E); with `scale` it also goes
+    with several copies of the stream); norm (None, or a PartSpec of a norm
     that offers `add_normed`) with norm_name (its tensor): the stream starts as norm(row), and the first block also gets
     these rows in the compute dtype (forward then returns the stream and a `StreamCopy`).
     Interface of an embedding: tensor_specs() / load(tensors) / forward(ctx) -> float32 [T, E]
@@ -52,8 +54,15 @@ class TableEmbedding(Part):
         pos = params.get("positions")
         self.pos_name = None if pos is None else str(pos["name"])
         self.max_positions = None if pos is None else int(pos["max_positions"])
-        if (self.scale is not None or pos is not None) and self.streams is not None:
-            raise ConfigError("an embedding with a scale or learned positions fills one copy of the stream")
+        self.waves = None if params.get("waves") is None else float(params["waves"])
+        if pos is not None and (self.streams is not None or self.waves is not None):
+            raise ConfigError("an embedding with learned positions fills one copy of the stream, and has no waves")
+        if self.waves is not None and not self.waves > 0:
+            raise ConfigError(f"an embedding's waves need a positive base, found {self.waves}")
+        self.inv = None
+        if self.waves is not None and env.lib is not None:
+            i = torch.arange((self.hidden + 1) // 2, dtype=torch.float64)
+            self.inv = torch.pow(torch.tensor(self.waves, dtype=torch.float64), -2.0 * i / self.hidden).to(env.device)
         self.norm = None
         if params.get("norm") is not None:
             self.norm = build_part("norm", params["norm"], env)
@@ -92,10 +101,17 @@ class TableEmbedding(Part):
     def forward(self, ctx) -> torch.Tensor:
         if self.streams is not None:
             x = torch.empty((self.streams, ctx.n_tokens, self.hidden), dtype=torch.float32, device=self.table.device)
-            self.env.lib.embed_streams(self.table, ctx.token_ids, x)
+            if self.waves is not None or self.scale is not None:
+                self.env.lib.embed_streams_waves(self.table, ctx.token_ids, 1.0 if self.scale is None else self.scale, self.inv,
+                                                 ctx.tok_pos, x)
+            else:
+                self.env.lib.embed_streams(self.table, ctx.token_ids, x)
             return x
         x = torch.empty((ctx.n_tokens, self.hidden), dtype=torch.float32, device=self.table.device)
-        if self.scale is not None or self.positions is not None:
+        if self.waves is not None:
+            self.env.lib.embed_streams_waves(self.table, ctx.token_ids, 1.0 if self.scale is None else self.scale, self.inv,
+                                             ctx.tok_pos, x.unsqueeze(0))
+        elif self.scale is not None or self.positions is not None:
             self.env.lib.embed_scaled_pos(self.table, ctx.token_ids, 1.0 if self.scale is None else self.scale,
                                           self.positions, ctx.tok_pos, x)
         else:

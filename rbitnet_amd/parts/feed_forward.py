@@ -63,18 +63,20 @@ class DenseAct(Part):
     """out = Wdown act(Wup h), the activation applied where the first product stores its float32 sums.
     activation "xielu": for z > 0, softplus(p) z^2 + z / 2; for z <= 0, (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2,
     (p, q) being the two numbers of the tensor `act`.  activation "gelu_tanh": z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))),
-    no tensor.  Parameters: intermediate_size, activation, names ({"up", "down", "act"})."""
+    no tensor.  activation "squared_relu": max(z, 0)^2, no tensor.  The output product may leave its K slices to the norm that
+    follows.  Parameters: intermediate_size, activation, names ({"up", "down", "act"})."""
     graph_safe = True
     plan_safe = True
     adds_to_stream = True
+    leaves_terms = True
     activation = "xielu"
 
     def __init__(self, params: Dict, env: BuildEnv):
         self.env = env
         self.ff = int(params["intermediate_size"])
         self.activation = str(params.get("activation", type(self).activation))
-        if self.activation not in ("xielu", "gelu_tanh"):
-            raise ConfigError(f"dense feed-forward: activation {self.activation!r} not supported (xielu, gelu_tanh)")
+        if self.activation not in ("xielu", "gelu_tanh", "squared_relu"):
+            raise ConfigError(f"dense feed-forward: activation {self.activation!r} not supported (xielu, gelu_tanh, squared_relu)")
         self.names = dict({"up": "up", "down": "down", "act": "act"}, **(params.get("names") or {}))
         self.hidden = env.hidden_size
 
@@ -92,8 +94,9 @@ class DenseAct(Part):
                                 down.device, allowed)
         if self.activation == "xielu":
             self.act = tensors[self.names["act"]]
-        else:       # the kernels read a first number that is no number as "the tanh form of GELU"
-            self.act = torch.tensor([float("nan"), 0.0], dtype=torch.float32, device=up.device)
+        else:       # a first number that is no number tells the kernels that the second names another activation
+            code = 0.0 if self.activation == "gelu_tanh" else 1.0
+            self.act = torch.tensor([float("nan"), code], dtype=torch.float32, device=up.device)
 
     def forward(self, h, ctx=None, stream: Optional[torch.Tensor] = None, next_norm=None):
         lib = self.env.lib

@@ -36,9 +36,14 @@ class RMSNorm(Part):
     below the part's prefix; an empty name is the prefix itself).
 
     `add_normed` is the norm on a sublayer's OUTPUT: x <- x + norm(sa a + sb b), for layers whose sublayers read the stream
-    itself; it also leaves the new rows in the compute dtype for the next sublayer."""
+    itself; it also leaves the new rows in the compute dtype for the next sublayer.
+
+    The stream may come in several copies [S, T, E]: the norm then reads sum_s coef[s] x[s] (`coef` None: the plain sum), behind
+    the update of the copies that delta (a `StreamsUpdate`) may still hold."""
     graph_safe = True
     plan_safe = True
+    reads_copies = True
+    adds_update_terms = True
     folds_into_products = True
     adds_terms = True
 
@@ -67,9 +72,15 @@ class RMSNorm(Part):
         self.env.lib.outnorm_residual(x, a, b, sa, sb, self.weight, self.eps, assign, h_out)
 
     def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor] = None,
-                rows: Optional[torch.Tensor] = None, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
-        n = x.shape[0] if rows is None else rows.shape[0]
+                rows: Optional[torch.Tensor] = None, out_dtype: Optional[torch.dtype] = None,
+                coef: Optional[torch.Tensor] = None) -> torch.Tensor:
+        n = x.shape[-2] if rows is None else rows.shape[0]
         out = torch.empty((n, self.size), dtype=out_dtype or self.env.dtype, device=x.device)
+        if x.dim() == 3:
+            if delta is not None and (not isinstance(delta, StreamsUpdate) or delta.scale is not None):
+                raise ConfigError("an RMS norm of a stream in several copies takes an update of the copies without a scale per channel")
+            self.env.lib.streams_rmsnorm(x, coef, self.weight, self.eps, rows, out, update=None if delta is None else delta.term_parts())
+            return out
         self.env.lib.add_rmsnorm(x, delta, self.weight, self.eps, rows, out)
         return out
 
@@ -81,6 +92,7 @@ class LayerNorm(Part):
     [S, T, E]: the norm then reads sum_s coef[s] x[s] (`coef` None: the plain sum)."""
     graph_safe = True
     plan_safe = True
+    reads_copies = True
     adds_scaled_sum = True        # delta may be a ScaledSum: scale * (a + b), added in the norm's own pass
 
     def __init__(self, params: Dict, env: BuildEnv):

@@ -20,10 +20,12 @@ A second family of routers is served by the same launches, each choice a paramet
     weight_on    "input" (above), or "output": out = sum over the chosen of s_e * expert_e(h)
     limit        None: no clamps, and the plain gate: expert(x) = Wd (silu(Wg x) * (Wu x))
     shared       None, or {"intermediate_size": f}: an expert of the plain gated form (tensors "shared.gate", "shared.up",
-                 "shared.down") that every token uses, added times sigmoid(w . h), w the tensor "shared.sg" [1, E]
+                 "shared.down") that every token uses, added times sigmoid(w . h), w the tensor "shared.sg" [1, E]; with
+                 {"gate": False} it is added as it is and has no such tensor
+    unit         "gated" (above), or "squared_relu": expert(x) = Wd max(Wu x, 0)^2, the shared expert likewise; no gate matrices
     bias         True: the tensor "router_bias" (one number per output) is added to the router's logits
-With score "chosen" the choice goes by the logits and the weights are the softmax over the chosen logits alone; otherwise the
-weights of the chosen are never renormalised.  Router logits, scores, the choice and all sums are float32.
+With score "chosen" the choice goes by the logits and the weights are the softmax over the chosen logits alone (which is also the
+softmax over all outputs, divided by the sum of the chosen ones); otherwise the weights of the chosen are never renormalised.  Router logits, scores, the choice and all sums are float32.
 """
 from __future__ import annotations
 
@@ -33,7 +35,7 @@ import torch
 
 from ..errors import ConfigError
 from .base import BuildEnv, Part, TensorSpec, register_feed_forward
-from .feed_forward import SwiGLU
+from .feed_forward import DenseAct, SwiGLU
 from .linear import linear, pack_rows
 from .stream import ExpertPairs
 
@@ -76,18 +78,29 @@ class RoutedExperts(Part):
             raise ConfigError("routed experts: outputs behind the experts go with weights on the experts' outputs")
         self.names = dict(DEFAULT_NAMES, **(params.get("names") or {}))
         self.hidden = env.hidden_size
+        self.unit = str(params.get("unit", "gated"))
+        if self.unit not in ("gated", "squared_relu"):
+            raise ConfigError(f"routed experts: unit {self.unit!r} not supported (gated, squared_relu)")
+        if self.unit != "gated" and self.limit is not None:
+            raise ConfigError("routed experts: limits belong to gated experts")
         shared = params.get("shared")
-        self.shared = None
+        self.shared, self.shared_gate = None, bool(shared is not None and shared.get("gate", True))
         if shared is not None:
             if self.weight_on != "output":
                 raise ConfigError("routed experts: a shared expert goes with weights on the experts' outputs")
             base = self.names["shared"]
-            self.shared = SwiGLU({"intermediate_size": int(shared["intermediate_size"]),
-                                  "names": {"gate": f"{base}.gate", "up": f"{base}.up", "down": f"{base}.down"}}, env)
+            names = {"gate": f"{base}.gate", "up": f"{base}.up", "down": f"{base}.down"}
+            size = int(shared["intermediate_size"])
+            if self.unit == "gated":
+                self.shared = SwiGLU({"intermediate_size": size, "names": names}, env)
+            else:
+                self.shared = DenseAct({"intermediate_size": size, "activation": self.unit, "names": names}, env)
         self.plain = (self.score == 0 and self.weight_on == "input" and not self.identity and self.shared is None
-                      and not self.has_bias)
+                      and not self.has_bias and self.unit == "gated")
         # the sum over a token's experts may be left to whoever reads it, where it is nothing but that
         self.leaves_pairs = self.weight_on == "output" and not self.identity and self.shared is None
+        self.leaves_shared_pairs = self.weight_on == "output" and not self.identity and not self.shared_gate
+        self.kinds = ("gate", "up") if self.unit == "gated" else ("up",)
 
     def _name(self, i: int, what: str) -> str:
         return f"{self.names['expert'].format(i=i)}.{self.names[what]}"
@@ -100,10 +113,11 @@ class RoutedExperts(Part):
             out[self.names["router_bias"]] = TensorSpec((self.n_outputs,), role="gain", init="normal")
         if self.shared is not None:
             out.update(self.shared.tensor_specs())
+        if self.shared_gate:
             out[self.names["shared_gate"]] = TensorSpec((1, self.hidden))
         for i in range(self.n_experts):
-            out[self._name(i, "gate")] = TensorSpec((self.ff, self.hidden))
-            out[self._name(i, "up")] = TensorSpec((self.ff, self.hidden))
+            for what in self.kinds:
+                out[self._name(i, what)] = TensorSpec((self.ff, self.hidden))
             out[self._name(i, "down")] = TensorSpec((self.hidden, self.ff))
         return out
 
@@ -111,8 +125,9 @@ class RoutedExperts(Part):
         lib, allowed = self.env.lib, not getattr(self.env, "generic_only", False)
         r = tensors[self.names["router"]]
         pieces = [(r, 0, None, None)]
-        if self.shared is not None:          # the shared expert's gate is one more row of the router's product
+        if self.shared_gate:                 # the shared expert's gate is one more row of the router's product
             pieces.append((tensors[self.names["shared_gate"]].reshape(1, self.hidden), r.shape[0], None, None))
+        if self.shared is not None:
             self.shared.load({name: tensors[name] for name in self.shared.tensor_specs()})
         rows = r.shape[0] + len(pieces) - 1
         self.w_router = pack_rows(lib, pieces, rows, r.shape[1], r.dtype, r.device, allowed)
@@ -129,10 +144,11 @@ class RoutedExperts(Part):
                 lib.place_rows(tensors[self._name(i, what)].contiguous(), out[i], frag=self.frag)
             return out
 
-        self.w_gate, self.w_up, self.w_down = stack("gate"), stack("up"), stack("down")
+        self.w_gate = stack("gate") if self.unit == "gated" else None
+        self.w_up, self.w_down = stack("up"), stack("down")
 
     def forward(self, h: torch.Tensor, ctx=None, stream: Optional[torch.Tensor] = None, next_norm=None, pairs: bool = False):
-        """-> float32 [T, E], or, with pairs=True (where `leaves_pairs`), the `ExpertPairs` of the step."""
+        """-> float32 [T, E], or, with pairs=True (where `leaves_pairs` or `leaves_shared_pairs`), the `ExpertPairs` of the step."""
         lib, t, dev = self.env.lib, h.shape[0], h.device
         z = linear(lib, h, self.w_router, torch.float32)
         n_pairs = t * self.top
@@ -151,13 +167,13 @@ class RoutedExperts(Part):
         lib.routed_experts(h, weight if self.weight_on == "input" else None, self.top, row_pair, tile_expert, self.w_gate,
                            self.w_up, self.w_down, y, out, self.limit or 0.0, self.alpha, w_frag=self.frag)
         if pairs:
-            if not self.leaves_pairs:
+            if not (self.leaves_pairs or self.leaves_shared_pairs):
                 raise ConfigError("routed experts: only a plain weighted sum of the experts' outputs can be left to its reader")
-            return ExpertPairs(out, weight)
+            return ExpertPairs(out, weight, None if self.shared is None else self.shared.forward(h, ctx))
         if self.weight_on == "output":
             total = torch.empty((t, self.hidden), dtype=torch.float32, device=dev)
             both = None if self.shared is None else self.shared.forward(h, ctx)
-            lib.experts_combine(out, sel, weight, self.top, self.n_experts, h, both, z if both is not None else None,
+            lib.experts_combine(out, sel, weight, self.top, self.n_experts, h, both, z if self.shared_gate else None,
                                 self.n_outputs, total)
             return total
         if self.top == 1:

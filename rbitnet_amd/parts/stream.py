@@ -13,7 +13,8 @@ prepared for the norm that follows, `GainedRows`).  What a sublayer has not yet 
     tensor [P,T,E]  P terms, the K slices of a product, to be added up in their order
     GainedRows      nothing to add, and the rows as the next norm's kernel would read them
     StreamsUpdate   (a stream kept in several copies [S, T, E]) the update of all copies by a sublayer's result that
-                    is still to be done; a norm that reads such a stream does it in its own pass over the rows
+                    is still to be done; a norm that reads such a stream does it in its own pass over the rows.  The result may
+                    be terms [P, T, E] or `ExpertPairs` where that norm says `adds_update_terms`
     ScaledSum       scale * (a + b) still to be added: the two sublayers of a layer whose mixer and feed-forward read
                     the same norm, and the layer's residual factor; a norm that says `adds_scaled_sum` takes it as delta
     StreamCopy      nothing to add, and the stream's rows as they are in the compute dtype: what the sublayers of a layer
@@ -34,8 +35,11 @@ returns plain tensors, a norm without any does every sum and every normalisation
     part.takes_gained_rows    forward's input may be GainedRows instead of a tensor
     norm.adds_terms           forward's delta may be [P, T, E]
     norm.adds_normed_terms    forward's delta may be a NormedTerm whose norm is of the same kind
+    norm.reads_copies         forward takes a stream in several copies [S, T, E] with coef, and a StreamsUpdate as delta
+    norm.adds_update_terms    that update's result may be terms [P, T, E] or `ExpertPairs` (with a shared expert's output)
     part.leaves_terms         forward takes next_norm (stream None) and may return [P, T, E] to one that `adds_terms`
     part.leaves_pairs         forward takes pairs=True and then returns `ExpertPairs`
+    part.leaves_shared_pairs  the same, and the pairs may come with a shared expert's output
     norm.folds_into_products  the norm is x * weight / sqrt(mean x^2 + eps) with `weight`, `eps`
                               and `size`, so that products may do its work (GainedRows)
     block.takes_next_norm     forward takes next_norm: the first norm of whatever runs after it
@@ -93,7 +97,15 @@ class StreamsUpdate:
     def parts(self):
         return self.mix, self.out_coef, self.y, self.scale
 
+    def term_parts(self):
+        """(mix, out_coef, y, weights, extra) for a norm that adds up the result's terms itself."""
+        if isinstance(self.y, ExpertPairs):
+            return self.mix, self.out_coef, self.y.outputs, self.y.weights, self.y.shared
+        return self.mix, self.out_coef, self.y, None, None
+
     def apply(self, x: torch.Tensor) -> None:
+        if not isinstance(self.y, torch.Tensor) or self.y.dim() != 2:
+            raise ValueError("an update whose result is still terms is for a norm that adds them up")
         self.lib.streams_update(x, self.mix, self.out_coef, self.y, self.scale)
 
 
@@ -123,10 +135,10 @@ class WeightedTerms:
 
 class ExpertPairs:
     """The outputs [T * top, E] of every token's chosen experts and their weights [T * top]: the sum over a token's experts,
-    weight times output, is still to be done."""
+    weight times output, is still to be done.  shared (or None): [T, E] or terms [P, T, E] to be added to that sum."""
 
-    def __init__(self, outputs: torch.Tensor, weights: torch.Tensor):
-        self.outputs, self.weights = outputs, weights
+    def __init__(self, outputs: torch.Tensor, weights: torch.Tensor, shared: Optional[torch.Tensor] = None):
+        self.outputs, self.weights, self.shared = outputs, weights, shared
 
 
 class NormedTerm:
