@@ -416,9 +416,32 @@ def lilevik_config(width: int, layers: int, heads: int, kv_heads: int, ff: int, 
     return {"architecture": "Lilevik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "layers": out}
 
 
+def goperax_config(width: int, layers: int, heads: int, kv_heads: int, ff: int, vocab: int, experts: int = 16, top: int = 4,
+                   window: int = 1024, head: int = 64, streams: int = 4, state: int = 128, groups: int = 8) -> dict:
+    """Groups of four layers on a stream in `streams` copies: three state-space mixers (heads of 64, twice the width together, a
+    state of `state` rows, `groups` groups) and windowed attention whose values are its keys; the first layer has a dense
+    feed-forward, the others routed experts whose `top` chosen ones are together as wide, beside a shared one of an eighth of it."""
+    scan = {"heads": width * 2 // 64, "vdim": 64, "state": state, "groups": groups, "conv": 4, "norm_groups": groups}
+    soft = {"heads": heads, "kv_heads": kv_heads, "dim": head, "vdim": head, "scale": head ** -0.5, "softcap": 30.0, "mask": {"size": window}}
+    moe = {"kind": "moe", "expert": {"ff": ff // top}, "router": {"experts": experts, "top": top}, "shared": {"ff": ff // 8}}
+    out = []
+    for i in range(layers):
+        kind, mixer = ("attention", soft) if i % 4 == 3 else ("mamba2", scan)
+        out.append({"type": kind, "mixer": dict(mixer), "mlp": {"kind": "dense", "ff": ff} if i == 0 else moe})
+    return {"architecture": "Goperax", "vocab": vocab, "width": width, "streams": streams, "embedding": {"scale": 8.0},
+            "norm": {"eps": 1e-5}, "layers": out}
+
+
 # size -> (the design's configuration, then the shapes beside it: the Llama shape of equal width, depth and feed-forward
 # width, and for Pulunex the Tigutar model of those sizes too, whose routed experts and attention kernels are the like ones)
 DESIGN_SIZES = {
+    # Goperax beside the Lilevik model (linear attention in chunks, routed experts), the Bagonex model (a stream in several copies, a
+    # recurrence with convolutions) and the Llama shape of those sizes
+    "goperax_w1024": (goperax_config(1024, 12, 16, 4, 4096, 32000), lilevik_config(1024, 12, 16, 4, 4096, 32000),
+                      bagonex_config(1024, 12, 8, 64, 4096, 384, 64, 32000, low_rank=64), _other(1024, 4096, 16, 4, 64, 12, vocab=32000)),
+    "goperax_w2048": (goperax_config(2048, 16, 32, 8, 8192, 128256), lilevik_config(2048, 16, 32, 8, 8192, 128256),
+                      bagonex_config(2048, 16, 16, 128, 8192, 768, 128, 128256), _other(2048, 8192, 32, 8, 64, 16)),
+    "goperax_w4096": (goperax_config(4096, 8, 32, 8, 14336, 128256, head=128), dict(LLAMA3_8B, num_hidden_layers=8)),
     # Lilevik beside the Tigutar model (routed experts, a linear recurrence), the Menerax model (latents, heads prepared in front
     # of attention, norms on the outputs) and the Llama shape of those sizes
     "lilevik_w1024": (lilevik_config(1024, 12, 16, 4, 4096, 32000), tigutar_config(1024, 12, 16, 4, 4096, 32000, experts=16),
@@ -557,7 +580,7 @@ def main(argv=None) -> int:
                     help="no benchmark line: the named shape's decode products of 8 tokens beside a kernel that only "
                          "reads as many bytes")
     ap.add_argument("--design", default="", metavar="SIZE",
-                    help=f"no benchmark line: a Bagonex, Tigutar, Pulunex, Menerax or Lilevik model of this size ({', '.join(sorted(DESIGN_SIZES))}) beside the Llama "
+                    help=f"no benchmark line: a Bagonex, Tigutar, Pulunex, Menerax, Lilevik or Goperax model of this size ({', '.join(sorted(DESIGN_SIZES))}) beside the Llama "
                          "shape of equal width, depth and feed-forward width (some beside other designs too): prefill and decode throughput, and the time per kernel")
     ap.add_argument("--tokens", default="1,8,64,512,2048", help="token counts of --planner-sweep")
     ap.add_argument("--sweep-detail", default=None, help="--planner-sweep: a file for every candidate's time")

@@ -237,6 +237,16 @@ int rb_selective_scan(const float* q, const float* k, long long qk_stride, const
                       long long dt_stride, const float* dt_bias, const float* a_log, const float* d, float* state,
                       const int32_t* cu_seqlens, const int32_t* slots, float* out, int n_seqs, int n_tokens, int n_heads, int n_groups,
                       int dim, int vdim, void* stream);
+// The same for steps of many tokens a sequence, in chunks of 128 tokens on the matrix cores, for states of dim x vdim numbers a head that
+// are multiples of 8 up to 256 and 128 (rb_selective_chunks_ok).  q, k, x bfloat16 with rows `stride` apart; scratch:
+// rb_selective_chunks_floats float32 numbers.
+int rb_selective_chunks_ok(int dim, int vdim);
+int rb_selective_chunks_most(int n_tokens, int n_seqs);        // the most chunks that the step's tokens can fill
+long long rb_selective_chunks_floats(int n_tokens, int n_seqs, int n_heads, int dim, int vdim);
+int rb_selective_chunks(const void* q, const void* k, const void* x, long long stride, const float* dt_in, long long dt_stride,
+                        const float* dt_bias, const float* a_log, const float* d, float* state, const int32_t* cu_seqlens,
+                        const int32_t* slots, float* scratch, float* out, int n_seqs, int n_tokens, int n_heads, int n_groups, int dim,
+                        int vdim, void* stream);
 // The gate in front of the norm, the row in `parts` equal parts with a norm each: g = o * silu(gate[t * gate_stride + :]);
 // out[part] = g[part] / sqrt(mean(g[part]^2) + eps) * weight[part]; o [T, width], weight [width].
 int rb_gate_rmsnorm_parts(const float* o, const float* weight, const float* gate, long long gate_stride, float eps, void* out,

@@ -105,7 +105,7 @@ class KernelTimes:
         return "\n".join(lines)
 
 
-TIMED_OPS = ("embed_streams_waves", "streams_rmsnorm", "selective_scan", "gate_rmsnorm_parts", "tanh_norm", "heads_prepare", "lightning_recurrence", "lightning_chunks", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
+TIMED_OPS = ("selective_chunks", "embed_streams_waves", "streams_rmsnorm", "selective_scan", "gate_rmsnorm_parts", "tanh_norm", "heads_prepare", "lightning_recurrence", "lightning_chunks", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
              "route_top", "routed_experts", "pairs_sum", "embed_streams", "streams_layernorm", "streams_update", "xielu", "tanh_cap", "short_conv",
              "delta_prep", "delta_rule", "gated_rmsnorm", "latent_norm_store", "heads_linear", "attention_sinks", "embed_gather", "add_rmsnorm", "rope_kv_write", "swiglu", "gemm_generic", "gemm_bf16", "gemm_bf16_terms",
              "gemm_bf16_few", "attention_generic", "attention_prefill_bf16", "attention_decode_bf16",
@@ -165,6 +165,8 @@ class Kernels:
             "rb_streams_rmsnorm": [_P, _I, _L, _P, _P, _P, _I, _L, _L, _P, _P, _I, _L, _P, _P, _F, _P, _I, _I, _P, _I, _P],
             "rb_short_conv_biases": [_P, _L, _P, _P, _P, _I, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _P],
             "rb_selective_scan": [_P, _P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
+            "rb_selective_chunks_ok": [_I, _I],
+            "rb_selective_chunks": [_P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
             "rb_gate_rmsnorm_parts": [_P, _P, _P, _L, _F, _P, _I, _I, _I, _I, _P],
             "rb_xielu": [_P, _P, _P, _I, _L, _P],
             "rb_tanh_cap": [_P, _F, _L, _P],
@@ -227,6 +229,8 @@ class Kernels:
         L.rb_plan_calls.argtypes, L.rb_plan_calls.restype = [_P], _I
         L.rb_plan_replay.argtypes, L.rb_plan_replay.restype = [_P, _P], _I
         L.rb_plan_free.argtypes, L.rb_plan_free.restype = [_P], None
+        L.rb_selective_chunks_floats.argtypes = [_I, _I, _I, _I, _I]
+        L.rb_selective_chunks_floats.restype = ctypes.c_longlong
         L.rb_gemm_workspace_floats.argtypes = [_I, _I, _I, _I]
         L.rb_gemm_workspace_floats.restype = ctypes.c_longlong
         L.rb_sample_workspace_bytes.argtypes = [_I, _I]
@@ -1548,6 +1552,24 @@ class Kernels:
         self._ok(self._lib.rb_selective_scan(k + 4 * n_groups * dim, k, width, base, width, dt_in.data_ptr() + 4 * dt_col, dt_in.shape[1],
                                              _ptr(dt_bias), _ptr(a_log), _ptr(d), _ptr(state), _ptr(ctx.cu_seqlens), _ptr(ctx.slots),
                                              _ptr(out), ctx.n_seqs, n, n_heads, n_groups, dim, vdim, self._stream()))
+
+    def selective_chunks_ok(self, dim: int, vdim: int) -> bool:
+        """Whether `selective_chunks` takes states of these sizes."""
+        return bool(self._lib.rb_selective_chunks_ok(int(dim), int(vdim)))
+
+    def selective_chunks(self, xkq: torch.Tensor, dim: int, n_groups: int, n_heads: int, vdim: int, dt_in: torch.Tensor, dt_col: int,
+                         dt_bias: torch.Tensor, a_log: torch.Tensor, d: torch.Tensor, state: torch.Tensor, ctx, out: torch.Tensor) -> None:
+        """`selective_scan` in chunks of 128 tokens on the matrix cores; xkq bfloat16."""
+        _check(xkq, "xkq", torch.bfloat16)
+        self._scan_operands("selective_chunks", xkq, dim, n_groups, n_heads, vdim, dt_in, dt_col, dt_bias, a_log, d, state, ctx, out)
+        n, width = xkq.shape
+        base = xkq.data_ptr()
+        k = base + 2 * n_heads * vdim
+        scratch = torch.empty(int(self._lib.rb_selective_chunks_floats(n, ctx.n_seqs, n_heads, dim, vdim)), dtype=torch.float32,
+                              device=xkq.device)
+        self._ok(self._lib.rb_selective_chunks(k + 2 * n_groups * dim, k, base, width, dt_in.data_ptr() + 4 * dt_col, dt_in.shape[1],
+                                               _ptr(dt_bias), _ptr(a_log), _ptr(d), _ptr(state), _ptr(ctx.cu_seqlens), _ptr(ctx.slots),
+                                               _ptr(scratch), _ptr(out), ctx.n_seqs, n, n_heads, n_groups, dim, vdim, self._stream()))
 
     def gate_rmsnorm_parts(self, o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, gate_col: int, parts: int, eps: float,
                            out: torch.Tensor) -> None:

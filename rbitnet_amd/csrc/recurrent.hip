@@ -107,6 +107,109 @@ __global__ void short_conv_kernel(const float* __restrict__ x, size_t x_stride, 
   }
 }
 
+// The same for four channels a thread (16-byte loads) and few taps (KEEP = taps - 1 of them before the current one), so that no
+// predicate stands at a tap.
+template <int KEEP>
+__device__ __forceinline__ void conv4(float (&win)[KEEP][4], const float (&wt)[KEEP][4], const float (&w_cur)[4], const float4& now,
+                                      const float (&bo)[4], int residual, int act, float (&acc)[4]) {
+  const float cur[4] = {now.x, now.y, now.z, now.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    float a = fmaf(w_cur[i], cur[i], residual ? cur[i] : bo[i]);
+#pragma unroll
+    for (int j = 0; j < KEEP; ++j) a = fmaf(wt[j][i], win[j][i], a);
+#pragma unroll
+    for (int j = 0; j + 1 < KEEP; ++j) win[j][i] = win[j + 1][i];
+    win[KEEP - 1][i] = cur[i];
+    acc[i] = act == 1 ? a * rb_sigmoid(a) : a;
+  }
+}
+__device__ __forceinline__ void conv_store4(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+__device__ __forceinline__ void conv_store4(bf16_t* p, const float (&v)[4]) {
+  *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
+}
+template <typename TO, int KEEP>
+__global__ __launch_bounds__(256) void short_conv_vec_kernel(const float* __restrict__ x, size_t x_stride, const float* __restrict__ bias,
+                                                             const float* __restrict__ bias_out, const float* __restrict__ w,
+                                                             float* __restrict__ state, const int32_t* __restrict__ tok_seq,
+                                                             const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ slots,
+                                                             TO* __restrict__ out, size_t out_stride, int residual, int act, int channels,
+                                                             int n_tokens, int n_tiles) {
+  const int c = 4 * (blockIdx.y * blockDim.x + threadIdx.x);
+  if (c >= channels) return;
+  float wt[KEEP][4], w_cur[4], bc[4], bo[4], win[KEEP][4], acc[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+#pragma unroll
+    for (int j = 0; j < KEEP; ++j) wt[j][i] = w[(size_t)(c + i) * (KEEP + 1) + j];
+    w_cur[i] = w[(size_t)(c + i) * (KEEP + 1) + KEEP];
+    bc[i] = bias ? bias[c + i] : 0.f;
+    bo[i] = bias_out ? bias_out[c + i] : 0.f;
+  }
+  auto row = [&](size_t t) {
+    float4 v = *reinterpret_cast<const float4*>(x + t * x_stride + c);
+    return make_float4(v.x + bc[0], v.y + bc[1], v.z + bc[2], v.w + bc[3]);
+  };
+  auto put = [&](int j, const float4& v) {
+    win[j][0] = v.x, win[j][1] = v.y, win[j][2] = v.z, win[j][3] = v.w;
+  };
+  if ((int)blockIdx.x < n_tiles) {
+    const int r0 = blockIdx.x * SC_TILE, r1 = r0 + SC_TILE < n_tokens ? r0 + SC_TILE : n_tokens;
+    if (tok_seq[r0] == tok_seq[r1 - 1] && r1 - r0 == SC_TILE && r0 - cu_seqlens[tok_seq[r0]] >= KEEP) {
+      // a whole tile inside one sequence's piece: all its rows are asked for together
+      float4 rows[SC_TILE];
+#pragma unroll
+      for (int j = 0; j < KEEP; ++j) put(j, row((size_t)(r0 - KEEP + j)));
+#pragma unroll
+      for (int t = 0; t < SC_TILE; ++t) rows[t] = row((size_t)(r0 + t));
+#pragma unroll
+      for (int t = 0; t < SC_TILE; ++t) {
+        conv4<KEEP>(win, wt, w_cur, rows[t], bo, residual, act, acc);
+        conv_store4(out + (size_t)(r0 + t) * out_stride + c, acc);
+      }
+      return;
+    }
+    bool have = false;
+    for (int t = r0; t < r1; ++t) {
+      if (t - cu_seqlens[tok_seq[t]] < KEEP) {               // the sequence's workgroup takes it
+        have = false;
+        continue;
+      }
+      if (!have) {
+#pragma unroll
+        for (int j = 0; j < KEEP; ++j) put(j, row((size_t)(t - KEEP + j)));
+        have = true;
+      }
+      conv4<KEEP>(win, wt, w_cur, row((size_t)t), bo, residual, act, acc);
+      conv_store4(out + (size_t)t * out_stride + c, acc);
+    }
+    return;
+  }
+  const int b = blockIdx.x - n_tiles;
+  const int row0 = cu_seqlens[b], n = cu_seqlens[b + 1] - row0;
+  float* st = state + (size_t)slots[b] * KEEP * channels + c;
+  const int first = n < KEEP ? n : KEEP;
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j) put(j, *reinterpret_cast<const float4*>(st + (size_t)j * channels));
+  float4 rows[KEEP];
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i)
+    if (i < first) rows[i] = row((size_t)(row0 + i));
+  __builtin_amdgcn_sched_barrier(0);                         // state, weights and rows: one trip to memory together
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i)
+    if (i < first) {
+      conv4<KEEP>(win, wt, w_cur, rows[i], bo, residual, act, acc);
+      conv_store4(out + (size_t)(row0 + i) * out_stride + c, acc);
+    }
+  if (n <= 0) return;
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j) {
+    const float4 v = n > KEEP ? row((size_t)(row0 + n - KEEP + j)) : make_float4(win[j][0], win[j][1], win[j][2], win[j][3]);
+    *reinterpret_cast<float4*>(st + (size_t)j * channels) = v;
+  }
+}
+
 extern "C" int rb_short_conv(const float* x, long long x_stride, const float* w, int taps, float* state,
                              const int32_t* tok_pos, const int32_t* tok_seq, const int32_t* cu_seqlens,
                              const int32_t* slots, void* out, long long out_stride, int out_dtype, int residual,
@@ -145,6 +248,30 @@ extern "C" int rb_short_conv_biases(const float* x, long long x_stride, const fl
   RB_REQUIRE(act == 0 || act == 1, "rb_short_conv: unknown activation %d", act);
   if (n_tokens == 0) return 0;
   const int n_tiles = (n_tokens + SC_TILE - 1) / SC_TILE;
+  auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (taps >= 2 && taps <= 4 && channels % 4 == 0 && x_stride % 4 == 0 && out_stride % 4 == 0 && aligned(x) && aligned(state) && aligned(out) &&
+      (out_dtype == RB_F32 || out_dtype == RB_BF16)) {
+    const int threads = n_tokens <= n_seqs ? RB_WAVE : 256;   // single tokens: few workgroups, so small ones
+    const dim3 vgrid((n_tokens <= n_seqs ? 0 : n_tiles) + n_seqs, (channels / 4 + threads - 1) / threads);
+    const int vtiles = n_tokens <= n_seqs ? 0 : n_tiles;
+    RB_REQUIRE(vgrid.y <= 65535, "rb_short_conv: %d channels are too many", channels);
+#define SC_GO(TO, KEEP)                                                                                                            \
+  short_conv_vec_kernel<TO, KEEP><<<vgrid, threads, 0, (hipStream_t)stream>>>(x, (size_t)x_stride, bias, bias_out, w, state, tok_seq,  \
+                                                                              cu_seqlens, slots, (TO*)out, (size_t)out_stride, residual, \
+                                                                              act, channels, n_tokens, vtiles)
+#define SC_BY_TAPS(TO)                \
+  do {                                \
+    if (taps == 2) SC_GO(TO, 1);      \
+    else if (taps == 3) SC_GO(TO, 2); \
+    else SC_GO(TO, 3);                \
+  } while (0)
+    if (out_dtype == RB_F32) SC_BY_TAPS(float);
+    else SC_BY_TAPS(bf16_t);
+#undef SC_BY_TAPS
+#undef SC_GO
+    RB_LAUNCH_CHECK();
+    return 0;
+  }
   dim3 grid(n_tiles + (taps > 1 ? n_seqs : 0), (channels + 255) / 256 < 64 ? (channels + 255) / 256 : 64);
   hipStream_t s = (hipStream_t)stream;
   if (out_dtype == RB_F32)

@@ -10,7 +10,9 @@ Per token, with h the mixer's input, heads x vdim = inner and `groups` groups of
     y <- y * silu(z), each of `norm_groups` equal parts of it divided by its root mean square, times norm [inner];  out = Wo y
 (k, q and t are often written B, C and dt.)
 
-In float32: everything from the step sizes on, the recurrence, the gate and the norm.  The state lives in the cache's
+In float32: everything from the step sizes on, the recurrence, the gate and the norm.  Steps of many tokens a sequence run in
+chunks on the matrix cores where the compute dtype is bfloat16 (the convolution then leaves bfloat16 numbers, which is what the
+products take), steps of few tokens, float32 and other sizes one token after another.  The state lives in the cache's
 per-slot storage (`view.states["scan"]`, [slots, heads, vdim, state], column by column), the convolution's last taps - 1 inputs
 beside it (`view.states["conv"]`).
 
@@ -28,6 +30,7 @@ from .linear import linear, linear_to_stream, pack_rows
 from .short_conv import ACT_SILU, ShortConv
 
 MAX_STATE = 512
+CHUNKS_FROM = 24           # tokens of a step's longest piece from which chunks are worth their launches
 
 
 class StateSpace(Part):
@@ -55,6 +58,8 @@ class StateSpace(Part):
         self.dt_col = self.inner + self.channels
         self.conv = ShortConv(self.channels, int(params["conv"]), env, residual=False, act=ACT_SILU)
         self.cache_from = None
+        self.in_chunks = bool(env.dtype == torch.bfloat16 and env.lib is not None and not getattr(env, "generic_only", False)
+                              and env.lib.selective_chunks_ok(self.state, self.vdim))
 
     # ------------------------------------------------------------------ tensors
     def tensor_specs(self) -> Dict[str, TensorSpec]:
@@ -93,10 +98,13 @@ class StateSpace(Part):
     def forward(self, h: torch.Tensor, ctx, view, stream: Optional[torch.Tensor] = None, next_norm=None) -> torch.Tensor:
         lib, t = self.env.lib, h.shape[0]
         proj = linear(lib, h, self.w_in, torch.float32)                       # [T, z | x | k | q | t]
-        xkq = self.conv.forward(proj, ctx, view.states.get("conv"), torch.float32, col0=self.inner, bias_out=self.conv_bias)
+        chunks = self.in_chunks and ctx.max_q_len >= CHUNKS_FROM
+        xkq = self.conv.forward(proj, ctx, view.states.get("conv"), torch.bfloat16 if chunks else torch.float32, col0=self.inner,
+                                bias_out=self.conv_bias)
         y = torch.empty((t, self.inner), dtype=torch.float32, device=h.device)
-        lib.selective_scan(xkq, self.state, self.groups, self.heads, self.vdim, proj, self.dt_col, self.dt_bias, self.a_log, self.d,
-                           view.states["scan"], ctx, y)
+        scan = lib.selective_chunks if chunks else lib.selective_scan
+        scan(xkq, self.state, self.groups, self.heads, self.vdim, proj, self.dt_col, self.dt_bias, self.a_log, self.d,
+             view.states["scan"], ctx, y)
         yn = torch.empty((t, self.inner), dtype=self.env.dtype, device=h.device)
         lib.gate_rmsnorm_parts(y, self.norm, proj, 0, self.norm_groups, self.eps, yn)
         return linear_to_stream(lib, yn, self.w_o, None, next_norm)
