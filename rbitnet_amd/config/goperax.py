@@ -151,16 +151,18 @@ class GoperaxConfig:
     def to_spec(self) -> ModelSpec:
         def norm() -> PartSpec:
             return PartSpec("rmsnorm", {"size": self.width, "eps": self.norm_eps, "names": {"weight": ""}})
-        layers = []
+        layers, unused = [], []
         for i, layer in enumerate(self.layers):
             ff = self._feed_forward(layer.get("mlp"))
+            if ff is None:                # a file may hold them all the same
+                unused += [f"l{i}.norm2"] + [f"l{i}.hc2.{k}" for k in ("in", "out", "mix")]
             layers.append(LayerSpec(prefix=f"l{i}", block="hyper", mixer=self._mixer(layer["type"], layer["mixer"]), feed_forward=ff,
                                     norm1=norm(), norm2=None if ff is None else norm(),
                                     segments={"norm1": "norm1", "mixer": "mix", "norm2": "norm2", "feed_forward": "mlp"},
                                     params={"streams": self.streams, "scale": False}))
         return ModelSpec(
             architecture=self.architecture, hidden_size=self.width, vocab_size=self.vocab, max_positions=self.max_positions,
-            layers=layers, schedule=self.schedule(),
+            layers=layers, schedule=self.schedule(), optional_tensors=unused,
             embedding=PartSpec("table", {"name": "embed", "vocab_size": self.vocab, "streams": self.streams,
                                          "scale": self.embedding_scale, "waves": WAVE_BASE}),
             head=PartSpec("linear", {"norm": norm(), "norm_name": "final.norm", "name": None, "vocab_size": self.vocab}))

@@ -261,7 +261,7 @@ def random_goperax_tensors(cfg: Dict, seed: int) -> Dict[str, torch.Tensor]:
             t = (1.0 + 0.3 * rand(shape)) / shape[0]
         elif last == "out":
             t = 0.6 + 0.4 * rand(shape)
-        elif name.rsplit(".", 2)[-2].startswith("hc") and last == "mix":
+        elif last == "mix" and ".hc" in name:
             t = 0.8 * torch.eye(shape[0]) + 0.15 * rand(shape)
         elif last == "A_log":
             t = -1.5 + 1.2 * rand(shape)
@@ -276,8 +276,8 @@ def random_goperax_tensors(cfg: Dict, seed: int) -> Dict[str, torch.Tensor]:
         elif name == "embed":
             t = rand(shape) * 0.5
         elif ".mix.q" in name or ".mix.k" in name:
-            t = rand(shape) * (2.0 / math.sqrt(shape[-1]))
+            t = rand(shape) * (1.6 / math.sqrt(shape[-1]))
         else:
-            t = rand(shape) * (1.3 / math.sqrt(shape[-1]))
+            t = rand(shape) * (0.9 / math.sqrt(shape[-1]))
         out[name] = t.to(torch.bfloat16).to(F64)
     return out
