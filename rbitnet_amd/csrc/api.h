@@ -421,6 +421,16 @@ int rb_gated_rmsnorm_rows(const float* o, const float* weight, const float* gate
 int rb_route_choose_bias(const float* z, long long z_stride, const float* bias, int n_outputs, int n_experts, int top, int score,
                          const float* correction, int32_t* sel, float* weight, int32_t* row_pair, int32_t* tile_expert, int max_rows,
                          int n_tokens, void* stream);
+// The same with every expert's run padded to a multiple of `unit` rows instead of 16, row_pair and tile_expert counting tiles of so many.
+int rb_route_choose_units(const float* z, long long z_stride, const float* bias, int n_outputs, int n_experts, int top, int score,
+                          const float* correction, int32_t* sel, float* weight, int32_t* row_pair, int32_t* tile_expert, int max_rows,
+                          int unit, int n_tokens, void* stream);
+// Experts without gates for steps of many tokens, on the dense product's tiles (gemm_grouped.hip): out[p] = Wd act(Wu h[p / top]) for
+// pairs sorted in runs padded to `unit` rows (64, 128 or 256); experts' matrices fragment-major bfloat16 with sizes that are multiples
+// of 64; act float32 [2] as rb_xielu takes it; y [max_rows, ff] bfloat16 is scratch.
+int rb_routed_experts_tiled(const void* h, int n_tokens, int top, const int32_t* row_pair, const int32_t* tile_expert, int unit, int max_rows,
+                            const void* w_up, const void* w_down, const float* act, void* y, float* out, int n_experts, int width, int ff,
+                            void* stream);
 // rb_rope_store with every query and key head RMS-normed first over its dim numbers, x / sqrt(mean(x^2) + eps) * w, with a
 // weight of dim numbers that the heads share (q_norm, k_norm float32 [dim]).
 int rb_norm_rope_store(const float* qkv, long long row_width, const float* cos, const float* sin, int rot, const float* q_norm,

@@ -105,7 +105,7 @@ class KernelTimes:
         return "\n".join(lines)
 
 
-TIMED_OPS = ("selective_chunks", "embed_streams_waves", "streams_rmsnorm", "selective_scan", "gate_rmsnorm_parts", "tanh_norm", "heads_prepare", "lightning_recurrence", "lightning_chunks", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
+TIMED_OPS = ("routed_experts_tiled", "selective_chunks", "embed_streams_waves", "streams_rmsnorm", "selective_scan", "gate_rmsnorm_parts", "tanh_norm", "heads_prepare", "lightning_recurrence", "lightning_chunks", "gated_rmsnorm_rows", "short_conv_bias", "decay_exp_exp", "gated_rmsnorm_heads", "outnorm_residual", "clamped_glu", "tanh_cast", "attention_opts", "norm_rope_store", "sigmoid_gate", "shift_mix", "time_mix_recurrence", "latent_norm_rope_store", "heads_linear_part", "route_choose", "experts_combine", "embed_scaled_pos", "scale", "bias_norm_store", "attention_mixed", "attention_mixed_bf16", "recurrence_prep", "linear_recurrence", "layernorm_residual", "rope_store", "head_gate", "pair_norm_mean",
              "route_top", "routed_experts", "pairs_sum", "embed_streams", "streams_layernorm", "streams_update", "xielu", "tanh_cap", "short_conv",
              "delta_prep", "delta_rule", "gated_rmsnorm", "latent_norm_store", "heads_linear", "attention_sinks", "embed_gather", "add_rmsnorm", "rope_kv_write", "swiglu", "gemm_generic", "gemm_bf16", "gemm_bf16_terms",
              "gemm_bf16_few", "attention_generic", "attention_prefill_bf16", "attention_decode_bf16",
@@ -216,6 +216,8 @@ class Kernels:
             "rb_lightning_chunks_ok": [_I, _I],
             "rb_lightning_chunks": [_P, _P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P],
             "rb_gated_rmsnorm_rows": [_P, _P, _P, _L, _I, _F, _P, _I, _I, _I, _P],
+            "rb_route_choose_units": [_P, _L, _P, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _I, _P],
+            "rb_routed_experts_tiled": [_P, _I, _I, _P, _P, _I, _I, _P, _P, _P, _P, _P, _I, _I, _I, _P],
             "rb_route_choose_bias": [_P, _L, _P, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
             "rb_attention_mixed": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P, _I, _I, _P],
             "rb_attention_mixed_bf16": [_P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P, _I, _I, _I, _P, _P],
@@ -884,9 +886,9 @@ class Kernels:
 
     # ------------------------------------------------------------------ routed experts
     @staticmethod
-    def routed_rows(n_tokens: int, top: int, n_experts: int) -> int:
-        """Rows that the sorted pairs of a step may take: every expert's run is padded to 16."""
-        return (n_tokens * top + 15) // 16 * 16 + 16 * n_experts
+    def routed_rows(n_tokens: int, top: int, n_experts: int, unit: int = 16) -> int:
+        """Rows that the sorted pairs of a step may take: every expert's run is padded to `unit`."""
+        return (n_tokens * top + unit - 1) // unit * unit + unit * n_experts
 
     def route_top(self, z: torch.Tensor, n_experts: int, top: int, sel: torch.Tensor, weight: torch.Tensor,
                   row_pair: torch.Tensor, tile_expert: torch.Tensor) -> None:
@@ -934,16 +936,16 @@ class Kernels:
 
     def route_choose(self, z: torch.Tensor, n_outputs: int, n_experts: int, top: int, score: int,
                      correction: Optional[torch.Tensor], sel: torch.Tensor, weight: torch.Tensor, row_pair: torch.Tensor,
-                     tile_expert: torch.Tensor, bias: Optional[torch.Tensor] = None) -> None:
+                     tile_expert: torch.Tensor, bias: Optional[torch.Tensor] = None, unit: int = 16) -> None:
         """`route_top` with its choices spelled out: the router's first n_experts outputs are experts with matrices, the
         rest stand for the token's own input; score 0 sigmoid, 1 softmax over all outputs with `correction` [n_outputs]
-        added for the choice only, 2 softmax over the chosen logits alone; `bias` [n_outputs] is added to the logits first."""
+        added for the choice only, 2 softmax over the chosen logits alone; `bias` [n_outputs] is added to the logits first; runs are padded to `unit` rows."""
         n = z.shape[0]
         _check(z, "z", torch.float32)
         if z.shape[1] < n_outputs or n_experts > n_outputs:
             raise KernelError("route_choose: rows too short for the router's outputs")
         max_rows = row_pair.shape[0]
-        if max_rows < self.routed_rows(n, top, n_experts) or max_rows % 16:
+        if max_rows < self.routed_rows(n, top, n_experts, unit) or max_rows % unit:
             raise KernelError("route_choose: too little room for the sorted pairs")
         if correction is not None:
             _check(correction, "correction", torch.float32, (n_outputs,))
@@ -952,10 +954,30 @@ class Kernels:
         _check(sel, "sel", torch.int32, (n * top,))
         _check(weight, "weight", torch.float32, (n * top,))
         _check(row_pair, "row_pair", torch.int32, (max_rows,))
-        _check(tile_expert, "tile_expert", torch.int32, (2 * (max_rows // 16),))
-        self._ok(self._lib.rb_route_choose_bias(_ptr(z), z.shape[1], _ptr(bias), n_outputs, n_experts, top, int(score),
-                                                _ptr(correction), _ptr(sel), _ptr(weight), _ptr(row_pair), _ptr(tile_expert), max_rows,
-                                                n, self._stream()))
+        _check(tile_expert, "tile_expert", torch.int32, (2 * (max_rows // unit),))
+        self._ok(self._lib.rb_route_choose_units(_ptr(z), z.shape[1], _ptr(bias), n_outputs, n_experts, top, int(score),
+                                                 _ptr(correction), _ptr(sel), _ptr(weight), _ptr(row_pair), _ptr(tile_expert), max_rows,
+                                                 int(unit), n, self._stream()))
+
+    def routed_experts_tiled(self, h: torch.Tensor, top: int, row_pair: torch.Tensor, tile_expert: torch.Tensor, unit: int,
+                             w_up: torch.Tensor, w_down: torch.Tensor, act: torch.Tensor, y: torch.Tensor, out: torch.Tensor) -> None:
+        """Experts without gates on the dense product's tiles: out[p] = Wd act(Wu h[p // top]) for pairs sorted in runs padded to
+        `unit` rows (64, 128, 256); bfloat16, fragment-major experts; act float32 [2] as `xielu` takes it; y [rows, ff] is scratch."""
+        n, width = h.shape
+        n_experts, ff, _ = w_up.shape
+        max_rows = row_pair.shape[0]
+        _check(h, "h", torch.bfloat16)
+        _check(row_pair, "row_pair", torch.int32)
+        if unit not in (64, 128, 256) or max_rows % unit or max_rows < self.routed_rows(n, top, n_experts, unit):
+            raise KernelError(f"routed_experts_tiled: {max_rows} rows in runs padded to {unit}")
+        _check(tile_expert, "tile_expert", torch.int32, (2 * (max_rows // unit),))
+        _check(w_up, "w_up", torch.bfloat16, (n_experts, ff, width))
+        _check(w_down, "w_down", torch.bfloat16, (n_experts, width, ff))
+        _check(act, "act", torch.float32, (2,))
+        _check(y, "y", torch.bfloat16, (max_rows, ff))
+        _check(out, "out", torch.float32, (n * top, width))
+        self._ok(self._lib.rb_routed_experts_tiled(_ptr(h), n, top, _ptr(row_pair), _ptr(tile_expert), int(unit), max_rows, _ptr(w_up),
+                                                   _ptr(w_down), _ptr(act), _ptr(y), _ptr(out), n_experts, width, ff, self._stream()))
 
     def experts_combine(self, pairs: torch.Tensor, sel: torch.Tensor, weight: torch.Tensor, top: int, n_experts: int,
                         h: torch.Tensor, shared: Optional[torch.Tensor], gate: Optional[torch.Tensor], gate_col: int,

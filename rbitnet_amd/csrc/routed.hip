@@ -2,7 +2,7 @@
 //
 //   route:  scores s = sigmoid(z) of a token's router logits z [n_experts]; the `top` largest are chosen (among equals
 //           the lowest index); pair p = t * top + k holds the k-th choice of token t: sel[p] its expert, weight[p] its score.
-//   sort:   the pairs in the order of their experts, every expert's run padded to a multiple of 16 rows, so that a
+//   sort:   the pairs in the order of their experts, every expert's run padded to a multiple of 16 rows (or another unit), so that a
 //           tile of 16 rows belongs to one expert: row_pair[row] (-1: padding), tile_expert[row / 16] (-1: past the end),
 //           and behind the experts of all tiles their positions in their experts' runs (0, 1, 2, ...).
 //   up:     for every row, x = weight * h[token] (the weight multiplies the expert's INPUT), g = min(Wg x, limit),
@@ -122,27 +122,27 @@ __global__ void route_kernel(const float* __restrict__ z, size_t z_stride, int n
 
 // ---------------------------------------------------------------- sort (one workgroup)
 __device__ void route_sort(const int32_t* sel, int n_pairs, int n_experts, int32_t* __restrict__ row_pair,
-                           int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_pos, int max_rows) {
+                           int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_pos, int max_rows, int unit) {
   __shared__ int counts[RT_MAX_EXPERTS], offs[RT_MAX_EXPERTS], cursor[RT_MAX_EXPERTS];
   for (int e = threadIdx.x; e < n_experts; e += blockDim.x) counts[e] = cursor[e] = 0;
   __syncthreads();
   for (int p = threadIdx.x; p < n_pairs; p += blockDim.x)
     if (sel[p] < n_experts) atomicAdd(&counts[sel[p]], 1);      // an output behind the experts has no matrices and no run
   for (int r = threadIdx.x; r < max_rows; r += blockDim.x) row_pair[r] = -1;
-  for (int i = threadIdx.x; i < max_rows / RT_TILE; i += blockDim.x) tile_expert[i] = -1;
+  for (int i = threadIdx.x; i < max_rows / unit; i += blockDim.x) tile_expert[i] = -1;
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0;
     for (int e = 0; e < n_experts; ++e) {
       offs[e] = at;
-      at += (counts[e] + RT_TILE - 1) / RT_TILE * RT_TILE;
+      at += (counts[e] + unit - 1) / unit * unit;
     }
   }
   __syncthreads();
   for (int e = threadIdx.x; e < n_experts; e += blockDim.x)
-    for (int i = 0; i < (counts[e] + RT_TILE - 1) / RT_TILE; ++i) {
-      tile_expert[offs[e] / RT_TILE + i] = e;
-      tile_pos[offs[e] / RT_TILE + i] = i;                 // which tile of its expert's run
+    for (int i = 0; i < (counts[e] + unit - 1) / unit; ++i) {
+      tile_expert[offs[e] / unit + i] = e;
+      tile_pos[offs[e] / unit + i] = i;                 // which tile of its expert's run
     }
   for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) {
     const int e = sel[p];
@@ -152,8 +152,8 @@ __device__ void route_sort(const int32_t* sel, int n_pairs, int n_experts, int32
 
 __global__ __launch_bounds__(1024) void route_sort_kernel(const int32_t* __restrict__ sel, int n_pairs, int n_experts,
                                                           int32_t* __restrict__ row_pair, int32_t* __restrict__ tile_expert,
-                                                          int32_t* __restrict__ tile_pos, int max_rows) {
-  route_sort(sel, n_pairs, n_experts, row_pair, tile_expert, tile_pos, max_rows);
+                                                          int32_t* __restrict__ tile_pos, int max_rows, int unit) {
+  route_sort(sel, n_pairs, n_experts, row_pair, tile_expert, tile_pos, max_rows, unit);
 }
 
 // A step of few tokens: the choice (a wave a token) and the sort in one launch of one workgroup.
@@ -161,12 +161,13 @@ __global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict
                                                          int top, int score, const float* __restrict__ bias,
                                                          const float* __restrict__ correction, int32_t* sel,
                                                          float* __restrict__ weight, int n_tokens, int32_t* __restrict__ row_pair,
-                                                         int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_pos, int max_rows) {
+                                                         int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_pos, int max_rows,
+                                                         int unit) {
   for (int t = threadIdx.x / RB_WAVE; t < n_tokens; t += blockDim.x / RB_WAVE)
     route_token(z, z_stride, n_outputs, top, score, bias, correction, sel, weight, t);
   __threadfence_block();
   __syncthreads();
-  route_sort(sel, n_tokens * top, n_experts, row_pair, tile_expert, tile_pos, max_rows);
+  route_sort(sel, n_tokens * top, n_experts, row_pair, tile_expert, tile_pos, max_rows, unit);
 }
 
 extern "C" int rb_route_choose(const float* z, long long z_stride, int n_outputs, int n_experts, int top, int score,
@@ -180,8 +181,17 @@ extern "C" int rb_route_choose(const float* z, long long z_stride, int n_outputs
 extern "C" int rb_route_choose_bias(const float* z, long long z_stride, const float* bias, int n_outputs, int n_experts, int top,
                                     int score, const float* correction, int32_t* sel, float* weight, int32_t* row_pair,
                                     int32_t* tile_expert, int max_rows, int n_tokens, void* stream) {
-  RB_RECORDED(rb_route_choose_bias(z, z_stride, bias, n_outputs, n_experts, top, score, correction, sel, weight, row_pair, tile_expert,
-                                   max_rows, n_tokens, stream));
+  return rb_route_choose_units(z, z_stride, bias, n_outputs, n_experts, top, score, correction, sel, weight, row_pair, tile_expert, max_rows,
+                               RT_TILE, n_tokens, stream);
+}
+
+// The same with every expert's run padded to a multiple of `unit` rows, tiles being of that many rows.
+extern "C" int rb_route_choose_units(const float* z, long long z_stride, const float* bias, int n_outputs, int n_experts, int top,
+                                    int score, const float* correction, int32_t* sel, float* weight, int32_t* row_pair,
+                                    int32_t* tile_expert, int max_rows, int unit, int n_tokens, void* stream) {
+  RB_RECORDED(rb_route_choose_units(z, z_stride, bias, n_outputs, n_experts, top, score, correction, sel, weight, row_pair, tile_expert,
+                                    max_rows, unit, n_tokens, stream));
+  RB_REQUIRE(unit > 0, "rb_route_choose: runs padded to %d rows", unit);
   RB_REQUIRE(n_tokens >= 0 && n_experts >= 0 && n_outputs >= n_experts && n_outputs > 0 && n_outputs <= RT_MAX_EXPERTS && top > 0 &&
                  top <= n_outputs && z_stride >= n_outputs,
              "rb_route_choose: bad sizes T=%d outputs=%d (at most %d) experts=%d top=%d", n_tokens, n_outputs, RT_MAX_EXPERTS, n_experts, top);
@@ -189,18 +199,18 @@ extern "C" int rb_route_choose_bias(const float* z, long long z_stride, const fl
   RB_REQUIRE(score != 2 || top <= RB_WAVE, "rb_route_choose: the softmax over the chosen takes at most %d of them, not %d", RB_WAVE, top);
   RB_REQUIRE(correction == nullptr || score == 1, "rb_route_choose: a correction goes with the softmax");
   const long long pairs = (long long)n_tokens * top;
-  RB_REQUIRE(max_rows % RT_TILE == 0 && max_rows >= (pairs + RT_TILE - 1) / RT_TILE * RT_TILE + (long long)RT_TILE * n_experts,
+  RB_REQUIRE(max_rows % unit == 0 && max_rows >= (pairs + unit - 1) / unit * unit + (long long)unit * n_experts,
              "rb_route_choose: room for %d rows, %lld pairs of %d experts may need more", max_rows, pairs, n_experts);
   if (n_tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   if (n_tokens <= RT_FEW_TOKENS) {
     route_few_kernel<<<1, 1024, 0, s>>>(z, (size_t)z_stride, n_outputs, n_experts, top, score, bias, correction, sel, weight, n_tokens,
-                                        row_pair, tile_expert, tile_expert + max_rows / RT_TILE, max_rows);
+                                        row_pair, tile_expert, tile_expert + max_rows / unit, max_rows, unit);
     RB_LAUNCH_CHECK();
     return 0;
   }
   route_kernel<<<(n_tokens + 3) / 4, 256, 0, s>>>(z, (size_t)z_stride, n_outputs, top, score, bias, correction, sel, weight, n_tokens);
-  route_sort_kernel<<<1, 1024, 0, s>>>(sel, (int)pairs, n_experts, row_pair, tile_expert, tile_expert + max_rows / RT_TILE, max_rows);
+  route_sort_kernel<<<1, 1024, 0, s>>>(sel, (int)pairs, n_experts, row_pair, tile_expert, tile_expert + max_rows / unit, max_rows, unit);
   RB_LAUNCH_CHECK();
   return 0;
 }
@@ -451,6 +461,7 @@ __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t
                                                              const bf16_t* __restrict__ w_gate, const bf16_t* __restrict__ w_up,
                                                              bf16_t* __restrict__ y, int width, int ff, float limit, float alpha,
                                                              int n_tiles) {
+  constexpr int CB = GATED ? 2 : 4;                     // blocks of 16 channels a wave: its loads and products keep their proportion
   // blockIdx.x counts the channels, so that workgroups that follow one another share their rows of the step (which
   // then come from memory once) and walk through an expert's matrices together
   const int e = tile_expert[blockIdx.y];
@@ -460,24 +471,25 @@ __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t
   if (t0 >= n_tiles || tile_expert[t0] != e) return;
   int nt = 1;
   while (nt < RT_GROUP && t0 + nt < n_tiles && tile_expert[t0 + nt] == e) ++nt;
-  const int c0 = (blockIdx.x * 2 + (wave >> 2)) * 32;
+  const int c0 = (blockIdx.x * 2 + (wave >> 2)) * 16 * CB;
   if (c0 >= ff) return;
+  const int n_cb = (ff - c0) / 16 < CB ? (ff - c0) / 16 : CB;        // ff is a multiple of 32, not always of 64
   const int r = lane & 15, grp = lane >> 4;
   const bf16_t* xr = xs + (size_t)t0 * RT_TILE * width + 8 * lane;
   const bf16_t* gr = GATED ? w_gate + ((size_t)e * ff + c0) * width + 8 * lane : nullptr;
   const bf16_t* ur = w_up + ((size_t)e * ff + c0) * width + 8 * lane;
   const size_t blk = (size_t)16 * width;               // 16 rows further: the next block of channels, the next tile
-  f32x4_t ag[RT_GROUP][2], au[RT_GROUP][2];
+  f32x4_t ag[RT_GROUP][CB], au[RT_GROUP][CB];
 #pragma unroll
   for (int j = 0; j < RT_GROUP; ++j)
 #pragma unroll
-    for (int cb = 0; cb < 2; ++cb) ag[j][cb] = au[j][cb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int cb = 0; cb < CB; ++cb) ag[j][cb] = au[j][cb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   for (int k = 0; k < 16 * width; k += 512) {            // a block of 16 rows x 32 depth values further
-    Frag8 fg[2], fu[2], fx[RT_GROUP];
+    Frag8 fg[CB], fu[CB], fx[RT_GROUP];
 #pragma unroll
-    for (int cb = 0; cb < 2; ++cb) {
+    for (int cb = 0; cb < CB; ++cb) {
       if (GATED) fg[cb].u = load16(gr + cb * blk + k);
-      fu[cb].u = load16(ur + cb * blk + k);
+      fu[cb].u = cb < n_cb ? load16(ur + cb * blk + k) : zero16();
     }
 #pragma unroll
     for (int j = 0; j < RT_GROUP; ++j) fx[j].u = j < nt ? load16(xr + j * blk + k) : zero16();
@@ -485,7 +497,7 @@ __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t
     for (int j = 0; j < RT_GROUP; ++j) {
       if (j < nt) {
 #pragma unroll
-        for (int cb = 0; cb < 2; ++cb) {
+        for (int cb = 0; cb < CB; ++cb) {
           if (GATED) ag[j][cb] = mfma16(fg[cb], fx[j], ag[j][cb]);
           au[j][cb] = mfma16(fu[cb], fx[j], au[j][cb]);
         }
@@ -498,7 +510,8 @@ __global__ __launch_bounds__(RT_THREADS) void routed_up_mfma_kernel(const bf16_t
     const int row = (t0 + j) * RT_TILE + r;
     if (row_pair[row] < 0) continue;
 #pragma unroll
-    for (int cb = 0; cb < 2; ++cb) {
+    for (int cb = 0; cb < CB; ++cb) {
+      if (cb >= n_cb) break;
       // channel c of this row lies, fragment-major, in block c / 32 of the tile at 8 * (16 * (c % 32 / 8) + r) + c % 8
       const int c = c0 + 16 * cb + 4 * grp;
       bf16_t* dst = y + (size_t)(t0 + j) * RT_TILE * ff + (size_t)(c / 32) * 512 + 8 * (16 * ((c % 32) / 8) + r) + c % 8;
@@ -589,7 +602,7 @@ extern "C" int rb_routed_experts(const void* h, int dtype, const float* weight, 
     bf16_t* xs = (bf16_t*)y + (size_t)max_rows * ff;
     routed_gather_kernel<<<tiles, 256, 0, s>>>((const bf16_t*)h, weight, top, row_pair, tile_expert, xs, width);
     auto up = w_gate ? routed_up_mfma_kernel<true> : routed_up_mfma_kernel<false>;
-    up<<<dim3((ff + 63) / 64, tiles), RT_THREADS, 0, s>>>(xs, row_pair, tile_expert, tile_expert + tiles, (const bf16_t*)w_gate,
+    up<<<dim3(w_gate ? (ff + 63) / 64 : (ff + 127) / 128, tiles), RT_THREADS, 0, s>>>(xs, row_pair, tile_expert, tile_expert + tiles, (const bf16_t*)w_gate,
                                                           (const bf16_t*)w_up, (bf16_t*)y, width, ff, limit, alpha, tiles);
     routed_down_mfma_kernel<<<dim3((width + 127) / 128, tiles), RT_THREADS, 0, s>>>((const bf16_t*)y, row_pair, tile_expert,
                                                                              tile_expert + tiles, (const bf16_t*)w_down, out, width,

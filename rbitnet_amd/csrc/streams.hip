@@ -344,8 +344,13 @@ __global__ void embed_streams_waves_kernel(const T* __restrict__ table, const in
     const float a = fmaf(Num<T>::load(row + 2 * i), scale, sn);
     const bool two = 2 * i + 1 < width;
     const float b = two ? fmaf(Num<T>::load(row + 2 * i + 1), scale, cs) : 0.f;
+    const bool pair = two && width % 2 == 0 && stream_stride % 2 == 0 && (reinterpret_cast<uintptr_t>(x) & 7) == 0;
     for (int s = 0; s < n_streams; ++s) {
       float* xr = x + (size_t)s * stream_stride + (size_t)t * width + 2 * i;
+      if (pair) {
+        *reinterpret_cast<float2*>(xr) = make_float2(a, b);
+        continue;
+      }
       xr[0] = a;
       if (two) xr[1] = b;
     }

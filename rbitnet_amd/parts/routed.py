@@ -43,6 +43,14 @@ DEFAULT_NAMES = {"router": "router", "expert": "e{i}", "gate": "gate", "up": "up
                  "shared": "shared", "shared_gate": "shared.sg", "router_bias": "router.b"}
 MAX_EXPERTS = 1024
 MAX_CHOSEN = 64            # of the softmax over the chosen logits
+TILED_FROM = 65            # tokens of a step from which experts without gates run on the dense product's tiles
+
+
+def tile_rows(n_pairs: int, n_experts: int) -> int:
+    """How many rows every expert's run is padded to where it runs on the dense product's tiles: large tiles where the runs fill
+    them."""
+    each = n_pairs / n_experts
+    return 256 if each >= 1536 else 128 if each >= 112 else 64
 
 
 class RoutedExperts(Part):
@@ -144,6 +152,9 @@ class RoutedExperts(Part):
                 lib.place_rows(tensors[self._name(i, what)].contiguous(), out[i], frag=self.frag)
             return out
 
+        # without gates a step of many tokens runs on the dense product's tiles
+        self.tiled = bool(self.frag and self.unit == "squared_relu" and self.weight_on == "output" and self.hidden % 64 == 0 and self.ff % 64 == 0)
+        self.act = torch.tensor([float("nan"), 1.0], dtype=torch.float32, device=r.device) if self.tiled else None     # (see DenseAct)
         self.w_gate = stack("gate") if self.unit == "gated" else None
         self.w_up, self.w_down = stack("up"), stack("down")
 
@@ -152,20 +163,26 @@ class RoutedExperts(Part):
         lib, t, dev = self.env.lib, h.shape[0], h.device
         z = linear(lib, h, self.w_router, torch.float32)
         n_pairs = t * self.top
-        max_rows = lib.routed_rows(t, self.top, self.n_experts)
+        tiled = self.tiled and t >= TILED_FROM
+        unit = tile_rows(n_pairs, self.n_experts) if tiled else 16
+        max_rows = lib.routed_rows(t, self.top, self.n_experts, unit)
         sel = torch.empty(n_pairs, dtype=torch.int32, device=dev)
         weight = torch.empty(n_pairs, dtype=torch.float32, device=dev)
         row_pair = torch.empty(max_rows, dtype=torch.int32, device=dev)
-        tile_expert = torch.empty(2 * (max_rows // 16), dtype=torch.int32, device=dev)      # experts, then positions in their runs
+        tile_expert = torch.empty(2 * (max_rows // unit), dtype=torch.int32, device=dev)      # experts, then positions in their runs
         if self.plain:
             lib.route_top(z, self.n_experts, self.top, sel, weight, row_pair, tile_expert)
         else:
             lib.route_choose(z, self.n_outputs, self.n_experts, self.top, self.score, self.correction, sel, weight, row_pair,
-                             tile_expert, bias=self.bias)
-        y = torch.empty((max_rows, self.ff + self.hidden), dtype=h.dtype, device=dev)         # scratch: gated units, scaled inputs
+                             tile_expert, bias=self.bias, unit=unit)
         out = torch.empty((n_pairs, self.hidden), dtype=torch.float32, device=dev)
-        lib.routed_experts(h, weight if self.weight_on == "input" else None, self.top, row_pair, tile_expert, self.w_gate,
-                           self.w_up, self.w_down, y, out, self.limit or 0.0, self.alpha, w_frag=self.frag)
+        if tiled:
+            y = torch.empty((max_rows, self.ff), dtype=h.dtype, device=dev)
+            lib.routed_experts_tiled(h, self.top, row_pair, tile_expert, unit, self.w_up, self.w_down, self.act, y, out)
+        else:
+            y = torch.empty((max_rows, self.ff + self.hidden), dtype=h.dtype, device=dev)     # scratch: gated units, scaled inputs
+            lib.routed_experts(h, weight if self.weight_on == "input" else None, self.top, row_pair, tile_expert, self.w_gate,
+                               self.w_up, self.w_down, y, out, self.limit or 0.0, self.alpha, w_frag=self.frag)
         if pairs:
             if not (self.leaves_pairs or self.leaves_shared_pairs):
                 raise ConfigError("routed experts: only a plain weighted sum of the experts' outputs can be left to its reader")

@@ -525,6 +525,31 @@ def test_experts_without_gates_beside_a_shared_one(lib, dtype, hidden, ff, exper
             assert _rel(part.forward(_dev(x[:n], dtype)), total[:n].double().cpu()) < tol, n
 
 
+@pytest.mark.parametrize("hidden,ff,experts,top,t_len", [(128, 64, 6, 2, 300), (64, 192, 3, 3, 900), (192, 128, 130, 4, 70), (64, 64, 1, 1, 65),
+                                                         (256, 320, 5, 1, 700)])
+def test_experts_on_the_dense_products_tiles_give_what_the_routed_kernels_give(lib, hidden, ff, experts, top, t_len, monkeypatch):
+    """Runs padded to 64, 128 and 256 rows, some of them empty, with one expert that nearly every token chooses: bit for bit the
+    same pairs."""
+    from rbitnet_amd.parts import routed as R
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    part = build_part("feed_forward", GoperaxConfig._feed_forward(mlp), _env(lib, hidden, torch.bfloat16))
+    w = _weights("attention", hidden, ATTENTIONS[0], experts + ff, "mlp", mlp)
+    x = _bf(torch.randn(t_len, hidden, dtype=F64))
+    x[:, 0] = 3.0
+    w["router"][0, 0] = 3.0
+    part.load(_place(part, w, torch.bfloat16))
+    assert part.tiled
+    want, h = P.experts(x, w, mlp), _dev(x, torch.bfloat16)
+    part.tiled = False
+    plain = part.forward(h, pairs=True)
+    part.tiled = True
+    for unit in (64, 128, 256):
+        monkeypatch.setattr(R, "tile_rows", lambda pairs, n: unit)
+        got = part.forward(h, pairs=True)
+        assert torch.equal(got.outputs, plain.outputs) and torch.equal(got.weights, plain.weights), unit
+        assert _close(part.forward(h), want, torch.bfloat16), unit
+
+
 # ---------------------------------------------------------------------------- whole models
 def _moe(ff, experts, top, shared=None):
     out = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
